@@ -35,7 +35,8 @@ typedef enum {
     UZU_ACT_GELU_EXACT = 2,
     UZU_ACT_IDENTITY = 3,
     UZU_ACT_SOFTPLUS = 4,
-    UZU_ACT_RELU_SQUARED = 5 /* max(z, 0)^2: the plain (ungated) dense MLP of an f32-stream design (uzu_layer_desc::mlp_plain) */
+    UZU_ACT_RELU_SQUARED = 5, /* max(z, 0)^2: the plain (ungated) dense MLP of an f32-stream design (uzu_layer_desc::mlp_plain) */
+    UZU_ACT_XIELU = 6 /* the same block with softplus(p) z^2 + z / 2 (z > 0), (1 / 2 + softplus(q)) (e^z - 1 - z) + z / 2 (z <= 0): uzu_layer_desc::xielu_p / xielu_q */
 } uzu_activation_type;
 
 /*
@@ -175,9 +176,17 @@ typedef struct {
      * (routing == 0) reads router_biases (bf16 [E], optional), takes the num_active_experts largest logits (ties: the lower index) and, with router_renorm, the
      * softmax over the winners' logits as weights; the experts have no biases. */
     float up_offset;
+    uint32_t plain_experts;        /* f32-stream designs: an expert has no gate, W_down max(W_up h, 0)^2; w13 is [E, d_ff, model_dim] (the field was `reserved`) */
+    /* Grouped sigmoid routing (f32-stream designs; routing == UZU_MOE_ROUTE_SIGMOID_GROUPS): s = sigmoid of the router logits, choice scores = s + selection_bias.
+     * The experts form router_groups equal groups of neighbours (0 / 1: one group); a group's strength is the sum of its two largest choice scores, and only experts
+     * of the router_groups_keep strongest groups can be chosen.  The num_active_experts largest choice scores among them win (ties: the lower index); a winner's
+     * weight is its s divided by the winners' sum of s (+ 1e-20), times router_scale (0 = 1). */
+    uint32_t router_groups;
+    uint32_t router_groups_keep;
+    float router_scale;
     uint32_t reserved;
 } uzu_moe_desc;
-typedef enum { UZU_MOE_ROUTE_TOPK_LOGITS = 0, UZU_MOE_ROUTE_SCORES = 1 } uzu_moe_routing;
+typedef enum { UZU_MOE_ROUTE_TOPK_LOGITS = 0, UZU_MOE_ROUTE_SCORES = 1, UZU_MOE_ROUTE_SIGMOID_GROUPS = 2 } uzu_moe_routing;
 
 typedef enum { UZU_MLP_DENSE = 0, UZU_MLP_MOE = 1 } uzu_mlp_kind;
 
@@ -312,7 +321,7 @@ typedef struct {
     /* Re-entry of the stream: before this run x <- W [x ; x0] with x0 the embedding rows (n = model_dim, k = 2 model_dim); absent = none */
     uzu_linear_desc stream_reentry;
     /* Input convolution of the sublayers (f32-stream designs): what a sublayer reads is h + conv(h), h = its input rows (the stream itself where the pre norm is
-     * absent -- with an input convolution pre_mixer_norm / pre_mlp_norm may be absent), conv = a causal convolution over positions on every channel:
+     * absent, the normed rows otherwise), conv = a causal convolution over positions on every channel:
      * conv(h)_t = sum_j w[:, j] h_(t - taps + 1 + j), zeros in front of the sequence; input_conv_mixer / input_conv_mlp f32 [model_dim, input_conv_taps] (either
      * may be NULL = that sublayer reads h).  The last taps - 1 inputs of each are sequence state. */
     uint32_t input_conv_taps;
@@ -346,6 +355,19 @@ typedef struct {
     uint32_t dn_decay_rank, dn_gate_rank;
     uzu_linear_desc dn_decay_up; /* n = heads dk, k = dn_decay_rank */
     uzu_linear_desc dn_gate_up;  /* n = heads dv, k = dn_gate_rank */
+    /* UZU_MIXER_LATENT_ATTENTION with latent_packed whose QUERIES go through a latent of their own: qkv_projection's rows are query down (latent_query_rank) | down
+     * projection (latent_rank + latent_rope_dim) | gates; the query latent is RMS-normed with latent_query_norm and latent_query_up turns it into the heads' queries
+     * (n = num_heads (head_dim + latent_rope_dim), k = latent_query_rank).  0 = queries straight from the packed projection. */
+    uint32_t latent_query_rank;
+    uint32_t gate_elementwise; /* has_gate on latent attention: one gate per coordinate (num_heads value_head_dim rows): the concatenated heads times sigmoid(rows h) */
+    uzu_norm_desc latent_query_norm;
+    uzu_linear_desc latent_query_up;
+    /* mlp_plain with activation UZU_ACT_XIELU */
+    float xielu_p, xielu_q;
+    /* Hyper-connections (uzu_model_desc::hyper_streams = s > 0): how the sublayer reads and joins the s copies of the stream.  f32 [s | s | s s] = in, out, mix:
+     * u = sum_a in[a] x_a; y = sublayer(norm(u)); then, all from the old ones, x_b <- sum_a mix[a, b] x_a + residual_mult out[b] y. */
+    const float* hyper_mixer;
+    const float* hyper_mlp; /* NULL on a layer without an MLP */
 } uzu_layer_desc;
 
 typedef struct {
@@ -393,6 +415,10 @@ typedef struct {
     uint32_t bigram_buckets;
     uint32_t bigram_mul_prev, bigram_mul_cur;
     uzu_linear_desc bigram_table;
+    /* Hyper-connections (f32-stream designs): != 0: the residual stream is hyper_streams copies, all equal to the embedding rows at the start; every sublayer reads and
+     * joins them as its layer's hyper_mixer / hyper_mlp say, and the read-out sees their sum.  residual_mult multiplies a sublayer's result. */
+    uint32_t hyper_streams;
+    float residual_mult;
 } uzu_model_desc;
 
 /*

@@ -28,6 +28,10 @@
 // gate per head, causal chunks, values that are the key rows, a temperature per head and a learned bias per distance bucket; and a SECOND mixer beside the first in one
 // layer -- a gated delta rule with a decay per head and key channel (k_channel_delta.hip) -- whose result is summed with the first's through their own out projections.
 //
+// A fifth family (Dironex) adds: hyper-connections (the stream is several copies; one launch between two sublayers joins the first one's result, reads, norms and --
+// on one-row passes -- convolves the second one's row; k_hyper.hip), input convolutions BEHIND a pre norm, latent attention whose queries pass a normed latent of
+// their own and whose concatenated heads are gated coordinate by coordinate, a plain dense block with xIELU, and experts without a gate behind grouped sigmoid routing.
+//
 // Precisions: `bf16_products` (default) rounds the activation operand of every matrix product to bf16 and keeps the latent cache in bf16; UZU_MODEL_FULL_F32
 // makes every product a true f32 product and the cache f32.  Everything else is f32 either way.
 #include <algorithm>
@@ -51,6 +55,7 @@ struct Stream32 {
     float *tmp = nullptr, *y1 = nullptr, *lru_u = nullptr, *lru_g = nullptr, *side_g = nullptr; // a sublayer's result in front of its post norm; [up | gate] of a gated dense block; LRU input / gates; token-input gate
     float *moe_y1 = nullptr, *moe_y2 = nullptr; // grouped expert form: [max_rows * top][2 ff] and [max_rows * top][d]
     uint32_t *moe_perm = nullptr, *moe_slot_pos = nullptr, *moe_offsets = nullptr, *moe_cursor = nullptr;
+    float *hyper = nullptr, *conv_rows = nullptr, *lat_q = nullptr, *moe_z = nullptr; // copies of the stream [s][max_rows][d]; a normed row + its convolution; queries behind their latent; router logits
     float *out_normed = nullptr, *logits = nullptr;
     size_t logit_rows = 0;
     k::SeqSpan* d_spans = nullptr;
@@ -83,6 +88,10 @@ struct Stream32 {
         uint32_t dist_rows = 0;
         float* head_temp = nullptr;   // f32 [heads]
         DLinear decay_up, gate_up;    // the delta rule's low-rank second factors
+        DLinear lat_q_up;             // latent attention: the queries of their latent
+        DNorm lat_q_norm;
+        float act_a = 0.f, act_b = 0.f; // xIELU: softplus(p), 1 / 2 + softplus(q)
+        float *hyper_mixer = nullptr, *hyper_mlp = nullptr; // f32 [in | out | mix]
     };
     std::vector<Layer> layers;
     float alpha_out = 0.f;
@@ -165,7 +174,7 @@ k::ExpertAct expert_act(const uzu_moe_desc& M) {
     a.alpha = M.silu_alpha != 0.0f ? M.silu_alpha : 1.0f;
     if (M.gate_clip_min != 0.0f || M.gate_clip_max != 0.0f) a.gate_min = M.gate_clip_min, a.gate_max = M.gate_clip_max; // (all zero: a description that never set them)
     if (M.up_clip_min != 0.0f || M.up_clip_max != 0.0f) a.up_min = M.up_clip_min, a.up_max = M.up_clip_max;
-    a.up_offset = M.up_offset;
+    a.up_offset = M.up_offset, a.plain = M.plain_experts;
     return a;
 }
 
@@ -256,24 +265,48 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             k::rms_norm_add_rows(s, y, residual, out, N.scales, N.offset, layer_scale, N.eps, rows, d, next ? S.normed : nullptr, next ? next->scales : nullptr,
                                  next ? next->offset : 0.0f, next ? next->eps : 0.0f, N.groups));
     };
-    // what a sublayer without a pre norm reads: the stream rows themselves, or (with an input convolution) rows + conv(rows) in S.normed; `which` = 0 the mixer's
+    // what a sublayer reads: the stream rows (no pre norm) or its normed rows (S.normed), or, with an input convolution, rows + conv(rows); `which` = 0 the mixer's
     // window of the layer's state, 1 the MLP's.  The window is replaced right away: `x` still holds the pass's inputs here.
     auto conv_input = [&](uint32_t l, const float* x, const float* w, uint32_t taps, uint32_t which) -> const float* {
         if (!w) return x;
+        float* out = x == S.normed ? S.conv_rows : S.normed;
         k::CausalConvParams cp{};
-        cp.x = x, cp.ldx = d, cp.out = S.normed, cp.ldo = d, cp.w = w, cp.channels = d, cp.taps = taps, cp.add_input = 1;
+        cp.x = x, cp.ldx = d, cp.out = out, cp.ldo = d, cp.w = w, cp.channels = d, cp.taps = taps, cp.add_input = 1;
         cp.states = S.d_inconv_ptrs + (size_t)l * S.max_seqs, cp.state_offset = (size_t)which * (taps - 1) * d, cp.spans = S.d_spans, cp.row_seq = S.d_row_seq, cp.nseq = nseq, cp.rows = rows;
         cp.max_count = max_count;
         RUN("causal_conv_rows", (size_t)rows * d * 4 * (taps + 1), k::causal_conv_rows(s, cp));
         if (taps > 1 && max_count > 1) RUN("causal_conv_commit", (size_t)nseq * d * 8 * (taps - 1), k::causal_conv_commit(s, cp));
-        return S.normed;
+        return out;
+    };
+    // Hyper-connections: the launch between two sublayers.  A sublayer leaves its result in S.tmp and its in | out | mix weights in `join`; the next one's launch joins
+    // them to the copies (at the start all equal to the embedding rows, one block read for every copy), reads and norms its own row.
+    const uint32_t hs = m->d.hyper_streams;
+    const float* join = nullptr;
+    bool copies = false; // S.hyper holds the copies (else they all equal the embedding rows)
+    auto hyper_params = [&]() {
+        k::HyperStepParams hp{};
+        hp.src = copies ? S.hyper : S.slots, hp.src_stride = copies ? slot_stride : 0, hp.dst_stride = slot_stride;
+        if (join) hp.y = S.tmp, hp.join = join, hp.mult = m->d.residual_mult;
+        hp.rows = rows, hp.d = d, hp.streams = hs;
+        return hp;
+    };
+    auto hyper_input = [&](uint32_t l, const float* read, const DNorm& N, const float* conv_w, uint32_t taps, uint32_t which, float* tap) -> const float* {
+        k::HyperStepParams hp = hyper_params();
+        if (join) hp.dst = S.hyper;
+        hp.sum_out = tap, hp.read = read, hp.h = S.normed, hp.scales = N.scales, hp.offset = N.offset, hp.eps = N.eps;
+        const bool fused = conv_w && max_count == 1;
+        if (fused)
+            hp.conv_w = conv_w, hp.taps = taps, hp.states = S.d_inconv_ptrs + (size_t)l * S.max_seqs, hp.state_offset = (size_t)which * (taps - 1) * d, hp.spans = S.d_spans, hp.row_seq = S.d_row_seq;
+        RUN("hyper_step", (size_t)rows * d * 4 * ((join ? 2 * hs + 2 : copies ? hs + 1 : 2) + (fused ? 3 * taps - 2 : 0)), k::hyper_step(s, hp));
+        copies |= join != nullptr;
+        return fused ? S.normed : conv_input(l, S.normed, conv_w, taps, which);
     };
     bool normed_ready = false; // S.normed already holds this run's pre-mixer norm (left by the run before)
     for (uint32_t l = 0; l < nl; ++l) {
         DLayer& L = m->layers[l];
         const Stream32::Layer& X = S.layers[l];
         const uzu_layer_desc& h = L.d;
-        float* slot = S.slots + (size_t)(l + 1) * slot_stride; // X_(l+1): the layer's own result
+        float* slot = hs ? S.tmp : S.slots + (size_t)(l + 1) * slot_stride; // X_(l+1): the layer's own result (hyper-connections: the sublayer's, joined by the launch that follows)
         void* const* caches = S.d_cache_ptrs + (size_t)l * S.max_seqs;
         if (X.reentry_a.w) { // x <- W [x ; x0]: the two halves of W on the stream and on the embedding rows, summed
             run_linear(e, lin(S, X.reentry_a, cur, S.xin, rows));
@@ -293,7 +326,9 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         const bool have_normed = normed_ready;
         normed_ready = false;
         const float* mix_in = S.normed; // the rows the mixer reads
-        if (have_normed) {
+        if (hs) {
+            mix_in = hyper_input(l, X.hyper_mixer, L.pre_mixer, X.in_conv_mixer, h.input_conv_taps, 0, S.taps && l ? S.taps + (size_t)(l - 1) * slot_stride : nullptr);
+        } else if (have_normed) {
         } else if (!L.pre_mixer.present) {
             mix_in = conv_input(l, cur, X.in_conv_mixer, h.input_conv_taps, 0);
         } else if (h.pre_mixer_norm.kind != UZU_NORM_DYNAMIC_TANH) {
@@ -304,6 +339,7 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             np.spans = S.d_spans, np.row_seq = S.d_row_seq, np.prev = S.d_shift_ptrs + (size_t)l * S.max_seqs, np.rows = rows, np.d = d;
             RUN("dyn_tanh_norm+shift", (size_t)rows * d * 8, k::dyn_tanh_norm(s, np));
         }
+        if (!hs && L.pre_mixer.present && X.in_conv_mixer) mix_in = conv_input(l, S.normed, X.in_conv_mixer, h.input_conv_taps, 0);
         const uint32_t H = h.num_heads, hd = h.head_dim, vd = h.value_head_dim, rank = h.latent_rank;
         // prompt-sized pass over a pair of mixers: the first one's projection, rotation / append and attention core go to the side stream (they touch S.q, S.attn and
         // the caches; the second mixer touches its own rows); not while a launch is being timed or captured
@@ -369,7 +405,10 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             RUN("head_rms_gate", (size_t)rows * H * vd * 12, k::head_rms_gate(s, S.attn, S.q + 2 * H * hd + H * vd, ldq, h.head_norm_epsilon, rows, H, vd));
         } else {
         // rd: the rotated key part every head shares; the cache row is [latent | rotated part] (kw wide), a query head [plain | rotated] (qw wide)
-        const uint32_t rd = h.latent_rope_dim, kw = rank + rd, qw = hd + rd, ldq = L.qkv.n;
+        const uint32_t rd = h.latent_rope_dim, kw = rank + rd, qw = hd + rd, ldq = L.qkv.n, qr = h.latent_query_rank;
+        const float* queries = S.q; // rows of [heads][qw]
+        uint32_t ldqueries = ldq;
+        const uint32_t c_col = qr ? qr : H * qw; // packed: where the down projection's numbers start
         if (!h.is_kv_sharing && !h.latent_packed) run_linear(e, lin(S, L.lat_down, mix_in, S.ckv, rows));
         if (!rd && !h.latent_packed) {
             if (!h.is_kv_sharing)
@@ -377,10 +416,21 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                     k::latent_norm_append(s, S.ckv, L.lat_norm.scales, L.lat_norm.eps, caches, bf, S.d_spans, S.d_row_seq, rows, rank));
         } else {
             k::LatentRopeAppendParams lp{};
-            lp.x = h.latent_packed ? S.q : S.ckv, lp.ldx = h.latent_packed ? ldq : L.lat_down.n, lp.c_col = h.latent_packed ? H * qw : 0, lp.rank = rank, lp.rope_dim = rd;
+            lp.x = h.latent_packed ? S.q : S.ckv, lp.ldx = h.latent_packed ? ldq : L.lat_down.n, lp.c_col = h.latent_packed ? c_col : 0, lp.rank = rank, lp.rope_dim = rd;
             lp.scales = L.lat_norm.scales, lp.eps = L.lat_norm.eps, lp.caches = h.is_kv_sharing ? nullptr : caches, lp.cache_bf16 = bf, lp.heads = H, lp.q_width = qw;
             lp.qlat = rd ? S.qlat : nullptr, lp.cosines = L.rope_cos, lp.sines = L.rope_sin, lp.interleaved = h.rope_interleaved, lp.spans = S.d_spans, lp.row_seq = S.d_row_seq, lp.rows = rows;
-            if (h.latent_packed) { // the rotated query parts are read from the packed rows; a separate down projection leaves them in S.q as well
+            if (qr) { // cache rows and the query latent's norm; the queries of that latent; their rotated parts
+                k::LatentRopeAppendParams cp = lp;
+                cp.qlat = nullptr, cp.q_rank = qr, cp.q_scales = X.lat_q_norm.scales, cp.q_latent = S.ckv;
+                RUN("latent_rope_append", (size_t)rows * (kw * 6 + qr * 8), k::latent_rope_append(s, cp));
+                run_linear(e, lin(S, X.lat_q_up, S.ckv, S.lat_q, rows));
+                queries = S.lat_q, ldqueries = H * qw;
+                if (rd) {
+                    k::LatentRopeAppendParams qp = lp;
+                    qp.x = queries, qp.ldx = ldqueries, qp.c_col = 0, qp.caches = nullptr;
+                    RUN("latent_rope_append", (size_t)rows * H * rd * 8, k::latent_rope_append(s, qp));
+                }
+            } else if (h.latent_packed) { // the rotated query parts are read from the packed rows; a separate down projection leaves them in S.q as well
                 RUN("latent_rope_append", (size_t)rows * (kw * 6 + H * rd * 8), k::latent_rope_append(s, lp));
             } else {
                 k::LatentRopeAppendParams cp = lp; // cache rows from the down projection's rows, query parts from the query rows
@@ -395,7 +445,7 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         }
         {   // the head's key projection folded into the query: qlat[r, h, :rank] = W_up_k[h]^T q[r, h, :hd]
             k::LinearF32Params p{};
-            p.x = S.q, p.w = X.up_keys_t, p.y = S.qlat, p.rows = rows, p.n = rank, p.k = hd, p.ldx = ldq, p.ldy = H * kw, p.batch = H;
+            p.x = queries, p.w = X.up_keys_t, p.y = S.qlat, p.rows = rows, p.n = rank, p.k = hd, p.ldx = ldqueries, p.ldy = H * kw, p.batch = H;
             p.x_batch = qw, p.w_batch = (size_t)rank * hd, p.y_batch = kw, p.bf16_products = bf;
             run_linear(e, p);
         }
@@ -417,7 +467,7 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             k::LinearF32Params p{};
             p.x = S.ctx, p.w = (const uint16_t*)L.lat_up_v.w, p.y = S.attn, p.rows = rows, p.n = vd, p.k = rank, p.ldx = H * kw, p.ldy = H * vd, p.batch = H;
             p.x_batch = kw, p.w_batch = (size_t)vd * rank, p.y_batch = vd, p.bf16_products = bf;
-            if (h.has_gate) p.gate = S.q + H * qw + (h.latent_packed ? kw : 0), p.ldgate = ldq;
+            if (h.has_gate) p.gate = S.q + c_col + (h.latent_packed ? kw : 0), p.ldgate = ldq, p.gate_batch = h.gate_elementwise ? vd : 0;
             run_linear(e, p);
         }
         } // latent attention
@@ -473,39 +523,55 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             normed_ready = h.no_mlp && !h.has_ple && next_pre;
         } else { // X_(l+1) = input + out projection
             k::LinearF32Params p = lin(S, L.out, S.attn, slot, rows);
-            p.residual = cur, p.ldr = d;
+            if (!hs) p.residual = cur, p.ldr = d;
             run_linear(e, p);
+            join = X.hyper_mixer;
         }
         if (!h.no_mlp) {
             // a parallel block's MLP reads the rows the mixer read (still in S.normed) and adds to the same sum; otherwise the MLP has its own norm of the sum so far
             const float* mlp_in = h.parallel_block ? mix_in : S.normed;
-            if (!h.parallel_block && !L.pre_mlp.present) mlp_in = conv_input(l, slot, X.in_conv_mlp, h.input_conv_taps, 1); // no pre norm: the stream itself (+ its convolution)
+            if (hs) mlp_in = hyper_input(l, X.hyper_mlp, L.pre_mlp, X.in_conv_mlp, h.input_conv_taps, 1, nullptr);
+            else if (!h.parallel_block && !L.pre_mlp.present) mlp_in = conv_input(l, slot, X.in_conv_mlp, h.input_conv_taps, 1); // no pre norm: the stream itself (+ its convolution)
             else if (!h.parallel_block && !pre_mlp_fused) run_norm(e, L.pre_mlp, h.pre_mlp_norm.kind, X.alpha2, slot, S.normed, rows, d, nullptr);
+            if (!hs && !h.parallel_block && L.pre_mlp.present && X.in_conv_mlp) mlp_in = conv_input(l, S.normed, X.in_conv_mlp, h.input_conv_taps, 1);
             if (h.mlp_kind == UZU_MLP_MOE) {
                 const uzu_moe_desc& M = h.moe;
                 const uint32_t E = M.num_routed_experts, top = M.num_active_experts, ff = M.expert_hidden_dim;
                 const k::ExpertAct act = expert_act(M);
-                if (M.routing == UZU_MOE_ROUTE_SCORES) {
+                const float* res = hs ? nullptr : slot; // (hyper-connections: the launch that follows joins the result)
+                if (M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS) {
+                    k::RouteGroupsParams rp{};
+                    rp.x = mlp_in, rp.router = L.moe.router_weights, rp.selection_bias = X.selection_bias, rp.ids = S.moe_ids, rp.weights = S.moe_w, rp.rows = rows, rp.d = d, rp.outputs = E;
+                    rp.top = top, rp.groups = M.router_groups ? M.router_groups : 1, rp.keep = M.router_groups_keep ? M.router_groups_keep : rp.groups, rp.bf16_products = bf;
+                    rp.scale = M.router_scale != 0.0f ? M.router_scale : 1.0f;
+                    if (rows > 16) { // many rows: the logits as one product (f32 sums)
+                        k::LinearF32Params zp{};
+                        zp.x = mlp_in, zp.w = L.moe.router_weights, zp.y = S.moe_z, zp.rows = rows, zp.n = E, zp.k = d, zp.ldx = d, zp.ldy = E, zp.batch = 1, zp.bf16_products = bf;
+                        run_linear(e, zp);
+                        rp.logits = S.moe_z;
+                    }
+                    RUN("moe_route_groups", (size_t)E * d * 2, k::moe_route_groups(s, rp));
+                } else if (M.routing == UZU_MOE_ROUTE_SCORES) {
                     RUN("moe_route_scores", (size_t)(E + M.num_identity_experts) * d * 2,
                         k::moe_route_scores(s, mlp_in, L.moe.router_weights, X.selection_bias, S.moe_ids, S.moe_w, rows, d, E + M.num_identity_experts, top));
                 } else {
                     RUN("moe_route_topk", (size_t)E * d * 2, k::moe_route_topk(s, mlp_in, L.moe.router_weights, L.moe.router_biases, S.moe_ids, S.moe_w, rows, d, E, top, M.router_renorm));
                 }
                 k::MoeGroupedParams gp{};
-                gp.x = mlp_in, gp.ids = S.moe_ids, gp.weights = S.moe_w, gp.w13 = L.moe.w13, gp.w2 = L.moe.w2, gp.residual = slot, gp.y = slot, gp.y1 = S.moe_y1, gp.hidden = S.hid;
+                gp.x = mlp_in, gp.ids = S.moe_ids, gp.weights = S.moe_w, gp.w13 = L.moe.w13, gp.w2 = L.moe.w2, gp.residual = res, gp.y = slot, gp.y1 = S.moe_y1, gp.hidden = S.hid;
                 gp.y2 = S.moe_y2, gp.perm = S.moe_perm, gp.slot_pos = S.moe_slot_pos, gp.offsets = S.moe_offsets, gp.cursor = S.moe_cursor;
                 gp.rows = rows, gp.d = d, gp.ff = ff, gp.routed = E, gp.top = top, gp.act = act;
                 if (bf && k::moe_experts_grouped_supported(gp)) { // prefill-sized: buckets per expert through the matrix-core linear
-                    RUN("moe_experts_grouped", (size_t)E * 3 * ff * d * 2 + (size_t)rows * top * (3 * ff + 2 * d) * 4, k::moe_experts_grouped(s, gp));
+                    RUN("moe_experts_grouped", (size_t)E * (act.plain ? 2 : 3) * ff * d * 2 + (size_t)rows * top * ((act.plain ? 1 : 3) * ff + 2 * d) * 4, k::moe_experts_grouped(s, gp));
                 } else {
-                    RUN("moe_experts_gate_up", (size_t)rows * top * 2 * ff * d * 2, k::moe_experts_gate_up(s, mlp_in, S.moe_ids, L.moe.w13, S.hid, rows, d, ff, E, top, bf, act));
+                    RUN("moe_experts_gate_up", (size_t)rows * top * (act.plain ? 1 : 2) * ff * d * 2, k::moe_experts_gate_up(s, mlp_in, S.moe_ids, L.moe.w13, S.hid, rows, d, ff, E, top, bf, act));
                     RUN("moe_experts_down_combine", (size_t)rows * top * ff * d * 2,
-                        k::moe_experts_down_combine(s, S.hid, mlp_in, S.moe_ids, S.moe_w, L.moe.w2, slot, slot, rows, d, ff, E, top, bf));
+                        k::moe_experts_down_combine(s, S.hid, mlp_in, S.moe_ids, S.moe_w, L.moe.w2, res, slot, rows, d, ff, E, top, bf));
                 }
             } else {
                 if (h.mlp_plain) {
                     k::LinearF32Params up = lin(S, L.up, mlp_in, S.hid, rows);
-                    up.act = 1;
+                    up.act = h.activation == UZU_ACT_XIELU ? 3 : 1, up.act_a = X.act_a, up.act_b = X.act_b;
                     run_linear(e, up);
                 } else { // gated: [up ; gate] rows of one projection, then the clamped gate product
                     run_linear(e, lin(S, L.up, mlp_in, S.y1, rows));
@@ -519,10 +585,11 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                     normed_ready = !h.has_ple && next_pre;
                 } else {
                     k::LinearF32Params down = lin(S, L.down, S.hid, slot, rows);
-                    down.residual = slot, down.ldr = d;
+                    if (!hs) down.residual = slot, down.ldr = d;
                     run_linear(e, down);
                 }
             }
+            if (hs) join = X.hyper_mlp;
         }
         if (h.has_ple) { // the per-layer token input: x <- x + norm(projection(gelu(gate x) * the token's slice of the side table))
             k::LinearF32Params g = lin(S, L.ple_gate, slot, S.side_g, rows); // gelu and the token's slice in the product's epilogue
@@ -539,12 +606,22 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         } else {
             cur = slot;
         }
-        if (S.taps) HIPCHK(hipMemcpyAsync(S.taps + (size_t)l * slot_stride, cur, (size_t)rows * d * 4, hipMemcpyDeviceToDevice, s));
+        if (S.taps && !hs) HIPCHK(hipMemcpyAsync(S.taps + (size_t)l * slot_stride, cur, (size_t)rows * d * 4, hipMemcpyDeviceToDevice, s));
     }
     S.tap_rows = rows;
     S.last_logit_rows = 0;
+    if (hs && S.taps) {
+        k::HyperStepParams hp = hyper_params();
+        hp.sum_out = S.taps + (size_t)(nl - 1) * slot_stride;
+        RUN("hyper_step", (size_t)rows * d * 4 * (hs + 2), k::hyper_step(s, hp));
+    }
     if (n_out) {
-        run_norm(e, m->output_norm, m->d.output_norm.kind, S.alpha_out, cur, S.out_normed, n_out, d, S.d_out_rows);
+        if (hs) { // the wanted rows alone: the last sublayer's result joins, the copies' sum is normed
+            k::HyperStepParams hp = hyper_params();
+            const DNorm& N = m->output_norm;
+            hp.h = S.out_normed, hp.scales = N.scales, hp.offset = N.offset, hp.eps = N.eps, hp.row_index = S.d_out_rows, hp.rows = n_out;
+            RUN("hyper_step", (size_t)n_out * d * 4 * (hs + 2), k::hyper_step(s, hp));
+        } else run_norm(e, m->output_norm, m->d.output_norm.kind, S.alpha_out, cur, S.out_normed, n_out, d, S.d_out_rows);
         k::LinearF32Params head = lin(S, m->d.tied_embeddings ? m->embedding : m->output_embedding, S.out_normed, S.logits, n_out);
         if (m->d.logit_scale != 1.0f) head.y_scale = m->d.logit_scale; // (0 = a description that never set it)
         head.soft_cap = m->d.logit_soft_cap;
@@ -626,6 +703,8 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     auto rms_vec = [](const uzu_norm_desc& n) { return n.present && n.kind == UZU_NORM_STATISTICS && n.scales && !n.subtract_mean && !n.biases; };
     auto norm_ok = [&](const uzu_norm_desc& n) { return n.present && ((n.kind == UZU_NORM_DYNAMIC_TANH && n.scales) || n.kind == UZU_NORM_RMS_SCALAR || rms_vec(n)); };
     UZU_REQUIRE(norm_ok(desc->output_norm), "model_create: an f32-stream design ends in a dynamic-tanh norm or an RMS norm (one gain, or a weight vector)");
+    UZU_REQUIRE(!desc->hyper_streams || (desc->hyper_streams <= k::kHyperMaxStreams && d <= k::kHyperMaxWidth && rms_vec(desc->output_norm) && desc->output_norm.groups <= 1),
+                "model_create: hyper-connections: at most %u copies of a stream of width %u, an undivided RMS norm with a weight vector at the end", k::kHyperMaxStreams, k::kHyperMaxWidth);
     UZU_UNSUPPORTED(desc->embedding_norm.present, "model_create: decoder options of the bf16-stream families on an f32-stream design");
     auto groups_ok = [&](const uzu_norm_desc& n, uint32_t dim) { return n.groups <= 1 || (rms_vec(n) && dim % n.groups == 0); };
     UZU_REQUIRE(groups_ok(desc->output_norm, d), "model_create: a norm in parts is an RMS norm with a weight vector over model_dim %% groups == 0 coordinates");
@@ -650,8 +729,14 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
         UZU_REQUIRE(groups_ok(h.pre_mixer_norm, d) && groups_ok(h.post_mixer_norm, d) && groups_ok(h.pre_mlp_norm, d) && groups_ok(h.post_mlp_norm, d),
                     "model_create: layer %u: a norm in parts is an RMS norm with a weight vector over model_dim %% groups == 0 coordinates", l);
         UZU_REQUIRE(!(h.input_conv_mixer || h.input_conv_mlp) || (h.input_conv_taps >= 1 && h.input_conv_taps <= 64), "model_create: layer %u: an input convolution of 1 .. 64 taps", l);
-        UZU_UNSUPPORTED((h.input_conv_mixer && h.pre_mixer_norm.present) || (h.input_conv_mlp && (h.pre_mlp_norm.present || h.parallel_block || h.no_mlp)),
-                        "model_create: layer %u: an input convolution feeds a sublayer that reads the stream itself (no pre norm)", l);
+        UZU_UNSUPPORTED((h.input_conv_mixer && h.token_shift) || (h.input_conv_mlp && (h.parallel_block || h.no_mlp)),
+                        "model_create: layer %u: an input convolution on token-shifted rows, or on the MLP of a parallel block or of a layer without one", l);
+        if (desc->hyper_streams) {
+            UZU_REQUIRE(rms_vec(h.pre_mixer_norm) && h.pre_mixer_norm.groups <= 1 && h.hyper_mixer && (h.no_mlp || (rms_vec(h.pre_mlp_norm) && h.pre_mlp_norm.groups <= 1 && h.hyper_mlp)),
+                        "model_create: layer %u: under hyper-connections a sublayer has an undivided RMS norm with a weight vector in front of it and its in | out | mix weights", l);
+            UZU_UNSUPPORTED(h.post_mixer_norm.present || h.post_mlp_norm.present || h.parallel_block || h.token_shift || h.depth_weights || h.has_ple || h.pair_mixer || h.stream_reentry.weights,
+                            "model_create: layer %u: post norms, parallel blocks, token shift, depth mix, token input, a pair of mixers and a re-entry projection belong to a single stream", l);
+        }
         UZU_UNSUPPORTED(!h.pre_mixer_norm.present && h.stream_reentry.weights, "model_create: layer %u: a re-entry projection in front of a mixer without a pre norm", l);
         UZU_UNSUPPORTED(h.token_shift && h.pre_mixer_norm.kind != UZU_NORM_DYNAMIC_TANH, "model_create: layer %u: the token shift follows a dynamic-tanh norm", l);
         UZU_REQUIRE(!h.post_mixer_norm.present || rms_vec(h.post_mixer_norm), "model_create: layer %u: a post-mixer norm is an RMS norm with a weight vector", l);
@@ -702,9 +787,13 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             UZU_REQUIRE(full(h.latent_up_keys, h.num_heads * h.head_dim, h.latent_rank) && full(h.latent_up_values, h.num_heads * h.value_head_dim, h.latent_rank),
                         "model_create: layer %u: latent up projections must be full-precision matrices of the configured shapes", l);
             if (h.latent_packed) {
-                UZU_REQUIRE(!h.is_kv_sharing && !h.latent_down.weights && full(h.qkv_projection, qn + kw + (h.has_gate ? h.num_heads : 0), d) && h.latent_norm.present && h.latent_norm.scales,
-                            "model_create: layer %u: the packed projection is queries | down projection | gates [heads (head_dim + rope) + rank + rope (+ heads), model_dim], with the latent norm", l);
+                const uint32_t qr = h.latent_query_rank, gates = h.has_gate ? (h.gate_elementwise ? h.num_heads * h.value_head_dim : h.num_heads) : 0;
+                UZU_REQUIRE(!h.is_kv_sharing && !h.latent_down.weights && full(h.qkv_projection, (qr ? qr : qn) + kw + gates, d) && h.latent_norm.present && h.latent_norm.scales,
+                            "model_create: layer %u: the packed projection is queries (or their latent) | down projection | gates [heads (head_dim + rope) + rank + rope (+ gates), model_dim], with the latent norm", l);
+                UZU_REQUIRE(!qr || (rms_vec(h.latent_query_norm) && h.latent_query_norm.epsilon == h.latent_norm.epsilon && h.latent_query_norm.scale_offset == 0.0f && full(h.latent_query_up, qn, qr) && !h.latent_query_up.out_biases),
+                            "model_create: layer %u: a query latent has an RMS norm with plain weights, the latent norm's epsilon, and an up projection [heads (head_dim + rope), query rank]", l);
             } else {
+                UZU_UNSUPPORTED(h.latent_query_rank || h.gate_elementwise, "model_create: layer %u: a query latent and a gate per coordinate come with a packed projection", l);
                 UZU_REQUIRE(full(h.qkv_projection, qn + (h.has_gate ? h.num_heads : 0), d), "model_create: layer %u: the query projection must be a full-precision matrix of the configured shape", l);
             }
             if (h.is_kv_sharing) {
@@ -761,14 +850,18 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                         "model_create: layer %u: a pre-MLP norm is a dynamic-tanh or RMS norm (absent: the MLP reads the stream), and none in a parallel block", l);
             if (h.mlp_kind == UZU_MLP_MOE) {
                 const uzu_moe_desc& M = h.moe;
-                UZU_REQUIRE((M.routing == UZU_MOE_ROUTE_SCORES || M.routing == UZU_MOE_ROUTE_TOPK_LOGITS) && M.num_active_experts &&
+                UZU_REQUIRE((M.routing == UZU_MOE_ROUTE_SCORES || M.routing == UZU_MOE_ROUTE_TOPK_LOGITS || M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS) && M.num_active_experts &&
                             M.num_active_experts <= M.num_routed_experts + M.num_identity_experts && M.router_weights &&
                             (M.num_routed_experts == 0 || (M.expert_hidden_dim && M.w13 && M.w2)) && M.gating_sel == 2 && !M.up_biases && !M.down_biases,
                             "model_create: layer %u: routed SiLU-gated experts without biases, with their router and expert tensors", l);
-                UZU_REQUIRE(M.routing == UZU_MOE_ROUTE_SCORES || (!M.num_identity_experts && !M.selection_bias), "model_create: layer %u: identity experts and selection biases belong to score routing", l);
+                if (M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS) {
+                    const uint32_t G = M.router_groups ? M.router_groups : 1, keep = M.router_groups_keep ? M.router_groups_keep : G;
+                    UZU_REQUIRE(!M.num_identity_experts && !M.router_biases && M.num_routed_experts % G == 0 && keep <= G && M.num_active_experts <= M.num_routed_experts / G * keep,
+                                "model_create: layer %u: %u winners among the experts of %u of %u equal groups", l, M.num_active_experts, keep, G);
+                } else UZU_REQUIRE(M.routing == UZU_MOE_ROUTE_SCORES || (!M.num_identity_experts && !M.selection_bias), "model_create: layer %u: identity experts and selection biases belong to score routing", l);
             } else if (h.mlp_plain) {
-                UZU_REQUIRE(h.activation == UZU_ACT_RELU_SQUARED && full(h.up_projection, h.hidden_dim, d) && full(h.down_projection, d, h.hidden_dim),
-                            "model_create: layer %u: the plain dense block is down(relu(up x + b)^2) + b with full-precision matrices", l);
+                UZU_REQUIRE((h.activation == UZU_ACT_RELU_SQUARED || h.activation == UZU_ACT_XIELU) && full(h.up_projection, h.hidden_dim, d) && full(h.down_projection, d, h.hidden_dim),
+                            "model_create: layer %u: the plain dense block is down(act(up x + b)) + b, act = the squared relu or xIELU, with full-precision matrices", l);
             } else {
                 UZU_REQUIRE((h.activation == UZU_ACT_SILU || h.activation == UZU_ACT_GELU_APPROX) && h.hidden_dim && full(h.up_projection, 2 * h.hidden_dim, d) &&
                             full(h.down_projection, d, h.hidden_dim) && !h.parallel_block,
@@ -801,13 +894,14 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     S.layers.resize(nl);
     uint32_t w_q = 0, w_rank = 0, w_lat = 0, w_attn = 0, w_hid = 0, w_top = 1, w_moe = 0, w_routed = 0, w_lru = 0, w_side = 0, w_y1 = 0;
     uint32_t w_dn_in = 0, w_dn_cv = 0, w_dn_k = 0, w_dn_v = 0;
-    bool any_pair = false, any_inconv = false;
+    bool any_pair = false, any_inconv = false, any_normed_conv = false;
+    uint32_t w_latq = 0;
     for (uint32_t l = 0; l < nl; ++l) {
         const uzu_layer_desc& h = desc->layers[l];
         DLayer& L = m->layers[l];
         Stream32::Layer& X = S.layers[l];
         uint32_t kw_l = h.latent_rank + h.latent_rope_dim;
-        w_q = std::max(w_q, h.qkv_projection.n), w_rank = std::max(w_rank, h.latent_down.n ? h.latent_down.n : kw_l), w_lat = std::max(w_lat, h.num_heads * kw_l);
+        w_q = std::max(w_q, h.qkv_projection.n), w_rank = std::max({w_rank, h.latent_down.n ? h.latent_down.n : kw_l, h.latent_query_rank}), w_lat = std::max(w_lat, h.num_heads * kw_l);
         w_attn = std::max(w_attn, std::max(h.num_heads * h.value_head_dim, h.lru_width)), w_lru = std::max(w_lru, h.lru_width), w_side = std::max(w_side, h.has_ple ? h.ple_dim : 0u);
         if (!h.no_mlp && h.mlp_kind != UZU_MLP_MOE) w_hid = std::max(w_hid, h.hidden_dim), w_y1 = std::max(w_y1, h.mlp_plain ? 0u : 2 * h.hidden_dim);
         if (h.weights_of_layer) { // the tensors of an earlier run: its device pointers, this run's own scalars; nothing is uploaded twice
@@ -815,6 +909,7 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             X = S.layers[h.weights_of_layer - 1];
             L.d = h;
             L.last_reader = l;
+            any_normed_conv |= (h.pre_mixer_norm.present && h.input_conv_mixer) || (h.pre_mlp_norm.present && h.input_conv_mlp);
             if (!h.no_mlp && h.mlp_kind == UZU_MLP_MOE) {
                 const uzu_moe_desc& M = h.moe;
                 w_hid = std::max<uint32_t>(w_hid, M.num_active_experts * M.expert_hidden_dim), w_top = std::max(w_top, M.num_active_experts);
@@ -884,6 +979,9 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
         }
         if (h.input_conv_mixer) TRY(upload(m, h.input_conv_mixer, (size_t)d * h.input_conv_taps * 4, &X.in_conv_mixer));
         if (h.input_conv_mlp) TRY(upload(m, h.input_conv_mlp, (size_t)d * h.input_conv_taps * 4, &X.in_conv_mlp));
+        any_normed_conv |= (h.pre_mixer_norm.present && h.input_conv_mixer) || (h.pre_mlp_norm.present && h.input_conv_mlp);
+        if (h.hyper_mixer && desc->hyper_streams) TRY(upload(m, h.hyper_mixer, (size_t)desc->hyper_streams * (desc->hyper_streams + 2) * 4, &X.hyper_mixer));
+        if (h.hyper_mlp && desc->hyper_streams) TRY(upload(m, h.hyper_mlp, (size_t)desc->hyper_streams * (desc->hyper_streams + 2) * 4, &X.hyper_mlp));
         any_pair |= h.pair_mixer != 0, any_inconv |= h.input_conv_mixer || h.input_conv_mlp;
         if (h.mixer_kind == UZU_MIXER_GATED_LRU) {
             const size_t w = h.lru_width, bw = w / h.lru_blocks;
@@ -903,6 +1001,11 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
         }
         if (h.mixer_kind == UZU_MIXER_LATENT_ATTENTION) {
         TRY(upload_linear(m, h.latent_up_values, &L.lat_up_v));
+        if (h.latent_query_rank) {
+            TRY(upload_linear(m, h.latent_query_up, &X.lat_q_up));
+            TRY(upload_norm(m, h.latent_query_norm, h.latent_query_rank, &X.lat_q_norm));
+            w_latq = std::max(w_latq, h.latent_query_up.n);
+        }
         {   // W_up_k [heads * head_dim, rank] -> per head [rank, head_dim] (bf16 bits move, nothing is rounded)
             const uint32_t H = h.num_heads, hd = h.head_dim, rank = h.latent_rank;
             const uint16_t* src = (const uint16_t*)h.latent_up_keys.weights;
@@ -934,7 +1037,7 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                 TRY(upload(m, M.router_weights, (E + M.num_identity_experts) * d * 2, &L.moe.router_weights));
                 if (M.router_biases) TRY(upload(m, M.router_biases, (E + M.num_identity_experts) * 2, &L.moe.router_biases));
                 if (E) {
-                    TRY(upload(m, M.w13, E * 2 * ff * d * 2, &L.moe.w13));
+                    TRY(upload(m, M.w13, E * (M.plain_experts ? 1 : 2) * ff * d * 2, &L.moe.w13)); // (experts without a gate: up rows alone)
                     TRY(upload(m, M.w2, E * d * ff * 2, &L.moe.w2));
                 }
                 if (M.selection_bias) TRY(upload(m, M.selection_bias, (E + M.num_identity_experts) * 4, &X.selection_bias));
@@ -942,6 +1045,10 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                 w_top = std::max(w_top, M.num_active_experts);
                 w_moe = std::max(w_moe, M.num_active_experts * 2 * M.expert_hidden_dim), w_routed = std::max(w_routed, M.num_routed_experts);
             } else {
+                if (h.activation == UZU_ACT_XIELU) {
+                    auto softplus = [](double z) { return z > 0.0 ? z + log1p(exp(-z)) : log1p(exp(z)); };
+                    X.act_a = (float)softplus((double)h.xielu_p), X.act_b = (float)(0.5 + softplus((double)h.xielu_q));
+                }
                 TRY(upload_linear(m, h.up_projection, &L.up));
                 TRY(upload_linear(m, h.down_projection, &L.down));
             }
@@ -976,7 +1083,11 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     const size_t R = S.max_rows;
     if (!w_lat) w_lat = 1;
     if (!w_rank) w_rank = 1;
-    TRY(need_f32(m, (size_t)(nl + 1) * R * d, &S.slots));
+    TRY(need_f32(m, (size_t)(desc->hyper_streams ? 1 : nl + 1) * R * d, &S.slots)); // (hyper-connections: the embedding rows alone)
+    if (desc->hyper_streams) TRY(need_f32(m, (size_t)desc->hyper_streams * R * d, &S.hyper));
+    if (any_normed_conv) TRY(need_f32(m, R * d, &S.conv_rows));
+    if (w_latq) TRY(need_f32(m, R * w_latq, &S.lat_q));
+    if (w_routed) TRY(need_f32(m, R * w_routed, &S.moe_z));
     TRY(need_f32(m, R * d, &S.xin));
     TRY(need_f32(m, R * d, &S.normed));
     TRY(need_f32(m, R * d, &S.out_normed));

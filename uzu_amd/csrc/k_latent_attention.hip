@@ -73,6 +73,13 @@ __global__ void __launch_bounds__(256) latent_rope_append_kernel(LatentRopeAppen
             else ((float*)cache)[base + p.rank + lo_of(i)] = a, ((float*)cache)[base + p.rank + hi_of(i)] = b;
         }
     }
+    if (wave == 1 && p.q_rank) { // the query latent's norm
+        float ss = 0.0f;
+        for (uint32_t i = lane; i < p.q_rank; i += 64) ss = fmaf(xr[i], xr[i], ss);
+        ss = wave_sum(ss);
+        const float inv = 1.0f / sqrtf(ss / (float)p.q_rank + p.eps);
+        for (uint32_t i = lane; i < p.q_rank; i += 64) p.q_latent[(size_t)r * p.q_rank + i] = xr[i] * inv * p.q_scales[i];
+    }
     if (!p.qlat) return;
     for (uint32_t idx = threadIdx.x; idx < p.heads * half; idx += 256) {
         const uint32_t a = idx / half, i = idx - a * half;
@@ -357,7 +364,8 @@ uzu_status latent_rope_append(hipStream_t s, const LatentRopeAppendParams& p) {
     if (!p.rows) return UZU_OK;
     UZU_REQUIRE(p.x && p.spans && p.row_seq && p.rank && (!p.caches || p.scales), "latent_rope_append: null argument");
     UZU_REQUIRE(p.rope_dim % 2 == 0 && (!p.rope_dim || (p.cosines && p.sines && p.q_width >= p.rope_dim)), "latent_rope_append: an even rotated width with its tables");
-    UZU_REQUIRE(p.c_col + p.rank + p.rope_dim <= p.ldx && (!p.qlat || p.heads * p.q_width <= p.ldx), "latent_rope_append: columns outside the row");
+    UZU_REQUIRE((!p.caches || p.c_col + p.rank + p.rope_dim <= p.ldx) && (!p.qlat || p.heads * p.q_width <= p.ldx), "latent_rope_append: columns outside the row");
+    UZU_REQUIRE(!p.q_rank || (p.q_scales && p.q_latent && !p.qlat && p.q_rank <= p.ldx), "latent_rope_append: a query latent needs its norm and rows of its own");
     return launch_check([&] { hipLaunchKernelGGL(latent_rope_append_kernel, dim3(p.rows), dim3(256), 0, s, p); }, "latent_rope_append");
 }
 

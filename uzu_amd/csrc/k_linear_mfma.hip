@@ -11,6 +11,7 @@
 #include "device_utils.h"
 #include "gemm_convert.h"
 #include "kernels_stream32.h"
+#include "stream32_epilogue.h"
 
 namespace uzu {
 namespace k {
@@ -120,23 +121,7 @@ __global__ void __launch_bounds__(256) linear_mfma_kernel(LinearF32Params p) {
             for (int r = 0; r < 16; ++r) {
                 const uint32_t row = m0 + (wm * MB + i) * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
                 if (row >= r_hi) continue;
-                float v = acc[i][j][r] + bias;
-                if (p.act == 1) {
-                    const float t = fmaxf(v, 0.0f);
-                    v = t * t;
-                } else if (p.act == 2) {
-                    v = 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)));
-                }
-                if (p.y_scale != 0.0f) v *= p.y_scale;
-                if (p.soft_cap != 0.0f) v = p.soft_cap * tanhf(v / p.soft_cap);
-                if (p.gate) v *= 1.0f / (1.0f + expf(-p.gate[(size_t)row * p.ldgate + z]));
-                if (p.mul_table) {
-                    uint32_t t = p.mul_tokens[row];
-                    if (t >= p.mul_vocab) t = 0;
-                    v *= bf16_to_f32(p.mul_table[(size_t)t * p.mul_ld + p.mul_col0 + n]);
-                }
-                if (p.residual) v += p.residual[(size_t)row * p.ldr + n];
-                y[(size_t)row * p.ldy + n] = v;
+                y[(size_t)row * p.ldy + n] = linear_epilogue(acc[i][j][r], bias, p, row, z, n);
             }
         }
     }

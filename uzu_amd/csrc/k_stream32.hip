@@ -5,6 +5,7 @@
 // would have held), otherwise the product is a true f32 product.  Reductions run in a fixed order: a result does not depend on what else is in the pass.
 #include "device_utils.h"
 #include "kernels_stream32.h"
+#include "stream32_epilogue.h"
 
 namespace uzu {
 namespace k {
@@ -180,8 +181,6 @@ __global__ void __launch_bounds__(256) rms_norm_add_rows_kernel(const float* y, 
     }
 }
 
-__device__ __forceinline__ float gelu_tanh_f32(float z) { return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z))); }
-
 __global__ void __launch_bounds__(256) dyn_tanh_kernel(DynTanhParams p) {
     const uint32_t r = blockIdx.x;
     const uint32_t src = p.row_index ? p.row_index[r] : r;
@@ -224,29 +223,6 @@ __device__ __forceinline__ float expert_act(float gate, float up, const ExpertAc
     const float g = fminf(fmaxf(gate, a.gate_min), a.gate_max), u = fminf(fmaxf(up, a.up_min), a.up_max);
     if (a.gelu) return gelu_tanh_f32(g) * (u + a.up_offset);
     return g / (1.0f + expf(-(a.alpha * g))) * (u + a.up_offset);
-}
-
-__device__ __forceinline__ float apply_act(float v, uint32_t act) {
-    if (act == 1) {
-        const float t = fmaxf(v, 0.0f);
-        return t * t;
-    }
-    if (act == 2) return gelu_tanh_f32(v);
-    return v;
-}
-// what follows the activation: the product's scale, a per-(row, product) sigmoid gate
-__device__ __forceinline__ float apply_tail(float v, const LinearF32Params& p, uint32_t r, uint32_t z) {
-    if (p.y_scale != 0.0f) v *= p.y_scale;
-    if (p.soft_cap != 0.0f) v = p.soft_cap * tanhf(v / p.soft_cap);
-    if (p.gate) v *= 1.0f / (1.0f + expf(-p.gate[(size_t)r * p.ldgate + z]));
-    return v;
-}
-// ... and a per-(row's token, column) multiplier from a bf16 table
-__device__ __forceinline__ float apply_token_mul(float v, const LinearF32Params& p, uint32_t r, uint32_t n) {
-    if (!p.mul_table) return v;
-    uint32_t t = p.mul_tokens[r];
-    if (t >= p.mul_vocab) t = 0;
-    return v * bf16_to_f32(p.mul_table[(size_t)t * p.mul_ld + p.mul_col0 + n]);
 }
 
 // thread = (row, hidden unit): a one-row decode step still spreads over ff / 256 workgroups
@@ -305,9 +281,7 @@ __global__ void __launch_bounds__(256) linear_rows_kernel(LinearF32Params p, uin
         for (int i = 0; i < RT; ++i) {
             const uint32_t r = r0 + i;
             if (r >= p.rows) break;
-            float v = apply_token_mul(apply_tail(apply_act(acc[i] + bias, p.act), p, r, z), p, r, n);
-            if (p.residual) v += p.residual[(size_t)r * p.ldr + n];
-            y[(size_t)r * p.ldy + n] = v;
+            y[(size_t)r * p.ldy + n] = linear_epilogue(acc[i], bias, p, r, z, n);
         }
     }
 }
@@ -360,9 +334,7 @@ __global__ void __launch_bounds__(256) linear_tile_kernel(LinearF32Params p) {
         for (int j = 0; j < 4; ++j) {
             const uint32_t n = n0 + tx * 4 + j;
             if (n >= p.n) continue;
-            float v = apply_token_mul(apply_tail(apply_act(acc[i][j] + (p.bias ? bf16_to_f32(p.bias[n]) : 0.0f), p.act), p, r, z), p, r, n);
-            if (p.residual) v += p.residual[(size_t)r * p.ldr + n];
-            y[(size_t)r * p.ldy + n] = v;
+            y[(size_t)r * p.ldy + n] = linear_epilogue(acc[i][j], p.bias ? bf16_to_f32(p.bias[n]) : 0.0f, p, r, z, n);
         }
     }
 }
@@ -441,6 +413,76 @@ __global__ void __launch_bounds__(64) moe_route_scores_kernel(const float* x, co
     }
 }
 
+// ---- grouped sigmoid routing: a workgroup per row; the waves share the router's outputs (or the logits are there already), wave 0 chooses
+__global__ void __launch_bounds__(1024) moe_route_groups_kernel(RouteGroupsParams p, uint32_t staged) {
+    extern __shared__ float s_mem[]; // [outputs] scores | [outputs] choice scores | [groups] strengths | [d] the row (staged)
+    float *s_score = s_mem, *s_choice = s_mem + p.outputs, *s_strength = s_choice + p.outputs, *s_x = s_strength + p.groups;
+    const uint32_t r = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
+    const float* xr = p.x + (size_t)r * p.d;
+    if (staged) {
+        for (uint32_t i = tid; i < p.d; i += blockDim.x) s_x[i] = opnd(xr[i], p.bf16_products);
+        __syncthreads();
+    }
+    for (uint32_t e = p.logits ? tid : wave; e < p.outputs; e += p.logits ? blockDim.x : nw) {
+        float z;
+        if (p.logits) z = p.logits[(size_t)r * p.outputs + e];
+        else if (staged) z = wave_sum(lane_dot(s_x, p.router + (size_t)e * p.d, p.d, lane));
+        else z = wave_sum(lane_dot(xr, p.router + (size_t)e * p.d, p.d, lane, p.bf16_products));
+        const float sc = 1.0f / (1.0f + expf(-z));
+        if (p.logits || lane == 0) s_score[e] = sc, s_choice[e] = sc + (p.selection_bias ? p.selection_bias[e] : 0.0f);
+    }
+    __syncthreads();
+    const uint32_t size = p.outputs / p.groups;
+    if (p.keep < p.groups) { // thread = group: the sum of its two largest choice scores, then its rank among the groups
+        for (uint32_t g = tid; g < p.groups; g += blockDim.x) {
+            float first = -INFINITY, second = -INFINITY;
+            for (uint32_t i = 0; i < size; ++i) {
+                const float c = s_choice[g * size + i];
+                if (c > first) second = first, first = c;
+                else second = fmaxf(second, c);
+            }
+            s_strength[g] = size > 1 ? first + second : first;
+        }
+        __syncthreads();
+        for (uint32_t g = tid; g < p.groups; g += blockDim.x) {
+            uint32_t stronger = 0;
+            for (uint32_t o = 0; o < p.groups; ++o) stronger += (s_strength[o] > s_strength[g] || (s_strength[o] == s_strength[g] && o < g)) ? 1u : 0u;
+            if (stronger >= p.keep)
+                for (uint32_t i = 0; i < size; ++i) s_choice[g * size + i] = -INFINITY;
+        }
+        __syncthreads();
+    }
+    if (wave) return;
+    float choice[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) choice[j] = j * 64 + lane < p.outputs ? s_choice[j * 64 + lane] : -INFINITY;
+    float sum = 0.0f, my_s = 0.0f; // lane t keeps the t-th winner
+    int32_t my_id = 0;
+    for (uint32_t t = 0; t < p.top; ++t) {
+        float best = -INFINITY;
+        uint32_t best_e = 0xFFFFFFFFu;
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (choice[j] > best) best = choice[j], best_e = j * 64 + lane;
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const float ob = __shfl_xor(best, off, 64);
+            const uint32_t oe = __shfl_xor(best_e, off, 64);
+            if (ob > best || (ob == best && oe < best_e)) best = ob, best_e = oe;
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if ((uint32_t)j * 64 + lane == best_e) choice[j] = -INFINITY;
+        const float sc = best_e < p.outputs ? s_score[best_e] : 0.0f; // (a row of NaNs has no winner: id -1, which every consumer passes over)
+        sum += sc;
+        if (t == lane) my_s = sc, my_id = (int32_t)best_e;
+    }
+    if (lane < p.top) {
+        p.ids[(size_t)r * p.top + lane] = my_id;
+        p.weights[(size_t)r * p.top + lane] = my_s / (sum + 1e-20f) * p.scale;
+    }
+}
+
 // a workgroup per (row, slot): the row once into LDS, then a wave per hidden unit (gate and up rows of the unit in the same pass)
 __global__ void __launch_bounds__(256) moe_experts_gate_up_kernel(const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t d, uint32_t ff, uint32_t routed,
                                                                   uint32_t top, uint32_t bf16_products, ExpertAct act) {
@@ -451,8 +493,13 @@ __global__ void __launch_bounds__(256) moe_experts_gate_up_kernel(const float* x
     for (uint32_t i = threadIdx.x; i < d; i += blockDim.x) s_x[i] = opnd(x[(size_t)r * d + i], bf16_products);
     __syncthreads();
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
-    const uint16_t* base = w13 + (size_t)e * 2 * ff * d;
+    const uint16_t* base = w13 + (size_t)e * (act.plain ? 1 : 2) * ff * d;
     for (uint32_t f = blockIdx.y * nw + wave; f < ff; f += gridDim.y * nw) {
+        if (act.plain) { // no gate rows
+            const float v = fmaxf(wave_sum(lane_dot(s_x, base + (size_t)f * d, d, lane)), 0.0f);
+            if (lane == 0) hidden[(size_t)slot * ff + f] = v * v;
+            continue;
+        }
         const uint16_t* wu = base + (size_t)f * d;
         const uint16_t* wg = base + (size_t)(ff + f) * d;
         const float au = wave_sum(lane_dot(s_x, wu, d, lane)), ag = wave_sum(lane_dot(s_x, wg, d, lane));
@@ -554,7 +601,8 @@ __global__ void __launch_bounds__(256) moe_combine_kernel(const float* y2, const
 bool moe_experts_grouped_supported(const MoeGroupedParams& p) {
     if (!p.routed || p.rows < 64 || p.routed > 8192 || !p.y1 || !p.y2 || !p.hidden || !p.perm) return false;
     LinearF32Params q{};
-    q.x = p.x, q.w = p.w13, q.y = p.y1, q.rows = p.rows * p.top, q.n = 2 * p.ff, q.k = p.d, q.ldx = p.d, q.ldy = 2 * p.ff, q.batch = p.routed, q.w_batch = (size_t)2 * p.ff * p.d;
+    const uint32_t n1 = p.act.plain ? p.ff : 2 * p.ff;
+    q.x = p.x, q.w = p.w13, q.y = p.y1, q.rows = p.rows * p.top, q.n = n1, q.k = p.d, q.ldx = p.d, q.ldy = n1, q.batch = p.routed, q.w_batch = (size_t)n1 * p.d;
     q.bf16_products = 1, q.row_offsets = p.offsets, q.row_map = p.perm;
     LinearF32Params r = q;
     r.x = p.hidden, r.w = p.w2, r.y = p.y2, r.n = p.d, r.k = p.ff, r.ldx = p.ff, r.ldy = p.d, r.w_batch = (size_t)p.d * p.ff, r.row_map = nullptr;
@@ -568,10 +616,12 @@ uzu_status moe_experts_grouped(hipStream_t s, const MoeGroupedParams& p) {
     UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_scatter_kernel, dim3((slots + 255) / 256), dim3(256), 0, s, p.ids, slots, p.routed, p.top, p.offsets, p.cursor, p.perm, p.slot_pos); },
                                "moe_scatter"));
     LinearF32Params q{};
-    q.x = p.x, q.w = p.w13, q.y = p.y1, q.rows = slots, q.n = 2 * p.ff, q.k = p.d, q.ldx = p.d, q.ldy = 2 * p.ff, q.batch = p.routed, q.w_batch = (size_t)2 * p.ff * p.d;
+    const uint32_t n1 = p.act.plain ? p.ff : 2 * p.ff;
+    q.x = p.x, q.w = p.w13, q.y = p.y1, q.rows = slots, q.n = n1, q.k = p.d, q.ldx = p.d, q.ldy = n1, q.batch = p.routed, q.w_batch = (size_t)n1 * p.d;
     q.bf16_products = 1, q.row_offsets = p.offsets, q.row_map = p.perm;
+    if (p.act.plain) q.y = p.hidden, q.act = 1; // no gate: the activation rides in the product's epilogue
     UZU_PROPAGATE(linear_mfma(s, q));
-    UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_act_mul_kernel, dim3(slots), dim3(256), 0, s, p.y1, p.hidden, p.offsets, p.routed, p.ff, p.act); }, "moe_act_mul"));
+    if (!p.act.plain) UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_act_mul_kernel, dim3(slots), dim3(256), 0, s, p.y1, p.hidden, p.offsets, p.routed, p.ff, p.act); }, "moe_act_mul"));
     LinearF32Params r{};
     r.x = p.hidden, r.w = p.w2, r.y = p.y2, r.rows = slots, r.n = p.d, r.k = p.ff, r.ldx = p.ff, r.ldy = p.d, r.batch = p.routed, r.w_batch = (size_t)p.d * p.ff;
     r.bf16_products = 1, r.row_offsets = p.offsets;
@@ -680,6 +730,19 @@ uzu_status moe_route_topk(hipStream_t s, const float* x, const uint16_t* router,
     UZU_UNSUPPORTED(outputs > kRouteMaxOutputs || top > 64 || top > outputs || !top, "moe_route_topk: at most %u router outputs and 64 winners (got %u, %u)", kRouteMaxOutputs, outputs, top);
     return launch_check([&] { hipLaunchKernelGGL(moe_route_scores_kernel, dim3(rows), dim3(64), 0, s, x, router, (const float*)nullptr, ids, weights, d, outputs, top, renorm ? 2u : 1u, router_bias); },
                         "moe_route_topk");
+}
+
+uzu_status moe_route_groups(hipStream_t s, const RouteGroupsParams& p) {
+    if (!p.rows) return UZU_OK;
+    UZU_REQUIRE(p.x && (p.router || p.logits) && p.ids && p.weights && p.d, "moe_route_groups: null argument");
+    UZU_UNSUPPORTED(p.outputs > kRouteMaxOutputs || p.top > 64 || !p.top, "moe_route_groups: at most %u router outputs and 64 winners (got %u, %u)", kRouteMaxOutputs, p.outputs, p.top);
+    UZU_REQUIRE(p.groups && p.outputs % p.groups == 0 && p.keep && p.keep <= p.groups && p.top <= p.outputs / p.groups * p.keep, "moe_route_groups: %u winners among %u of %u groups of %u outputs",
+                p.top, p.keep, p.groups, p.outputs);
+    const uint32_t staged = !p.logits && (size_t)p.d * 4 <= 40 * 1024 ? 1u : 0u;
+    const size_t lds = ((size_t)2 * p.outputs + p.groups + (staged ? p.d : 0)) * 4;
+    // with the logits at hand one wave per row will do; without them the outputs' dot products are spread over sixteen
+    const uint32_t threads = p.logits ? 64 : p.outputs <= 4 ? 256 : 1024;
+    return launch_check([&] { hipLaunchKernelGGL(moe_route_groups_kernel, dim3(p.rows), dim3(threads), lds, s, p, staged); }, "moe_route_groups");
 }
 
 uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed,

@@ -9,6 +9,7 @@
 //   k_gated_lru.hip          the gated linear recurrent unit: short causal convolution over a carried window, gates / decays / state update
 //   k_causal_conv.hip        a causal per-channel convolution of row blocks over a carried window (sublayer inputs, the delta rule's q / k / v), per-head norm + gate
 //   k_channel_delta.hip      the gated delta rule with a decay per head and key channel
+//   k_hyper.hip              hyper-connections: join a sublayer's result to the copies of the stream, read + norm (+ input convolution) the next sublayer's row
 #pragma once
 
 #include <hip/hip_runtime.h>
@@ -84,7 +85,7 @@ uzu_status depth_mix(hipStream_t s, const float* slots, size_t slot_stride, cons
 
 // Y[z][r, n] = act(sum_k X[z][r, k] * W[z][n, k] + bias[n]) + residual[r, n]        z < batch (grid.z): a batch of independent products of one shape
 //   X[z] = x + z * x_batch (row pitch ldx), W[z] = w + z * w_batch ([n, k] bf16), Y[z] = y + z * y_batch (row pitch ldy)
-//   act: 0 none, 1 max(.,0)^2, 2 gelu (tanh form).  residual (pitch ldr, only with batch == 1) may alias y.
+//   act: 0 none, 1 max(.,0)^2, 2 gelu (tanh form), 3 xIELU (v > 0: act_a v^2 + v / 2, else act_b (e^v - 1 - v) + v / 2).  residual (pitch ldr, only with batch == 1) may alias y.
 struct LinearF32Params {
     const float* x;
     const uint16_t* w;
@@ -99,8 +100,11 @@ struct LinearF32Params {
     uint32_t bf16_products;
     float y_scale;     // != 0: the product (behind bias and act, before the residual) is multiplied by it
     float soft_cap;    // != 0: ... and then capped, cap * tanh(v / cap) (the read-out's logit cap)
-    const float* gate; // batched products: product z of row r is multiplied by sigmoid(gate[r * ldgate + z]) (a scalar gate per head); null = none
-    uint32_t ldgate;
+    float act_a, act_b; // act 3
+    // batched products: product z of row r is multiplied by sigmoid(gate[r * ldgate + z]) (a scalar gate per head) or, with gate_batch != 0, element by element by
+    // sigmoid(gate[r * ldgate + z * gate_batch + n]); null = none
+    const float* gate;
+    uint32_t ldgate, gate_batch;
     // a multiplier per (row's token, column) behind all of that: y[r, n] *= f32(mul_table[token[r] * mul_ld + mul_col0 + n])  (bf16 table, an id >= mul_vocab reads
     // row 0; one product per launch; null = none) -- the gate of a per-layer token input
     const uint16_t* mul_table;
@@ -126,12 +130,28 @@ uzu_status moe_route_scores(hipStream_t s, const float* x, const uint16_t* route
 // winners' logits (renorm != 0) or the logits themselves.  ids / weights [rows, top], winners by falling logit.
 uzu_status moe_route_topk(hipStream_t s, const float* x, const uint16_t* router, const uint16_t* router_bias, int32_t* ids, float* weights, uint32_t rows, uint32_t d,
                           uint32_t outputs, uint32_t top, uint32_t renorm);
+// Grouped sigmoid routing: per row s = sigmoid(router x) in f32 (bf16_products: x rounded to bf16 first), choice scores c = s + selection_bias (f32 [outputs] or null).  The outputs form
+// `groups` equal groups of neighbours; a group's strength is the sum of its two largest c (of its one, if it has one); only outputs of the `keep` strongest groups
+// can be chosen (ties: the lower group).  The `top` largest c among them win (ties: the lower index); weights = s / (sum of the winners' s + 1e-20) * scale.
+// logits (f32 [rows][outputs] or null): router x as the caller has computed it (many rows: one matrix product); null: the launch computes it.
+struct RouteGroupsParams {
+    const float* x;
+    const float* logits;
+    const uint16_t* router;
+    const float* selection_bias;
+    int32_t* ids;
+    float* weights;
+    uint32_t rows, d, outputs, top, groups, keep, bf16_products;
+    float scale;
+};
+uzu_status moe_route_groups(hipStream_t s, const RouteGroupsParams& p);
 // The gated product of an expert's hidden unit: g = clamp(gate, gate_min, gate_max), u = clamp(up, up_min, up_max), g * sigmoid(alpha * g) * (u + up_offset).
 // The default is silu(gate) * up.
 // gelu != 0: the gate's activation is the tanh form of gelu instead of g * sigmoid(alpha * g).
+// plain != 0: no gate, max(up, 0)^2 -- w13 then holds [ff][d] per expert.
 struct ExpertAct {
     float alpha = 1.0f, gate_min = -INFINITY, gate_max = INFINITY, up_min = -INFINITY, up_max = INFINITY, up_offset = 0.0f;
-    uint32_t gelu = 0;
+    uint32_t gelu = 0, plain = 0;
 };
 // The gated product of a dense block: hidden[r, f] = act(gate = y1[r, ff + f], up = y1[r, f])   (y1 f32 [rows][2 ff]: up rows first, as the packed projection yields them)
 uzu_status gated_act_rows(hipStream_t s, const float* y1, float* hidden, uint32_t rows, uint32_t ff, const ExpertAct& act);
@@ -203,7 +223,12 @@ constexpr uint32_t kLatentMaxRank = 2048;
 // row t of the sequence's cache (width rank + rope_dim, bf16 or f32).  Every query head's rotated part turns the same way and lands in
 // qlat[r, head, rank .. rank + rope_dim) (qlat f32 [rows][heads][rank + rope_dim]; the first rank columns of a head are filled by the folded key projection).
 // rope_dim == 0: normalisation + append alone.
+// q_rank != 0: the row's first q_rank numbers (column 0) are a query latent, not queries: its RMS norm (q_scales, eps) goes to q_latent[r, :] (f32 [rows][q_rank]) and
+// qlat must be null -- the queries are turned by a second launch over their own rows (caches null).
 struct LatentRopeAppendParams {
+    uint32_t q_rank;
+    const float* q_scales;
+    float* q_latent;
     const float* x;
     uint32_t ldx, c_col, rank, rope_dim;
     const float* scales;
@@ -285,6 +310,38 @@ struct WindowAttentionParams {
 size_t window_attention_split_ws_bytes(uint32_t rows, uint32_t heads, uint32_t splits);
 bool window_attention_mfma_supported(const WindowAttentionParams& p);
 uzu_status window_attention(hipStream_t s, const WindowAttentionParams& p);
+
+// Hyper-connections.  The residual stream is `streams` = s copies x_a of every row (copy a at src + a * src_stride, rows of width d).  Per row, in this order:
+//   join (y != null):  x_b <- sum_a mix[a, b] x_a + mult * out[b] * y       all from the old ones; stored at dst + b * dst_stride (dst may be src; null: not stored)
+//   sum_out (or null): sum_a x_a
+//   read (h != null):  u = sum_a read[a] x_a (read null: the plain sum),  h[r, :] = u / sqrt(mean(u^2) + eps) * (scales + offset)
+//   conv_w (or null; only where every sequence of the pass brings one row): h <- h + conv(h), the causal convolution of causal_conv_rows over the sequence's window
+//                      (states[z] + state_offset, f32 [taps - 1][d]), which moves on by this row's h
+// join = f32 [s | s | s s]: in | out | mix[from, to] of the sublayer that yielded y; read = in of the sublayer that follows.  src_stride 0: all copies equal the one
+// row (the embedding rows).  row_index: row r of `h` is row row_index[r] of the stream.
+struct HyperStepParams {
+    const float* src;
+    float* dst;
+    size_t src_stride, dst_stride;
+    const float* y;
+    const float* join;
+    float mult;
+    float* sum_out;
+    const float* read;
+    float* h;
+    const float* scales;
+    float offset, eps;
+    const uint32_t* row_index;
+    uint32_t rows, d, streams;
+    const float* conv_w;
+    uint32_t taps;
+    float* const* states;
+    size_t state_offset;
+    const SeqSpan* spans;
+    const uint32_t* row_seq;
+};
+constexpr uint32_t kHyperMaxStreams = 16, kHyperMaxWidth = 32768;
+uzu_status hyper_step(hipStream_t s, const HyperStepParams& p);
 
 // Retention.  Row r (sequence z, position t), head a, with q, k [heads][dim] and v [heads][vdim] taken from the f32 rows `qkv` (pitch ld; columns q_col, k_col,
 // v_col; q and k rotated and k scaled already):   S <- decay[a] S + k v^T,   out[r, a, :] = S^T q.

@@ -17,10 +17,10 @@ import numpy as np
 
 # enums (uzu_model_desc.h)
 QUANT_SCALE_BIAS, QUANT_SCALE_ZERO_POINT, QUANT_SCALE_SYMMETRIC, QUANT_NONE = 0, 1, 2, 3
-ACT_SILU, ACT_GELU_APPROX, ACT_GELU_EXACT, ACT_IDENTITY, ACT_SOFTPLUS, ACT_RELU_SQUARED = 0, 1, 2, 3, 4, 5
+ACT_SILU, ACT_GELU_APPROX, ACT_GELU_EXACT, ACT_IDENTITY, ACT_SOFTPLUS, ACT_RELU_SQUARED, ACT_XIELU = 0, 1, 2, 3, 4, 5, 6
 MIXER_ATTENTION, MIXER_DELTA_NET, MIXER_LATENT_ATTENTION, MIXER_RETENTION, MIXER_GATED_LRU = 0, 1, 2, 3, 4
 NORM_STATISTICS, NORM_DYNAMIC_TANH, NORM_RMS_SCALAR = 0, 1, 2
-MOE_ROUTE_TOPK_LOGITS, MOE_ROUTE_SCORES = 0, 1
+MOE_ROUTE_TOPK_LOGITS, MOE_ROUTE_SCORES, MOE_ROUTE_SIGMOID_GROUPS = 0, 1, 2
 ROPE_NONE, ROPE_UNSCALED, ROPE_LLAMA, ROPE_LINEAR, ROPE_YARN, ROPE_LONGROPE = 0, 1, 2, 3, 4, 5
 
 
@@ -63,7 +63,8 @@ class MoeDesc(C.Structure):
         ("gate_clip_min", C.c_float), ("gate_clip_max", C.c_float), ("up_clip_min", C.c_float), ("up_clip_max", C.c_float),
         ("router_weights", C.c_void_p), ("router_biases", C.c_void_p), ("w13", C.c_void_p), ("w2", C.c_void_p), ("up_biases", C.c_void_p), ("down_biases", C.c_void_p),
         ("routing", C.c_uint32), ("num_identity_experts", C.c_uint32), ("selection_bias", C.c_void_p),
-        ("up_offset", C.c_float), ("reserved", C.c_uint32),
+        ("up_offset", C.c_float), ("plain_experts", C.c_uint32),
+        ("router_groups", C.c_uint32), ("router_groups_keep", C.c_uint32), ("router_scale", C.c_float), ("reserved", C.c_uint32),
     ]
 
 
@@ -109,6 +110,8 @@ class LayerDesc(C.Structure):
         ("rel_bias", C.c_void_p), ("head_temperature", C.c_void_p),
         ("pair_mixer", C.c_uint32), ("pair_scale_main", C.c_float), ("pair_scale_second", C.c_float),
         ("dn_channel_decay", C.c_uint32), ("dn_decay_rank", C.c_uint32), ("dn_gate_rank", C.c_uint32), ("dn_decay_up", LinearDesc), ("dn_gate_up", LinearDesc),
+        ("latent_query_rank", C.c_uint32), ("gate_elementwise", C.c_uint32), ("latent_query_norm", NormDesc), ("latent_query_up", LinearDesc),
+        ("xielu_p", C.c_float), ("xielu_q", C.c_float), ("hyper_mixer", C.c_void_p), ("hyper_mlp", C.c_void_p),
     ]
 
 
@@ -129,6 +132,7 @@ class ModelDesc(C.Structure):
         ("ple_model_projection_scale", C.c_float), ("ple_input_scale", C.c_float), ("reserved", C.c_uint32),
         ("ple_token_embedding", LinearDesc), ("ple_model_projection", LinearDesc), ("ple_projection_norm", NormDesc),
         ("f32_stream", C.c_uint32), ("bigram_buckets", C.c_uint32), ("bigram_mul_prev", C.c_uint32), ("bigram_mul_cur", C.c_uint32), ("bigram_table", LinearDesc),
+        ("hyper_streams", C.c_uint32), ("residual_mult", C.c_float),
     ]
 
 
@@ -247,12 +251,17 @@ class MoeWeights:
     num_identity_experts: int = 0
     selection_bias: Optional[np.ndarray] = None  # f32 [E + identity]
     up_offset: float = 0.0       # expert = down(act(gate) * (up + up_offset))
+    plain_experts: bool = False  # an expert without a gate, down(max(up x, 0)^2): w13 is [E, d_ff, model_dim]
+    # grouped sigmoid routing (MOE_ROUTE_SIGMOID_GROUPS): choice among the experts of the strongest groups by sigmoid score + selection_bias, weights = scores / sum * scale
+    router_groups: int = 1
+    router_groups_keep: int = 1
+    router_scale: float = 1.0
 
     def desc(self) -> MoeDesc:
         return MoeDesc(self.num_routed_experts, self.num_active_experts, self.expert_hidden_dim, int(self.router_renorm), self.gating_sel, self.silu_alpha,
                        self.gate_clip[0], self.gate_clip[1], self.up_clip[0], self.up_clip[1], _ptr(self.router_weights), _ptr(self.router_biases), _ptr(self.w13),
                        _ptr(self.w2), _ptr(self.up_biases), _ptr(self.down_biases), int(self.routing), int(self.num_identity_experts), _ptr(self.selection_bias),
-                       float(self.up_offset), 0)
+                       float(self.up_offset), int(self.plain_experts), int(self.router_groups), int(self.router_groups_keep), float(self.router_scale), 0)
 
     def nbytes_active(self) -> int:
         """bytes one decoded token streams: the router + the k active experts' matrices and biases"""
@@ -365,13 +374,21 @@ class LayerWeights:
     dn_channel_decay: bool = False
     dn_decay_up: Optional[LinearWeights] = None    # [heads dk, rank]
     dn_gate_up: Optional[LinearWeights] = None     # [heads dv, rank]
+    # latent attention whose queries go through a latent of their own (packed projection rows: query down | down projection | gates), a gate per coordinate
+    latent_query_norm: NormWeights = field(default_factory=lambda: ABSENT_NORM)
+    latent_query_up: Optional[LinearWeights] = None  # [heads (head_dim + rope), query rank]
+    gate_elementwise: bool = False
+    xielu: tuple = (0.0, 0.0)                      # (p, q) of a plain dense MLP with ACT_XIELU
+    # hyper-connections (ModelBundle.hyper_streams = s): f32 [s + s + s s] = in | out | mix[from, to] of each sublayer
+    hyper_mixer: Optional[np.ndarray] = None
+    hyper_mlp: Optional[np.ndarray] = None
 
     def _moe_desc(self) -> MoeDesc:
         if self.moe is not None:
             return self.moe.desc()
         if self.gated_act is not None:
             slope, gate, up, off = self.gated_act
-            return MoeDesc(0, 0, 0, 0, 2, float(slope), float(gate[0]), float(gate[1]), float(up[0]), float(up[1]), None, None, None, None, None, None, 0, 0, None, float(off), 0)
+            return MoeDesc(0, 0, 0, 0, 2, float(slope), float(gate[0]), float(gate[1]), float(up[0]), float(up[1]), None, None, None, None, None, None, 0, 0, None, float(off), 0, 0, 0, 0.0, 0)
         return MoeDesc()
 
     def desc(self) -> LayerDesc:
@@ -410,11 +427,13 @@ class LayerWeights:
             0 if self.pair_mixer is None else int(self.pair_mixer) + 1, float(self.pair_scales[0]), float(self.pair_scales[1]),
             int(self.dn_channel_decay), 0 if self.dn_decay_up is None else int(self.dn_decay_up.k), 0 if self.dn_gate_up is None else int(self.dn_gate_up.k),
             ld(self.dn_decay_up), ld(self.dn_gate_up),
+            0 if self.latent_query_up is None else int(self.latent_query_up.k), int(self.gate_elementwise), self.latent_query_norm.desc(), ld(self.latent_query_up),
+            float(self.xielu[0]), float(self.xielu[1]), _ptr(self.hyper_mixer), _ptr(self.hyper_mlp),
         )
 
     def linears(self):
         names = ("qkv_projection", "gate_projection", "out_projection", "dn_in_proj", "dn_out_proj", "up_projection",
-                 "down_projection", "latent_down", "latent_up_keys", "latent_up_values", "stream_reentry", "dn_decay_up", "dn_gate_up")
+                 "down_projection", "latent_down", "latent_up_keys", "latent_up_values", "stream_reentry", "dn_decay_up", "dn_gate_up", "latent_query_up")
         out = [(n, getattr(self, n)) for n in names if getattr(self, n) is not None]
         if self.ple is not None:
             out += [("ple.gate", self.ple.gate), ("ple.projection", self.ple.projection)]
@@ -579,6 +598,8 @@ class ModelBundle:
     side_dim: int = 0
     bigram: Optional[LinearWeights] = None       # f32-stream designs: a hashed (previous token, token) table [buckets + 1, model_dim] added to the embedding rows
     bigram_mul: tuple = (0, 0)                   # (multiplier of the previous token, of the token)
+    hyper_streams: int = 0                       # f32-stream designs: the residual stream is that many copies joined by hyper-connections (LayerWeights.hyper_*)
+    residual_mult: float = 1.0                   # ... and a sublayer's result is multiplied by it
     _keep: list = field(default_factory=list, repr=False)
 
     def desc(self) -> ModelDesc:
@@ -595,7 +616,7 @@ class ModelBundle:
             return ModelDesc(self.vocab_size, self.model_dim, len(self.layers), int(self.tied_embeddings), self.input_scale, self.logit_scale, self.logit_soft_cap,
                              self.max_context_length, self.rope.desc(), self.embedding.desc(), out_emb, self.output_norm.desc(), C.cast(arr, C.POINTER(LayerDesc)),
                              len(self.ropes) if self.ropes else 0, 1, C.cast(ropes, C.POINTER(RopeDesc)) if ropes is not None else None, self.embedding_norm.desc(),
-                             int(self.side_dim), int(self.side_table.n), 1.0, 0.0, 0.0, 0, self.side_table.desc(), e, ABSENT_NORM.desc(), int(self.f32_stream), *self._bigram_desc())
+                             int(self.side_dim), int(self.side_table.n), 1.0, 0.0, 0.0, 0, self.side_table.desc(), e, ABSENT_NORM.desc(), int(self.f32_stream), *self._stream_tail_desc())
         return ModelDesc(self.vocab_size, self.model_dim, len(self.layers), int(self.tied_embeddings),
                          self.input_scale, self.logit_scale, self.logit_soft_cap, self.max_context_length,
                          self.rope.desc(), self.embedding.desc(), out_emb, self.output_norm.desc(),
@@ -606,12 +627,13 @@ class ModelBundle:
                          p.ple_dim if p else 0, p.ple_vocab_size if p else 0, p.ple_embed_scale if p else 0.0,
                          p.model_projection_scale if p else 0.0, p.input_scale if p else 0.0, 0,
                          p.token_embedding.desc() if p else e, p.model_projection.desc() if p else e,
-                         (p.projection_norm if p else ABSENT_NORM).desc(), int(self.f32_stream), *self._bigram_desc())
+                         (p.projection_norm if p else ABSENT_NORM).desc(), int(self.f32_stream), *self._stream_tail_desc())
 
-    def _bigram_desc(self):
+    def _stream_tail_desc(self):
+        hyper = (int(self.hyper_streams), float(self.residual_mult))
         if self.bigram is None:
-            return 0, 0, 0, LinearDesc()
-        return int(self.bigram.n) - 1, int(self.bigram_mul[0]), int(self.bigram_mul[1]), self.bigram.desc()
+            return (0, 0, 0, LinearDesc()) + hyper
+        return (int(self.bigram.n) - 1, int(self.bigram_mul[0]), int(self.bigram_mul[1]), self.bigram.desc()) + hyper
 
     # ---- algorithmic bytes per decoded token (SURVEY.md §8d formula) ----
     def weight_stream_bytes(self) -> int:
@@ -639,8 +661,6 @@ class ModelBundle:
                     total += 2 * l.dn_num_heads * l.dn_value_head_dim * l.dn_head_dim * 4
                     conv_dim = 2 * l.dn_num_groups * l.dn_head_dim + l.dn_num_heads * l.dn_value_head_dim
                     total += conv_dim * (3 * l.dn_kernel_size - 2) * 4
-                if l.input_conv_taps:  # the sublayers' input convolutions: window read + write, taps
-                    total += 2 * self.model_dim * (3 * l.input_conv_taps - 2) * 4
             elif l.mixer_kind == MIXER_RETENTION:
                 total += 2 * l.num_heads * l.head_dim * l.value_head_dim * 4  # f32 state read + write
             elif l.mixer_kind == MIXER_LATENT_ATTENTION:
@@ -654,6 +674,8 @@ class ModelBundle:
                 conv_dim = 2 * l.dn_num_groups * l.dn_head_dim + l.dn_num_heads * l.dn_value_head_dim
                 total += 2 * conv_dim * (l.dn_kernel_size - 1) * 4            # conv state read + write
                 total += conv_dim * l.dn_kernel_size * 4                      # conv taps
+            if l.input_conv_taps:  # the sublayers' input convolutions: window read + write, taps
+                total += 2 * self.model_dim * (3 * l.input_conv_taps - 2) * 4
         return total
 
     def prefill_flops(self, tokens: int, context_before: int = 0) -> float:
@@ -665,7 +687,7 @@ class ModelBundle:
                 macs += w.n * w.k
             if l.moe is not None:  # router for every token + the k active experts' up | gate and down matrices
                 mo = l.moe
-                macs += mo.num_routed_experts * self.model_dim + mo.num_active_experts * 3 * mo.expert_hidden_dim * self.model_dim
+                macs += mo.num_routed_experts * self.model_dim + mo.num_active_experts * (2 if mo.plain_experts else 3) * mo.expert_hidden_dim * self.model_dim
         flops = 2.0 * tokens * macs
         readout = self.embedding if self.tied_embeddings else self.output_embedding
         flops += 2.0 * readout.n * readout.k
