@@ -12,7 +12,7 @@ Prints ONE JSON line on rank 0 with two extra o
   roofline     -- the dominant kernel (the int4 GEMV family) : algorithmic bytes / HIP-event time, vs 8 TB/s HBM
   cpu_baseline -- the CPU oracle (port of the reference's single-threaded CPU backend) timed on this host
 
-Side runs (their own JSON line, never the headline): --config c3|c4|c5, --exact, and --design lazolix | relulix | begasun | zovolorn (prefill / chained decode / batched
+Side runs (their own JSON line, never the headline): --config c3|c4|c5, --exact, and --design lazolix | relulix | begasun | zovolorn | dironex (prefill / chained decode / batched
 decode of an f32-stream design at real layer sizes beside the engine's closest existing model at equal sizes).
 """
 import argparse
@@ -59,12 +59,13 @@ def parse_args():
                     help="BASELINE.json configs[1..4]: c2 (default, the headline) Qwen3.5-0.8B int4 ctx-2048 decode; c3 Llama-3-8B int4, 4k prefill x 8 "
                          "sequences in batched passes (prefill tokens/s, MFMA roofline); c4 Llama-3-8B int8 decode (TP = --gpus); c5 Qwen3-14B-class int4 at "
                          "ctx 8192, one sequence decoding while another is prefilled (TP = --gpus)")
-    ap.add_argument("--design", choices=["", "lazolix", "relulix", "begasun", "zovolorn"], default="", help="side runs of a design outside BASELINE.json (never the headline): `lazolix` times prefill, "
+    ap.add_argument("--design", choices=["", "lazolix", "relulix", "begasun", "zovolorn", "dironex"], default="", help="side runs of a design outside BASELINE.json (never the headline): `lazolix` times prefill, "
                     "chained decode and batched decode of the f32-stream design at layer sizes of real models (random weights), beside the closest "
                     "bf16-stream model of the engine at equal sizes (windowed attention with sinks + int4 dense / bf16 expert MLPs); `relulix` does the same for the "
                     "design of parallel blocks with rotated attention, retention layers and clamped experts, beside Lazolix with experts at equal sizes; `begasun` for the looped stack of recurrent units, latent attention with a rotated key part "
                     "and grouped attention, beside Lazolix with dense blocks at equal sizes; `zovolorn` for the pairs of chunked attention + channel-decay delta rule alternating with grouped attention, "
-                    "beside Begasun's recurrent units alternating with grouped attention at equal sizes")
+                    "beside Begasun's recurrent units alternating with grouped attention at equal sizes; `dironex` for hyper-connected latent attention (a query latent, a rotated key part) and windowed grouped "
+                    "attention with xIELU dense blocks and ungated experts, beside Lazolix with the same pattern of dense blocks and experts at equal sizes")
     ap.add_argument("--design-sizes", default="w1024,w2048", help="--design: comma-separated size presets")
     ap.add_argument("--sequences", type=int, default=8, help="c3: sequences per batched prefill pass")
     ap.add_argument("--prompt", type=int, default=4096, help="c3: prompt tokens per sequence")
@@ -676,8 +677,49 @@ def bench_zovolorn(args):
     print(json.dumps(out), flush=True)
 
 
+def bench_dironex(args):
+    """Prefill / decode throughput of Dironex models (three latent-attention layers and a windowed grouped-attention layer, dense blocks alternating with routed experts;
+    four copies of the stream, four convolution taps in front of every sublayer) beside the closest existing model at equal size: Lazolix with the same pattern of plain
+    dense blocks and routed experts (norms in front, latent attention; same width / heads / head widths / cache row width / dense width / experts / vocabulary / layer
+    count; an expert of Dironex has two matrices instead of three and 3 / 2 of the width: equal bytes).  One JSON line."""
+    import tempfile
+    from uzu_amd import dironex, lazolix, loader, synthetic as S
+    from uzu_amd.backend import Context
+    ctx = Context.new(0)
+    prompt_len, steps, warm, nbatch = 2048, max(8, min(args.steps, 128)), max(2, min(args.warmup, 8)), 8
+    out = {"metric": "dironex_side_run", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16 products, f32 stream", "data": "synthetic (random weights, synthetic token ids)",
+           "prompt_tokens": prompt_len, "decode_steps": steps, "batched_decode_sequences": nbatch, "sizes": {}}
+    for size in [s for s in args.design_sizes.split(",") if s]:
+        z = LAZOLIX_SIZES[size]
+        prompt = S.synthetic_prompt(prompt_len, z["vocab"]).astype(np.uint32)
+        context = prompt_len + steps + warm + 64
+        H, G, dim, vd, rot_dim, window = z["heads"], max(1, z["heads"] // 4), z["dim"], z["vdim"], 64, z["window"]
+        rank, q_rank = z["rank"] - rot_dim, z["width"] * 3 // 8  # the cache row [latent | rotated part] is as wide as the closest model's latent
+        yarn = {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+        dense, moe = dironex.dense_mlp(z["ff"]), dironex.moe_mlp(z["experts"], z["top"], z["eff"] * 3 // 2, 2, 1, 2.5)
+        lat = lambda mlp: dironex.latent_attention_layer(H, dim, rot_dim, vd, rank, q_rank, dironex.rotation(rot_dim, 500000.0, yarn), mlp=mlp)
+        layers = ([lat(dense), lat(moe), dironex.attention_layer(H, G, dim, vd, window, mlp=dense), lat(moe)] * ((z["layers"] + 3) // 4))[:z["layers"]]
+        cfg = dironex.config(z["vocab"], z["width"], layers, taps=4, streams=4, residual_mult=0.5)
+        with tempfile.TemporaryDirectory() as tmp:
+            dironex.save(tmp, cfg, dironex.random_tensors(cfg, seed=1))
+            bundle = loader.load_model_dir(tmp, max_context_length=context)
+        lmlp = lambda l: lazolix.moe_mlp(z["experts"], z["top"], z["eff"], 0) if l % 2 else lazolix.dense_mlp(z["ff"])
+        lcfg = {"vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+                "layers": [lazolix.layer_config(H, dim, vd, z["rank"], window if l % 4 == 2 else None, mlp=lmlp(l)) for l in range(z["layers"])]}
+        with tempfile.TemporaryDirectory() as tmp:
+            lazolix.save(tmp, lcfg, lazolix.random_tensors(lcfg, seed=1))
+            closest = loader.load_model_dir(tmp, max_context_length=context)
+        rec = {"dironex": _time_f32_stream(ctx, bundle, prompt, steps, warm, nbatch), "closest": _time_f32_stream(ctx, closest, prompt, steps, warm, nbatch)}
+        out["sizes"][size] = {"shape": dict(z, kv_heads=G, kv_rank=rank, rot_dim=rot_dim, q_rank=q_rank, expert_ff=z["eff"] * 3 // 2, streams=4, taps=4,
+                                            pattern="latent + dense, latent + experts, windowed attention + dense, latent + experts", closest="Lazolix, the same pattern of feed-forwards"), **rec}
+    ctx.close()
+    print(json.dumps(out), flush=True)
+
+
 def main():
     args = parse_args()
+    if args.design == "dironex":
+        return bench_dironex(args)
     if args.design == "zovolorn":
         return bench_zovolorn(args)
     if args.design == "begasun":

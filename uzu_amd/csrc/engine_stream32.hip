@@ -419,17 +419,12 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             lp.x = h.latent_packed ? S.q : S.ckv, lp.ldx = h.latent_packed ? ldq : L.lat_down.n, lp.c_col = h.latent_packed ? c_col : 0, lp.rank = rank, lp.rope_dim = rd;
             lp.scales = L.lat_norm.scales, lp.eps = L.lat_norm.eps, lp.caches = h.is_kv_sharing ? nullptr : caches, lp.cache_bf16 = bf, lp.heads = H, lp.q_width = qw;
             lp.qlat = rd ? S.qlat : nullptr, lp.cosines = L.rope_cos, lp.sines = L.rope_sin, lp.interleaved = h.rope_interleaved, lp.spans = S.d_spans, lp.row_seq = S.d_row_seq, lp.rows = rows;
-            if (qr) { // cache rows and the query latent's norm; the queries of that latent; their rotated parts
+            if (qr) { // cache rows and the query latent's norm; the queries of that latent
                 k::LatentRopeAppendParams cp = lp;
                 cp.qlat = nullptr, cp.q_rank = qr, cp.q_scales = X.lat_q_norm.scales, cp.q_latent = S.ckv;
                 RUN("latent_rope_append", (size_t)rows * (kw * 6 + qr * 8), k::latent_rope_append(s, cp));
                 run_linear(e, lin(S, X.lat_q_up, S.ckv, S.lat_q, rows));
-                queries = S.lat_q, ldqueries = H * qw;
-                if (rd) {
-                    k::LatentRopeAppendParams qp = lp;
-                    qp.x = queries, qp.ldx = ldqueries, qp.c_col = 0, qp.caches = nullptr;
-                    RUN("latent_rope_append", (size_t)rows * H * rd * 8, k::latent_rope_append(s, qp));
-                }
+                queries = S.lat_q, ldqueries = H * qw; // (their rotated parts turn as the attention core loads them)
             } else if (h.latent_packed) { // the rotated query parts are read from the packed rows; a separate down projection leaves them in S.q as well
                 RUN("latent_rope_append", (size_t)rows * (kw * 6 + H * rd * 8), k::latent_rope_append(s, lp));
             } else {
@@ -453,6 +448,7 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             k::LatentAttentionParams ap{};
             ap.qlat = S.qlat, ap.out = S.ctx, ap.caches = caches, ap.cache_bf16 = bf, ap.sinks = X.sinks, ap.spans = S.d_spans, ap.row_seq = S.d_row_seq;
             ap.rows = rows, ap.heads = H, ap.rank = kw, ap.window = h.sliding_window_size;
+            if (qr && rd) ap.queries = queries, ap.ldqueries = ldqueries, ap.q_width = qw, ap.rope_dim = rd, ap.interleaved = h.rope_interleaved, ap.cosines = L.rope_cos, ap.sines = L.rope_sin;
             if (rd && rank % 4 == 0) ap.value_rank = rank; // the rotated columns score and carry no value
             ap.scale = h.attention_scale != 0.0f ? h.attention_scale : 1.0f / sqrtf((float)hd);
             ap.nseq = nseq;

@@ -49,6 +49,54 @@ __global__ void __launch_bounds__(256) causal_conv_rows_kernel(CausalConvParams 
     if (sp.count == 1 && p.taps > 1) window_update(p, sp, z, c);
 }
 
+// The same sums for many rows: thread = (four channels, kConvRows consecutive rows of the pass).  A channel's taps are loaded once, the last T - 1 input rows travel in
+// registers; a row in front of which its sequence has fewer rows in this pass takes the older inputs from the state (or zeros), as above.
+constexpr uint32_t kConvRows = 8;
+template <int T>
+__global__ void __launch_bounds__(256) causal_conv_block_kernel(CausalConvParams p) {
+    const uint32_t c = (blockIdx.x * 256 + threadIdx.x) * 4, r0 = blockIdx.y * kConvRows;
+    if (c >= p.channels) return;
+    const uint32_t r1 = r0 + kConvRows < p.rows ? r0 + kConvRows : p.rows;
+    const float* x = p.x + p.x_col + c;
+    float w[4][T];
+    f32x4_v past[T]; // past[b]: the input b rows back (past[0]: the row itself)
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < T; ++j) w[i][j] = p.w[((size_t)c + i) * T + j];
+    const f32x4_v zero{0.f, 0.f, 0.f, 0.f}, bias = p.bias ? f32x4_v{p.bias[c], p.bias[c + 1], p.bias[c + 2], p.bias[c + 3]} : zero;
+#pragma unroll
+    for (int b = 0; b < T; ++b) past[b] = b && r0 >= (uint32_t)b ? *(const f32x4_v*)(x + (size_t)(r0 - b) * p.ldx) : zero;
+#pragma unroll
+    for (uint32_t k = 0; k < kConvRows; ++k) {
+        const uint32_t r = r0 + k;
+        if (r >= r1) break;
+        past[0] = *(const f32x4_v*)(x + (size_t)r * p.ldx);
+        const uint32_t z = p.row_seq[r];
+        const SeqSpan sp = p.spans[z];
+        const uint32_t i = r - sp.row0, t = sp.start + i;
+        f32x4_v acc = bias;
+#pragma unroll
+        for (int j = 0; j < T; ++j) {
+            const uint32_t back = T - 1 - j;
+            f32x4_v in = past[back];
+            if (back > i) in = back <= t ? *(const f32x4_v*)(p.states[z] + p.state_offset + (size_t)(T - 1 - (back - i)) * p.channels + c) : zero;
+#pragma unroll
+            for (int q = 0; q < 4; ++q) acc[q] = fmaf(w[q][j], in[q], acc[q]);
+        }
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+            if (p.act == 1) acc[q] = acc[q] / (1.0f + expf(-acc[q]));
+            if (p.add_input) acc[q] = past[0][q] + acc[q];
+        }
+        *(f32x4_v*)(p.out + (size_t)r * p.ldo + p.o_col + c) = acc;
+        if (sp.count == 1 && T > 1)
+            for (uint32_t q = 0; q < 4; ++q) window_update(p, sp, z, c + q);
+#pragma unroll
+        for (int b = T - 1; b > 0; --b) past[b] = past[b - 1];
+    }
+}
+
 // thread = (sequence, channel): the windows of the sequences that bring several rows (their first rows' threads read the old window in the launch before)
 __global__ void __launch_bounds__(256) causal_conv_commit_kernel(CausalConvParams p) {
     const uint32_t z = blockIdx.x, c = blockIdx.y * 256 + threadIdx.x;
@@ -84,6 +132,21 @@ uzu_status causal_conv_rows(hipStream_t s, const CausalConvParams& p) {
     UZU_REQUIRE(p.x && p.out && p.w && (p.states || p.taps == 1) && p.spans && p.row_seq && p.channels && p.taps >= 1, "causal_conv: null argument");
     UZU_REQUIRE(p.x_col + p.channels <= p.ldx && p.o_col + p.channels <= p.ldo, "causal_conv: %u channels at columns %u / %u of rows of %u / %u", p.channels, p.x_col, p.o_col, p.ldx, p.ldo);
     UZU_REQUIRE(p.out != p.x || p.taps == 1, "causal_conv: a row reads earlier rows of the pass: the result goes to another block of rows");
+    const uintptr_t at = (uintptr_t)(p.x + p.x_col) | (uintptr_t)(p.out + p.o_col);
+    if (p.rows >= 64 && p.taps <= 6 && p.channels % 4 == 0 && p.ldx % 4 == 0 && p.ldo % 4 == 0 && p.state_offset % 4 == 0 && at % 16 == 0) {
+        const dim3 grid((p.channels / 4 + 255) / 256, (p.rows + kConvRows - 1) / kConvRows);
+        UZU_REQUIRE(grid.y <= 65535, "causal_conv: too many rows for one launch");
+#define UZU_CONV(T) case T: return launch_check([&] { hipLaunchKernelGGL(causal_conv_block_kernel<T>, grid, dim3(256), 0, s, p); }, "causal_conv_block")
+        switch (p.taps) {
+            UZU_CONV(1);
+            UZU_CONV(2);
+            UZU_CONV(3);
+            UZU_CONV(4);
+            UZU_CONV(5);
+            UZU_CONV(6);
+        }
+#undef UZU_CONV
+    }
     return launch_check([&] { hipLaunchKernelGGL(causal_conv_rows_kernel, dim3(p.rows, (p.channels + 255) / 256), dim3(256), 0, s, p); }, "causal_conv_rows");
 }
 

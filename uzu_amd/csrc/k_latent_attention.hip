@@ -39,7 +39,32 @@ __global__ void __launch_bounds__(256) latent_norm_append_kernel(const float* x,
     }
 }
 
-// a workgroup per row: wave 0 norms the latent and writes [latent | rotated key part] to the cache, all waves turn the query heads' rotated parts into qlat
+// a wave norms the n numbers at x: put(i, x_i / sqrt(mean(x^2) + eps) * scales_i).  Rows of up to 64 kNormAhead numbers stay in registers, every load in front of the first use
+constexpr int kNormAhead = 16;
+template <class Put> __device__ __forceinline__ void wave_rms_norm(const float* x, const float* scales, uint32_t n, float eps, uint32_t lane, Put put) {
+    float ss = 0.0f;
+    if (n <= 64 * kNormAhead) {
+        float v[kNormAhead], w[kNormAhead];
+#pragma unroll
+        for (int k = 0; k < kNormAhead; ++k) {
+            const uint32_t i = k * 64 + lane;
+            v[k] = i < n ? x[i] : 0.0f, w[k] = i < n ? scales[i] : 0.0f;
+        }
+#pragma unroll
+        for (int k = 0; k < kNormAhead; ++k) ss = fmaf(v[k], v[k], ss);
+        const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
+#pragma unroll
+        for (int k = 0; k < kNormAhead; ++k)
+            if (k * 64 + lane < n) put(k * 64 + lane, v[k] * inv * w[k]);
+        return;
+    }
+    for (uint32_t i = lane; i < n; i += 64) ss = fmaf(x[i], x[i], ss);
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + eps);
+    for (uint32_t i = lane; i < n; i += 64) put(i, x[i] * inv * scales[i]);
+}
+
+// a workgroup per row: wave 0 norms the latent, wave 1 the query latent, wave 2 turns the rotated key part, each to its place; all waves turn the query heads' rotated
+// parts into qlat
 __global__ void __launch_bounds__(256) latent_rope_append_kernel(LatentRopeAppendParams p) {
     const uint32_t r = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t q = p.row_seq[r];
@@ -53,19 +78,17 @@ __global__ void __launch_bounds__(256) latent_rope_append_kernel(LatentRopeAppen
     auto lo_of = [&](uint32_t i) { return p.interleaved ? 2 * i : i; };
     auto hi_of = [&](uint32_t i) { return p.interleaved ? 2 * i + 1 : i + half; };
     if (wave == 0 && p.caches) {
-        const float* c = xr + p.c_col;
-        float ss = 0.0f;
-        for (uint32_t i = lane; i < p.rank; i += 64) ss = fmaf(c[i], c[i], ss);
-        ss = wave_sum(ss);
-        const float inv = 1.0f / sqrtf(ss / (float)p.rank + p.eps);
         void* cache = p.caches[q];
         const size_t base = (size_t)t * kw;
-        for (uint32_t i = lane; i < p.rank; i += 64) {
-            const float v = c[i] * inv * p.scales[i];
+        wave_rms_norm(xr + p.c_col, p.scales, p.rank, p.eps, lane, [&](uint32_t i, float v) {
             if (p.cache_bf16) ((uint16_t*)cache)[base + i] = f32_to_bf16(v);
             else ((float*)cache)[base + i] = v;
-        }
-        const float* kr = c + p.rank;
+        });
+    }
+    if (wave == 2 && p.caches) {
+        void* cache = p.caches[q];
+        const size_t base = (size_t)t * kw;
+        const float* kr = xr + p.c_col + p.rank;
         for (uint32_t i = lane; i < half; i += 64) {
             const float u = kr[lo_of(i)], v = kr[hi_of(i)], co = cs[i], si = sn[i];
             const float a = u * co - v * si, b = v * co + u * si;
@@ -74,11 +97,8 @@ __global__ void __launch_bounds__(256) latent_rope_append_kernel(LatentRopeAppen
         }
     }
     if (wave == 1 && p.q_rank) { // the query latent's norm
-        float ss = 0.0f;
-        for (uint32_t i = lane; i < p.q_rank; i += 64) ss = fmaf(xr[i], xr[i], ss);
-        ss = wave_sum(ss);
-        const float inv = 1.0f / sqrtf(ss / (float)p.q_rank + p.eps);
-        for (uint32_t i = lane; i < p.q_rank; i += 64) p.q_latent[(size_t)r * p.q_rank + i] = xr[i] * inv * p.q_scales[i];
+        float* dst = p.q_latent + (size_t)r * p.q_rank;
+        wave_rms_norm(xr, p.q_scales, p.q_rank, p.eps, lane, [&](uint32_t i, float v) { dst[i] = v; });
     }
     if (!p.qlat) return;
     for (uint32_t idx = threadIdx.x; idx < p.heads * half; idx += 256) {
@@ -89,6 +109,17 @@ __global__ void __launch_bounds__(256) latent_rope_append_kernel(LatentRopeAppen
         dst[lo_of(i)] = u * co - v * si;
         dst[hi_of(i)] = v * co + u * si;
     }
+}
+
+// coordinate i of the rotated part of row `row`'s head `head` (LatentAttentionParams::queries) at position t
+__device__ __forceinline__ float turned_query(const LatentAttentionParams& p, uint32_t row, uint32_t head, uint32_t t, uint32_t i) {
+    const uint32_t half = p.rope_dim / 2;
+    const bool second = p.interleaved ? (i & 1) != 0 : i >= half;
+    const uint32_t pair = p.interleaved ? i >> 1 : second ? i - half : i;
+    const float* q = p.queries + (size_t)row * p.ldqueries + (size_t)head * p.q_width + (p.q_width - p.rope_dim);
+    const float u = q[p.interleaved ? 2 * pair : pair], v = q[p.interleaved ? 2 * pair + 1 : pair + half];
+    const float c = p.cosines[(size_t)t * p.rope_dim + pair], s = p.sines[(size_t)t * p.rope_dim + pair];
+    return second ? v * c + u * s : u * c - v * s;
 }
 
 // Simple form: a wave per (row, head), lane = latent elements lane, lane + 64, ...; the keys one after the other with a running maximum.
@@ -108,7 +139,7 @@ __global__ void __launch_bounds__(256) latent_attention_rows_kernel(LatentAttent
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
         const uint32_t e = i * 64 + lane;
-        qv[i] = e < p.rank ? ql[e] * p.scale : 0.0f;
+        qv[i] = e < p.rank ? (!p.rope_dim || e + p.rope_dim < p.rank ? ql[e] : turned_query(p, r, h, t, e + p.rope_dim - p.rank)) * p.scale : 0.0f;
         acc[i] = 0.0f;
     }
     // the sink takes part in the maximum and in the denominator only
@@ -186,12 +217,36 @@ __global__ void __launch_bounds__(256) latent_attention_mfma_kernel(LatentAttent
     u32x4_t qf[2 * NB];
     {
         const float* qrow = p.qlat + ((size_t)(sp.row0 + row) * p.heads + head) * p.rank;
+        const bool turn_vec = p.rope_dim && !p.interleaved && p.rope_dim % 16 == 0 && p.q_width % 4 == 0 && p.ldqueries % 4 == 0 && ((uintptr_t)p.queries & 15) == 0; // (rank % 8 == 0)
 #pragma unroll
         for (int s = 0; s < 2 * NB; ++s) {
             const uint32_t k0 = s * 16 + half * 8;
             u32x4_t f{0u, 0u, 0u, 0u};
             if (valid && k0 < p.rank) { // rank % 8 == 0: a fragment is inside the row or outside it
-                const f32x4_v a = *(const f32x4_v*)(qrow + k0), b = *(const f32x4_v*)(qrow + k0 + 4);
+                f32x4_v a, b;
+                if (!p.rope_dim || k0 + 8 + p.rope_dim <= p.rank) {
+                    a = *(const f32x4_v*)(qrow + k0), b = *(const f32x4_v*)(qrow + k0 + 4);
+                } else if (turn_vec) { // the fragment lies in one half of the rotated part: eight pairs' coordinates, cosines and sines as vectors
+                    const uint32_t i = k0 + p.rope_dim - p.rank, hw = p.rope_dim / 2;
+                    const bool second = i >= hw;
+                    const float* q = p.queries + (size_t)(sp.row0 + row) * p.ldqueries + (size_t)head * p.q_width + (p.q_width - p.rope_dim) + (second ? i - hw : i);
+                    const float* c = p.cosines + (size_t)t * p.rope_dim + i; // (the tables repeat their first half)
+                    const float* sn = p.sines + (size_t)t * p.rope_dim + i;
+                    const f32x4_v u0 = *(const f32x4_v*)q, u1 = *(const f32x4_v*)(q + 4), v0 = *(const f32x4_v*)(q + hw), v1 = *(const f32x4_v*)(q + hw + 4);
+                    const f32x4_v c0 = *(const f32x4_v*)c, c1 = *(const f32x4_v*)(c + 4), s0 = *(const f32x4_v*)sn, s1 = *(const f32x4_v*)(sn + 4);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        a[e] = second ? v0[e] * c0[e] + u0[e] * s0[e] : u0[e] * c0[e] - v0[e] * s0[e];
+                        b[e] = second ? v1[e] * c1[e] + u1[e] * s1[e] : u1[e] * c1[e] - v1[e] * s1[e];
+                    }
+                } else { // the fragment reaches into the rotated part
+                    const uint32_t plain = p.rank - p.rope_dim, r = sp.row0 + row;
+#pragma unroll
+                    for (uint32_t e = 0; e < 4; ++e) {
+                        a[e] = k0 + e < plain ? qrow[k0 + e] : turned_query(p, r, head, t, k0 + e - plain);
+                        b[e] = k0 + 4 + e < plain ? qrow[k0 + 4 + e] : turned_query(p, r, head, t, k0 + 4 + e - plain);
+                    }
+                }
                 f.x = (uint32_t)f32_to_bf16(a.x) | ((uint32_t)f32_to_bf16(a.y) << 16), f.y = (uint32_t)f32_to_bf16(a.z) | ((uint32_t)f32_to_bf16(a.w) << 16);
                 f.z = (uint32_t)f32_to_bf16(b.x) | ((uint32_t)f32_to_bf16(b.y) << 16), f.w = (uint32_t)f32_to_bf16(b.z) | ((uint32_t)f32_to_bf16(b.w) << 16);
             }
@@ -336,6 +391,7 @@ __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const float
     const float inv = s_inv;
     for (uint32_t e = tid; e < cols; e += blockDim.x) {
         float acc = 0.0f;
+#pragma unroll 8
         for (uint32_t s = 0; s < splits; ++s) acc = fmaf(s_w[s], base[(size_t)s * (rp + 4) + e], acc);
         out[(size_t)item * rank + e] = acc * inv;
     }
@@ -373,6 +429,7 @@ uzu_status latent_attention(hipStream_t s, const LatentAttentionParams& p) {
     if (!p.rows) return UZU_OK;
     UZU_REQUIRE(p.qlat && p.out && p.caches && p.spans && p.row_seq && p.heads && p.rank, "latent_attention: null argument");
     UZU_UNSUPPORTED(p.rank > kLatentMaxRank, "latent_attention: latent rank %u above %u", p.rank, kLatentMaxRank);
+    UZU_REQUIRE(!p.rope_dim || (p.queries && p.cosines && p.sines && p.rope_dim % 2 == 0 && p.rope_dim < p.rank && p.q_width >= p.rope_dim), "latent_attention: a rotated query part with its rows and tables");
     UZU_REQUIRE(p.value_rank <= p.rank && p.value_rank % 4 == 0, "latent_attention: value_rank is a multiple of 4 of at most rank");
     UZU_UNSUPPORTED(p.form == 2 && !latent_attention_tiled_supported(p), "latent_attention: the tiled form takes a bf16 cache, rank %% 8 == 0, rank <= 256");
     if (p.form != 1 && latent_attention_tiled_supported(p)) {

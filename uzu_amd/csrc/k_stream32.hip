@@ -19,6 +19,20 @@ __device__ __forceinline__ float opnd(float v, uint32_t bf16_products) { return 
 __device__ __forceinline__ float lane_dot(const float* x, const uint16_t* w, uint32_t n, uint32_t lane, uint32_t round_x = 0) {
     float acc = 0.0f;
     if (round_x) { // operand rows that were not rounded when they were staged (read straight from global memory)
+        if ((n & 7) == 0 && (((uintptr_t)w | (uintptr_t)x) & 15) == 0) {
+            for (uint32_t i0 = lane * 8; i0 < n; i0 += 512) {
+                const uint4 wv = *(const uint4*)(w + i0);
+                const float4 a = *(const float4*)(x + i0), b = *(const float4*)(x + i0 + 4);
+                const uint32_t ww[4] = {wv.x, wv.y, wv.z, wv.w};
+                const float xv[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    acc = fmaf(round_bf16(xv[2 * j]), bits_to_f32(ww[j] << 16), acc);
+                    acc = fmaf(round_bf16(xv[2 * j + 1]), bits_to_f32(ww[j] & 0xFFFF0000u), acc);
+                }
+            }
+            return acc;
+        }
         for (uint32_t i = lane; i < n; i += 64) acc = fmaf(round_bf16(x[i]), bf16_to_f32(w[i]), acc);
         return acc;
     }
@@ -539,6 +553,24 @@ __global__ void __launch_bounds__(256) moe_experts_down_kernel(const float* hidd
     }
 }
 
+// few rows (decode): a wave per (row, output) and nothing staged, so that the experts' rows stream through the whole chip; the winners' weighted parts meet per lane
+// and are summed over the wave once
+__global__ void __launch_bounds__(256) moe_experts_down_rows_kernel(const float* hidden, const float* x, const int32_t* ids, const float* weights, const uint16_t* w2,
+                                                                    const float* residual, float* y, uint32_t d, uint32_t ff, uint32_t routed, uint32_t top, uint32_t bf16_products) {
+    const uint32_t r = blockIdx.x, lane = threadIdx.x & 63, n = blockIdx.y * 4 + (threadIdx.x >> 6);
+    if (n >= d) return;
+    float acc = 0.0f, same = 0.0f; // same: identity experts
+    for (uint32_t j = 0; j < top; ++j) {
+        const int32_t e = ids[(size_t)r * top + j];
+        const float wt = weights[(size_t)r * top + j];
+        if (e < 0) continue;
+        if ((uint32_t)e >= routed) same = fmaf(wt, x[(size_t)r * d + n], same);
+        else acc = fmaf(wt, lane_dot(hidden + ((size_t)r * top + j) * ff, w2 + ((size_t)e * d + n) * ff, ff, lane, bf16_products), acc);
+    }
+    acc = wave_sum(acc) + same;
+    if (lane == 0) y[(size_t)r * d + n] = residual ? residual[(size_t)r * d + n] + acc : acc;
+}
+
 // ---- bucketing of the (row, slot) pairs by expert for the grouped matrix-core form
 __global__ void __launch_bounds__(1024) moe_bucket_kernel(const int32_t* ids, uint32_t slots, uint32_t routed, uint32_t* offsets, uint32_t* cursor) {
     extern __shared__ uint32_t s_hist[];
@@ -750,7 +782,7 @@ uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids
     if (!rows || !routed) return UZU_OK;
     UZU_UNSUPPORTED((size_t)d * 4 > 48 * 1024, "moe_experts_gate_up: model_dim %u does not fit the workgroup's LDS row", d);
     // few (row, slot) pairs (decode): the hidden units of a pair are spread over more workgroups, so that the expert's rows stream through many CUs
-    const uint32_t want = (1024 + rows * top - 1) / (rows * top), most = (ff + 15) / 16;
+    const uint32_t want = (1024 + rows * top - 1) / (rows * top), most = (ff + 3) / 4;
     const uint32_t gy = want < 1 ? 1 : (want > most ? most : want);
     return launch_check([&] { hipLaunchKernelGGL(moe_experts_gate_up_kernel, dim3(rows * top, gy), dim3(256), (size_t)d * 4, s, x, ids, w13, hidden, d, ff, routed, top, bf16_products, act); },
                         "moe_experts_gate_up");
@@ -759,6 +791,9 @@ uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids
 uzu_status moe_experts_down_combine(hipStream_t s, const float* hidden, const float* x, const int32_t* ids, const float* weights, const uint16_t* w2, const float* residual,
                                     float* y, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed, uint32_t top, uint32_t bf16_products) {
     if (!rows) return UZU_OK;
+    if (rows <= 16)
+        return launch_check([&] { hipLaunchKernelGGL(moe_experts_down_rows_kernel, dim3(rows, (d + 3) / 4), dim3(256), 0, s, hidden, x, ids, weights, w2, residual, y, d, ff, routed, top, bf16_products); },
+                            "moe_experts_down_rows");
     const uint32_t staged = (size_t)top * ff * 4 <= 48 * 1024 ? 1u : 0u;
     const uint32_t want = (1024 + rows - 1) / rows, most = (d + 15) / 16;
     const uint32_t gy = want < 1 ? 1 : (want > most ? most : want);

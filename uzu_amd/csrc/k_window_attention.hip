@@ -18,8 +18,8 @@ __device__ __forceinline__ void cache_st(void* p, uint32_t is_bf16, size_t i, fl
     else ((float*)p)[i] = v;
 }
 
-// a workgroup per row: query pairs in place, key pairs (+ the unrotated tail) to the cache or in place, values to the cache
-__global__ void __launch_bounds__(256) rope_append_kernel(RopeAppendParams p) {
+// a workgroup per row (256 threads; few rows: 1024, so that the heads' norms run side by side): query pairs in place, key pairs (+ the unrotated tail) to the cache or in place, values to the cache
+__global__ void __launch_bounds__(1024) rope_append_kernel(RopeAppendParams p) {
     const uint32_t r = blockIdx.x;
     const uint32_t z = p.row_seq[r];
     const SeqSpan sp = p.spans[z];
@@ -32,7 +32,7 @@ __global__ void __launch_bounds__(256) rope_append_kernel(RopeAppendParams p) {
     if (p.kv_heads && p.value_caches) {
         void* vc = p.value_caches[z];
         const size_t vrow = (size_t)t * p.kv_heads * p.vdim;
-        for (uint32_t idx = threadIdx.x; idx < p.kv_heads * p.vdim; idx += 256) cache_st(vc, p.cache_bf16, vrow + idx, row[p.v_col + idx]);
+        for (uint32_t idx = threadIdx.x; idx < p.kv_heads * p.vdim; idx += blockDim.x) cache_st(vc, p.cache_bf16, vrow + idx, row[p.v_col + idx]);
         __syncthreads();
     }
     if (p.norm_whole && (p.q_norm || p.k_norm)) { // one RMS norm over all query coordinates of the row, one over all key coordinates: 256 strided partial sums, a fixed tree
@@ -57,7 +57,7 @@ __global__ void __launch_bounds__(256) rope_append_kernel(RopeAppendParams p) {
         __syncthreads();
     } else if (p.q_norm || p.k_norm) { // a wave per head: x <- x / sqrt(mean(x^2) + eps) * w over the head's coordinates, in front of the rotation
         const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-        for (uint32_t a = wave; a < p.heads + p.kv_heads; a += 4) {
+        for (uint32_t a = wave; a < p.heads + p.kv_heads; a += blockDim.x >> 6) {
             const bool is_q = a < p.heads;
             const float* w = is_q ? p.q_norm : p.k_norm;
             if (!w) continue;
@@ -70,7 +70,7 @@ __global__ void __launch_bounds__(256) rope_append_kernel(RopeAppendParams p) {
         }
         __syncthreads();
     }
-    for (uint32_t idx = threadIdx.x; idx < p.heads * half; idx += 256) {
+    for (uint32_t idx = threadIdx.x; idx < p.heads * half; idx += blockDim.x) {
         const uint32_t a = idx / half, i = idx - a * half;
         float* h = row + (size_t)a * p.dim;
         const uint32_t iu = p.interleaved ? 2 * i : i, iv = p.interleaved ? 2 * i + 1 : i + half;
@@ -82,7 +82,7 @@ __global__ void __launch_bounds__(256) rope_append_kernel(RopeAppendParams p) {
     const float ks = p.key_scale;
     void* kc = p.key_caches ? p.key_caches[z] : nullptr;
     const size_t krow = (size_t)t * p.kv_heads * p.dim;
-    for (uint32_t idx = threadIdx.x; idx < p.kv_heads * p.dim; idx += 256) {
+    for (uint32_t idx = threadIdx.x; idx < p.kv_heads * p.dim; idx += blockDim.x) {
         const uint32_t g = idx / p.dim, c = idx - g * p.dim;
         float* h = row + p.k_col + (size_t)g * p.dim;
         if (c >= p.rope_dim) {
@@ -190,7 +190,7 @@ uzu_status rope_append(hipStream_t s, const RopeAppendParams& p) {
     UZU_REQUIRE(p.rope_dim % 2 == 0 && p.rope_dim <= p.dim && (!p.rope_dim || (p.cosines && p.sines)), "rope_append: rotation width %u of a head of %u (even, with its tables)", p.rope_dim, p.dim);
     UZU_REQUIRE(!p.kv_heads || ((p.key_caches != nullptr) == (p.value_caches != nullptr)), "rope_append: key and value caches come together");
     UZU_REQUIRE(p.v_col != p.k_col || !p.kv_heads || (p.vdim == p.dim && p.value_caches), "rope_append: values that are the key rows have the keys' width and go to a cache");
-    return launch_check([&] { hipLaunchKernelGGL(rope_append_kernel, dim3(p.rows), dim3(256), 0, s, p); }, "rope_append");
+    return launch_check([&] { hipLaunchKernelGGL(rope_append_kernel, dim3(p.rows), dim3(p.rows <= 64 && !p.norm_whole ? 1024 : 256), 0, s, p); }, "rope_append");
 }
 
 uzu_status window_attention_mfma(hipStream_t s, const WindowAttentionParams& p); // k_window_attention_mfma.hip

@@ -198,14 +198,21 @@ __global__ void __launch_bounds__(128) window_attention_merge_kernel(const float
                                                                      uint32_t heads) {
     const uint32_t item = blockIdx.x, tid = threadIdx.x;
     const float* base = ws + (size_t)item * splits * (rp + 4);
-    float M = -1.0e30f;
-    for (uint32_t s = 0; s < splits; ++s) M = fmaxf(M, base[(size_t)s * (rp + 4) + rp]);
+    // the splits' weights once, a lane per split (at most 64 splits); the sums over the splits run in split order
+    __shared__ float s_w[64], s_l[64];
+    if (tid < 64) {
+        const float m = tid < splits ? base[(size_t)tid * (rp + 4) + rp] : -1.0e30f;
+        s_l[tid] = tid < splits ? base[(size_t)tid * (rp + 4) + rp + 1] : 0.0f;
+        s_w[tid] = fast_exp(m - wave_max(m));
+    }
+    __syncthreads();
     float den = 0.0f;
-    for (uint32_t s = 0; s < splits; ++s) den = fmaf(fast_exp(base[(size_t)s * (rp + 4) + rp] - M), base[(size_t)s * (rp + 4) + rp + 1], den);
+    for (uint32_t s = 0; s < splits; ++s) den = fmaf(s_w[s], s_l[s], den);
     if (gate) den *= 1.0f + expf(-gate[(size_t)(item / heads) * ldgate + item % heads]);
     for (uint32_t c = tid; c < vdim; c += 128) {
         float acc = 0.0f;
-        for (uint32_t s = 0; s < splits; ++s) acc = fmaf(fast_exp(base[(size_t)s * (rp + 4) + rp] - M), base[(size_t)s * (rp + 4) + c], acc);
+#pragma unroll 8
+        for (uint32_t s = 0; s < splits; ++s) acc = fmaf(s_w[s], base[(size_t)s * (rp + 4) + c], acc);
         out[(size_t)item * vdim + c] = acc / den;
     }
 }

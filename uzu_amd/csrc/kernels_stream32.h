@@ -205,6 +205,11 @@ struct LatentAttentionParams {
     uint32_t nseq;  // entries of `spans`
     uint32_t tiles; // sum over the sequences of ceil(count * heads / 128): the tiled form's workgroups (the caller knows the counts)
     uint32_t value_rank;
+    // rope_dim != 0: the last rope_dim columns of a query are not in qlat but turned as they are loaded: the last rope_dim coordinates of head a of `queries`
+    // (f32 rows of pitch ldqueries, a head q_width wide), by the row's position (tables and pairs as latent_rope_append reads them)
+    const float* queries;
+    uint32_t ldqueries, q_width, rope_dim, interleaved;
+    const float *cosines, *sines;
     // tiled form, few rows over many keys (decode): `splits` > 1 workgroups share the key blocks of an item tile, partial sums go through split_ws
     // (latent_attention_split_ws_bytes(rows, heads, rank, splits) bytes) and a merge launch.  0 / null: one workgroup walks all keys of its tile.
     uint32_t splits;
