@@ -110,6 +110,8 @@ MECHANISMS = {
     "latent_rotation_wider_than_the_plain_part": one_layer(lat(dim=2, rot_dim=24, rotation=O.rot(24, 50.0))),
     "latent_scaled_rotation": one_layer(lat(rot_dim=16, rotation=O.rot(16, 1e4, O.yarn(8.0, 64, 8.0, 0.25)))),
     "latent_scaled_rotation_with_an_empty_ramp": one_layer(lat(rot_dim=8, rotation=O.rot(8, 1e6, O.yarn(2.5, 8, 4.0, 4.0)))),
+    "latent_rank_not_a_multiple_of_four": one_layer(lat(kv_rank=14, rot_dim=2)),
+    "latent_fragment_across_the_rotated_part": one_layer(lat(kv_rank=12, rot_dim=20, heads=3)),
     "latent_wider_than_the_tiled_core": one_layer(lat(kv_rank=280, q_rank=48)),
     "latent_query_rank_above_a_wave's_registers": one_layer(lat(q_rank=1100)),
     "attention": one_layer(att()),
@@ -144,18 +146,19 @@ MECHANISMS = {
 
 
 @pytest.mark.parametrize("which", sorted(MECHANISMS))
-def test_each_mechanism_alone_in_a_one_layer_model(hip_ctx, tmp_path, which):
+@pytest.mark.parametrize("full", [True, False])
+def test_each_mechanism_alone_in_a_one_layer_model(hip_ctx, tmp_path, which, full):
     cfg = MECHANISMS[which]
-    W, m = make(hip_ctx, tmp_path, cfg, 5)
+    W, m = make(hip_ctx, tmp_path, cfg, 5, flags=MODEL_FULL_F32 if full else 0)
     toks = prompt(cfg, 90, 3)
     want, behind = O.forward(cfg, W, toks)
     st = m.new_state()
     got, _ = m.step_batch([st], [toks], [list(range(len(toks)))])
     for l, ref in enumerate(behind):
-        assert np.abs(m.read_layer_output_f32(l) - ref).max() < 2e-5 * np.abs(ref).max(), l
-    assert O.logit_error(got, want).max() < TOL[True]
+        assert rows_ok(np.abs(m.read_layer_output_f32(l) - ref).max(-1) / np.abs(ref).max(), full, 2e-5 if full else 5e-2), l
+    assert rows_ok(O.logit_error(got, want), full)
     st.reset()  # and token by token from a reused state: the decode forms of the same kernels
-    assert O.logit_error(in_portions(m, st, toks[:40], [1] * 40), want[:40]).max() < TOL[True]
+    assert rows_ok(O.logit_error(in_portions(m, st, toks[:40], [1] * 40), want[:40]), full)
     st.close()
     m.close()
 
@@ -193,6 +196,30 @@ def test_head_widths_of_real_models_in_both_precisions(hip_ctx, tmp_path, full):
     want, _ = O.forward(cfg, W, toks)
     st = m.new_state()
     assert rows_ok(O.logit_error(in_portions(m, st, toks, [110, 30] + [1] * 20), want), full)
+    st.close()
+    m.close()
+
+
+@pytest.mark.parametrize("kv_rank,rot_dim", [(48, 16), (12, 4)])
+@pytest.mark.parametrize("full", [True, False])
+def test_interleaved_pairs_are_a_permutation_of_the_rotated_coordinates(hip_ctx, tmp_path, full, kv_rank, rot_dim):
+    """the engine's other pairing of the rotated coordinates in the attention core's query load: pairs (2i, 2i + 1) over rows brought into that order give the same model"""
+    cfg = one_layer(lat(kv_rank=kv_rank, rot_dim=rot_dim))
+    W, m = make(hip_ctx, tmp_path, cfg, 5, flags=MODEL_FULL_F32 if full else 0)
+    m.close()
+    bundle = loader.load_model_dir(str(tmp_path / "m"), max_context_length=256)
+    l = bundle.layers[0]
+    order = np.arange(rot_dim).reshape(2, rot_dim // 2).T.ravel()  # i, i + rot_dim / 2, i + 1, ...
+    up, packed = l.latent_query_up.weights.reshape(l.num_heads, l.head_dim + rot_dim, -1).copy(), l.qkv_projection.weights.copy()
+    up[:, l.head_dim:] = up[:, l.head_dim:][:, order]
+    lo = l.latent_query_up.k + kv_rank
+    packed[lo:lo + rot_dim] = packed[lo:lo + rot_dim][order]
+    turned = dataclasses.replace(l, rope_interleaved=True, latent_query_up=dataclasses.replace(l.latent_query_up, weights=np.ascontiguousarray(up.reshape(l.latent_query_up.weights.shape))),
+                                 qkv_projection=dataclasses.replace(l.qkv_projection, weights=packed))
+    m = HipModel(hip_ctx, dataclasses.replace(bundle, layers=[turned]), MODEL_BATCH(2) | (MODEL_FULL_F32 if full else 0))
+    toks = prompt(cfg, 100, 3)
+    st = m.new_state()
+    assert rows_ok(O.logit_error(in_portions(m, st, toks, [85] + [1] * 15), O.forward(cfg, W, toks)[0]), full)
     st.close()
     m.close()
 
