@@ -23,8 +23,8 @@ constexpr int PITCH = 144;   // bytes per staged row: 64 bf16 + 16 bytes of pad
 
 __device__ __forceinline__ uint32_t pack_bf16(float a, float b) { return (uint32_t)f32_to_bf16(a) | ((uint32_t)f32_to_bf16(b) << 16); }
 
-template <int MB, int NB, bool GROUPED> // GROUPED: per-product row buckets (row_offsets) and gathered operand rows (row_map); the plain form carries neither
-__global__ void __launch_bounds__(256) linear_mfma_kernel(LinearF32Params p) {
+template <int MB, int NB, bool GROUPED, int KIND> // KIND: EpilogueKind; GROUPED: per-product row buckets (row_offsets) and gathered operand rows (row_map); the plain form carries neither
+__global__ void __launch_bounds__(256, MB * NB == 4 && KIND != kEpilogueFull ? 3 : 1) linear_mfma_kernel(LinearF32Params p) {
     constexpr int BM = 64 * MB, BN = 64 * NB;
     constexpr int A_PASSES = BM / 16; // 16 threads cover a row's 64 k (one float4 each), 16 rows per pass
     constexpr int B_PASSES = BN / 32; // 8 threads cover a row's 64 k (one 16-byte vector each), 32 rows per pass
@@ -54,13 +54,41 @@ __global__ void __launch_bounds__(256) linear_mfma_kernel(LinearF32Params p) {
     u32x4_v b_reg[B_PASSES];
     const uint32_t a_row = tid >> 4, a_k = (tid & 15) * 4;
     const uint32_t b_row = tid >> 3, b_k = (tid & 7) * 8;
+    // GROUPED: where this thread's rows start, once (element offsets; the gather's indices must not be read again in every k-step): a row or column outside the product
+    // is read from inside it and its sums are not stored
+    uint32_t a_at[A_PASSES], b_at[B_PASSES];
+    if (GROUPED) {
+#pragma unroll
+        for (int i = 0; i < A_PASSES; ++i) {
+            const uint32_t r = m0 + a_row + i * 16, in = r < r_hi ? r : r_hi - 1;
+            a_at[i] = (p.row_map ? p.row_map[in] : in) * p.ldx + a_k;
+        }
+#pragma unroll
+        for (int i = 0; i < B_PASSES; ++i) {
+            const uint32_t n = n0 + b_row + i * 32;
+            b_at[i] = (n < p.n ? n : p.n - 1) * p.k + b_k;
+        }
+    }
     auto load = [&](uint32_t k0) {
+        if (GROUPED) {
+            const bool a_ok = k0 + a_k < p.k, b_ok = k0 + b_k < p.k; // (the last k-step)
+#pragma unroll
+            for (int i = 0; i < A_PASSES; ++i) {
+                const f32x4_v v = *(const f32x4_v*)(x + (a_ok ? a_at[i] + k0 : 0u));
+                a_reg[i] = a_ok ? v : f32x4_v{0.f, 0.f, 0.f, 0.f};
+            }
+#pragma unroll
+            for (int i = 0; i < B_PASSES; ++i) {
+                const u32x4_v v = *(const u32x4_v*)(w + (b_ok ? b_at[i] + k0 : 0u));
+                b_reg[i] = b_ok ? v : u32x4_v{0u, 0u, 0u, 0u};
+            }
+            return;
+        }
 #pragma unroll
         for (int i = 0; i < A_PASSES; ++i) {
             const uint32_t r = m0 + a_row + i * 16, kk = k0 + a_k;
             const bool ok = r < r_hi && kk < p.k;
-            const uint32_t sr = ok ? ((GROUPED && p.row_map) ? p.row_map[r] : r) : 0;
-            const float* src = x + (size_t)sr * p.ldx + (ok ? kk : 0);
+            const float* src = x + (size_t)(ok ? r : 0) * p.ldx + (ok ? kk : 0);
             const f32x4_v v = *(const f32x4_v*)src;
             a_reg[i] = ok ? v : f32x4_v{0.f, 0.f, 0.f, 0.f};
         }
@@ -117,13 +145,31 @@ __global__ void __launch_bounds__(256) linear_mfma_kernel(LinearF32Params p) {
         const float bias = p.bias ? bf16_to_f32(p.bias[n]) : 0.0f;
 #pragma unroll
         for (int i = 0; i < MB; ++i) {
+            const uint32_t row0 = m0 + (wm * MB + i) * 32 + 4 * half;
+            float res[16]; // (the residual may be y itself: a block's rows are read before any of them is stored)
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
-                const uint32_t row = m0 + (wm * MB + i) * 32 + (r & 3) + 8 * (r >> 2) + 4 * half;
+                const uint32_t row = row0 + (r & 3) + 8 * (r >> 2);
+                res[r] = p.residual && row < r_hi ? p.residual[(size_t)row * p.ldr + n] : 0.0f;
+            }
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const uint32_t row = row0 + (r & 3) + 8 * (r >> 2);
                 if (row >= r_hi) continue;
-                y[(size_t)row * p.ldy + n] = linear_epilogue(acc[i][j][r], bias, p, row, z, n);
+                const float v = linear_value<KIND>(acc[i][j][r], bias, p, row, z, n);
+                y[(size_t)row * p.ldy + n] = p.residual ? v + res[r] : v;
             }
         }
+    }
+}
+
+template <int MB, int NB> uzu_status launch(hipStream_t s, const LinearF32Params& p, const char* what) {
+    const dim3 grid((p.n + 64 * NB - 1) / (64 * NB), (p.rows + 64 * MB - 1) / (64 * MB), p.batch);
+    UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535, "linear_mfma: grid too large");
+    switch (epilogue_kind(p)) {
+    case kEpilogueLean: return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<MB, NB, false, kEpilogueLean>), grid, dim3(256), 0, s, p); }, what);
+    case kEpilogueXielu: return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<MB, NB, false, kEpilogueXielu>), grid, dim3(256), 0, s, p); }, what);
+    default: return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<MB, NB, false, kEpilogueFull>), grid, dim3(256), 0, s, p); }, what);
     }
 }
 
@@ -132,6 +178,7 @@ __global__ void __launch_bounds__(256) linear_mfma_kernel(LinearF32Params p) {
 bool linear_mfma_supported(const LinearF32Params& p) {
     if (!p.bf16_products || (p.rows < 32 && !p.row_offsets) || p.k % 8 || p.ldx % 4 || p.x_batch % 4 || p.w_batch % 8) return false;
     if ((uintptr_t)p.x % 16 || (uintptr_t)p.w % 16) return false;
+    if (p.row_offsets && ((uint64_t)p.rows * p.ldx >= 1ull << 32 || (uint64_t)p.n * p.k >= 1ull << 32)) return false; // (grouped: element offsets inside a product are 32-bit)
     return true;
 }
 
@@ -141,24 +188,14 @@ uzu_status linear_mfma(hipStream_t s, const LinearF32Params& p) {
     // tile choice: the widest tile that still fills the chip; narrow outputs (the per-head products) take the narrow tiles
     if (p.row_offsets) { // grouped: every product may need the whole row range, the workgroups beyond a bucket leave at once
         const dim3 grid((p.n + 127) / 128, (p.rows + 127) / 128 + 1, p.batch);
-        UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535 && !p.residual, "linear_mfma: grouped grid too large");
-        return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<2, 2, true>), grid, dim3(256), 0, s, p); }, "linear_mfma_grouped");
+        UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535 && !p.residual && epilogue_kind(p) == kEpilogueLean, "linear_mfma: a grouped launch of that size, with a residual or more than a bias and an activation");
+        return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<2, 2, true, kEpilogueLean>), grid, dim3(256), 0, s, p); }, "linear_mfma_grouped");
     }
     const bool small_m = p.rows <= 64, small_n = p.n <= 64;
     auto tiles = [&](uint32_t bm, uint32_t bn) { return (size_t)((p.rows + bm - 1) / bm) * ((p.n + bn - 1) / bn) * p.batch; };
-    if (!small_m && !small_n && tiles(128, 128) >= 256) {
-        const dim3 grid((p.n + 127) / 128, (p.rows + 127) / 128, p.batch);
-        UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535, "linear_mfma: grid too large");
-        return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<2, 2, false>), grid, dim3(256), 0, s, p); }, "linear_mfma<2,2>");
-    }
-    if (!small_m && (small_n || tiles(128, 64) >= 256)) {
-        const dim3 grid((p.n + 63) / 64, (p.rows + 127) / 128, p.batch);
-        UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535, "linear_mfma: grid too large");
-        return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<2, 1, false>), grid, dim3(256), 0, s, p); }, "linear_mfma<2,1>");
-    }
-    const dim3 grid((p.n + 63) / 64, (p.rows + 63) / 64, p.batch);
-    UZU_REQUIRE(grid.y <= 65535 && grid.z <= 65535, "linear_mfma: grid too large");
-    return launch_check([&] { hipLaunchKernelGGL((linear_mfma_kernel<1, 1, false>), grid, dim3(256), 0, s, p); }, "linear_mfma<1,1>");
+    if (!small_m && !small_n && tiles(128, 128) >= 256) return launch<2, 2>(s, p, "linear_mfma<2,2>");
+    if (!small_m && (small_n || tiles(128, 64) >= 256)) return launch<2, 1>(s, p, "linear_mfma<2,1>");
+    return launch<1, 1>(s, p, "linear_mfma<1,1>");
 }
 
 } // namespace k
