@@ -55,7 +55,7 @@ struct Stream32 {
     float *tmp = nullptr, *y1 = nullptr, *lru_u = nullptr, *lru_g = nullptr, *side_g = nullptr; // a sublayer's result in front of its post norm; [up | gate] of a gated dense block; LRU input / gates; token-input gate
     float *moe_y1 = nullptr, *moe_y2 = nullptr; // grouped expert form: [max_rows * top][2 ff] and [max_rows * top][d]
     uint32_t *moe_perm = nullptr, *moe_slot_pos = nullptr, *moe_offsets = nullptr, *moe_cursor = nullptr;
-    float *hyper = nullptr, *conv_rows = nullptr, *lat_q = nullptr, *moe_z = nullptr; // copies of the stream [s][max_rows][d]; a normed row + its convolution; queries behind their latent; router logits
+    float *hyper = nullptr, *conv_rows = nullptr, *lat_q = nullptr; // copies of the stream [s][max_rows][d]; a normed row + its convolution; queries behind their latent
     float *out_normed = nullptr, *logits = nullptr;
     size_t logit_rows = 0;
     k::SeqSpan* d_spans = nullptr;
@@ -540,12 +540,6 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                     rp.x = mlp_in, rp.router = L.moe.router_weights, rp.selection_bias = X.selection_bias, rp.ids = S.moe_ids, rp.weights = S.moe_w, rp.rows = rows, rp.d = d, rp.outputs = E;
                     rp.top = top, rp.groups = M.router_groups ? M.router_groups : 1, rp.keep = M.router_groups_keep ? M.router_groups_keep : rp.groups, rp.bf16_products = bf;
                     rp.scale = M.router_scale != 0.0f ? M.router_scale : 1.0f;
-                    if (rows > 16) { // many rows: the logits as one product (f32 sums)
-                        k::LinearF32Params zp{};
-                        zp.x = mlp_in, zp.w = L.moe.router_weights, zp.y = S.moe_z, zp.rows = rows, zp.n = E, zp.k = d, zp.ldx = d, zp.ldy = E, zp.batch = 1, zp.bf16_products = bf;
-                        run_linear(e, zp);
-                        rp.logits = S.moe_z;
-                    }
                     RUN("moe_route_groups", (size_t)E * d * 2, k::moe_route_groups(s, rp));
                 } else if (M.routing == UZU_MOE_ROUTE_SCORES) {
                     RUN("moe_route_scores", (size_t)(E + M.num_identity_experts) * d * 2,
@@ -1083,7 +1077,6 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     if (desc->hyper_streams) TRY(need_f32(m, (size_t)desc->hyper_streams * R * d, &S.hyper));
     if (any_normed_conv) TRY(need_f32(m, R * d, &S.conv_rows));
     if (w_latq) TRY(need_f32(m, R * w_latq, &S.lat_q));
-    if (w_routed) TRY(need_f32(m, R * w_routed, &S.moe_z));
     TRY(need_f32(m, R * d, &S.xin));
     TRY(need_f32(m, R * d, &S.normed));
     TRY(need_f32(m, R * d, &S.out_normed));

@@ -427,49 +427,81 @@ __global__ void __launch_bounds__(64) moe_route_scores_kernel(const float* x, co
     }
 }
 
-// ---- grouped sigmoid routing: a workgroup per row; the waves share the router's outputs (or the logits are there already), wave 0 chooses
+// ---- grouped sigmoid routing: a workgroup per RT rows; its waves share the router's outputs (an output's weights are read once for the RT rows), then a wave per row
+// chooses.  staged: the rows go through LDS (rounded there), else (rows too wide) RT is 1 and the row is read from global memory.
+template <int RT>
 __global__ void __launch_bounds__(1024) moe_route_groups_kernel(RouteGroupsParams p, uint32_t staged) {
-    extern __shared__ float s_mem[]; // [outputs] scores | [outputs] choice scores | [groups] strengths | [d] the row (staged)
-    float *s_score = s_mem, *s_choice = s_mem + p.outputs, *s_strength = s_choice + p.outputs, *s_x = s_strength + p.groups;
-    const uint32_t r = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
-    const float* xr = p.x + (size_t)r * p.d;
-    if (staged) {
-        for (uint32_t i = tid; i < p.d; i += blockDim.x) s_x[i] = opnd(xr[i], p.bf16_products);
+    extern __shared__ __attribute__((aligned(16))) float s_mem[]; // RT x [d] rows (staged) | RT x ([outputs] scores | [outputs] choice scores | [groups] strengths)
+    const uint32_t r0 = blockIdx.x * RT, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, nw = blockDim.x >> 6;
+    const uint32_t rows = p.rows - r0 < (uint32_t)RT ? p.rows - r0 : (uint32_t)RT, per_row = 2 * p.outputs + p.groups;
+    float *s_x = s_mem, *s_row = s_mem + (staged ? (size_t)RT * p.d : 0);
+    const float* x = p.x + (size_t)r0 * p.d;
+    if (staged) { // (rows the pass does not have: zeros)
+        for (uint32_t i = tid; i < RT * p.d; i += blockDim.x) s_x[i] = i < rows * p.d ? opnd(x[i], p.bf16_products) : 0.0f;
         __syncthreads();
     }
-    for (uint32_t e = p.logits ? tid : wave; e < p.outputs; e += p.logits ? blockDim.x : nw) {
-        float z;
-        if (p.logits) z = p.logits[(size_t)r * p.outputs + e];
-        else if (staged) z = wave_sum(lane_dot(s_x, p.router + (size_t)e * p.d, p.d, lane));
-        else z = wave_sum(lane_dot(xr, p.router + (size_t)e * p.d, p.d, lane, p.bf16_products));
-        const float sc = 1.0f / (1.0f + expf(-z));
-        if (p.logits || lane == 0) s_score[e] = sc, s_choice[e] = sc + (p.selection_bias ? p.selection_bias[e] : 0.0f);
+    const bool vec = staged && (p.d & 7) == 0 && ((uintptr_t)p.router & 15) == 0;
+    for (uint32_t e = wave; e < p.outputs; e += nw) {
+        const uint16_t* w = p.router + (size_t)e * p.d;
+        float z[RT];
+#pragma unroll
+        for (int i = 0; i < RT; ++i) z[i] = 0.0f;
+        if (vec) {
+            for (uint32_t k0 = lane * 8; k0 < p.d; k0 += 512) {
+                const u32x4_v wv = *(const u32x4_v*)(w + k0);
+#pragma unroll
+                for (int i = 0; i < RT; ++i) {
+                    const f32x4_v a = *(const f32x4_v*)(s_x + i * p.d + k0), b = *(const f32x4_v*)(s_x + i * p.d + k0 + 4);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        z[i] = fmaf(j < 2 ? a[2 * j] : b[2 * j - 4], bits_to_f32(wv[j] << 16), z[i]);
+                        z[i] = fmaf(j < 2 ? a[2 * j + 1] : b[2 * j - 3], bits_to_f32(wv[j] & 0xFFFF0000u), z[i]);
+                    }
+                }
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < RT; ++i) z[i] = staged ? lane_dot(s_x + i * p.d, w, p.d, lane) : lane_dot(x, w, p.d, lane, p.bf16_products);
+        }
+#pragma unroll
+        for (int i = 0; i < RT; ++i) {
+            const float sc = 1.0f / (1.0f + expf(-wave_sum(z[i])));
+            float* row = s_row + i * per_row;
+            if (lane == 0) row[e] = sc, row[p.outputs + e] = sc + (p.selection_bias ? p.selection_bias[e] : 0.0f);
+        }
     }
     __syncthreads();
     const uint32_t size = p.outputs / p.groups;
-    if (p.keep < p.groups) { // thread = group: the sum of its two largest choice scores, then its rank among the groups
-        for (uint32_t g = tid; g < p.groups; g += blockDim.x) {
+    if (p.keep < p.groups) { // thread = (row, group): the sum of its two largest choice scores, then its rank among the row's groups
+        for (uint32_t i = tid; i < RT * p.groups; i += blockDim.x) {
+            float* row = s_row + i / p.groups * per_row;
+            const uint32_t g = i % p.groups;
             float first = -INFINITY, second = -INFINITY;
-            for (uint32_t i = 0; i < size; ++i) {
-                const float c = s_choice[g * size + i];
+            for (uint32_t k = 0; k < size; ++k) {
+                const float c = row[p.outputs + g * size + k];
                 if (c > first) second = first, first = c;
                 else second = fmaxf(second, c);
             }
-            s_strength[g] = size > 1 ? first + second : first;
+            row[2 * p.outputs + g] = size > 1 ? first + second : first;
         }
         __syncthreads();
-        for (uint32_t g = tid; g < p.groups; g += blockDim.x) {
+        for (uint32_t i = tid; i < RT * p.groups; i += blockDim.x) {
+            float* row = s_row + i / p.groups * per_row;
+            const float* strength = row + 2 * p.outputs;
+            const uint32_t g = i % p.groups;
             uint32_t stronger = 0;
-            for (uint32_t o = 0; o < p.groups; ++o) stronger += (s_strength[o] > s_strength[g] || (s_strength[o] == s_strength[g] && o < g)) ? 1u : 0u;
+            for (uint32_t o = 0; o < p.groups; ++o) stronger += (strength[o] > strength[g] || (strength[o] == strength[g] && o < g)) ? 1u : 0u;
             if (stronger >= p.keep)
-                for (uint32_t i = 0; i < size; ++i) s_choice[g * size + i] = -INFINITY;
+                for (uint32_t k = 0; k < size; ++k) row[p.outputs + g * size + k] = -INFINITY;
         }
         __syncthreads();
     }
-    if (wave) return;
+    if (wave >= rows) return; // (RT <= the workgroup's waves)
+    const float *score = s_row + wave * per_row, *choices = score + p.outputs;
+    const size_t out = (size_t)(r0 + wave) * p.top + lane;
     float choice[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) choice[j] = j * 64 + lane < p.outputs ? s_choice[j * 64 + lane] : -INFINITY;
+    for (int j = 0; j < 8; ++j) choice[j] = j * 64 + lane < p.outputs ? choices[j * 64 + lane] : -INFINITY;
     float sum = 0.0f, my_s = 0.0f; // lane t keeps the t-th winner
     int32_t my_id = 0;
     for (uint32_t t = 0; t < p.top; ++t) {
@@ -487,14 +519,11 @@ __global__ void __launch_bounds__(1024) moe_route_groups_kernel(RouteGroupsParam
 #pragma unroll
         for (int j = 0; j < 8; ++j)
             if ((uint32_t)j * 64 + lane == best_e) choice[j] = -INFINITY;
-        const float sc = best_e < p.outputs ? s_score[best_e] : 0.0f; // (a row of NaNs has no winner: id -1, which every consumer passes over)
+        const float sc = best_e < p.outputs ? score[best_e] : 0.0f; // (a row of NaNs has no winner: id -1, which every consumer passes over)
         sum += sc;
         if (t == lane) my_s = sc, my_id = (int32_t)best_e;
     }
-    if (lane < p.top) {
-        p.ids[(size_t)r * p.top + lane] = my_id;
-        p.weights[(size_t)r * p.top + lane] = my_s / (sum + 1e-20f) * p.scale;
-    }
+    if (lane < p.top) p.ids[out] = my_id, p.weights[out] = my_s / (sum + 1e-20f) * p.scale;
 }
 
 // a workgroup per (row, slot): the row once into LDS, then a wave per hidden unit (gate and up rows of the unit in the same pass)
@@ -766,15 +795,16 @@ uzu_status moe_route_topk(hipStream_t s, const float* x, const uint16_t* router,
 
 uzu_status moe_route_groups(hipStream_t s, const RouteGroupsParams& p) {
     if (!p.rows) return UZU_OK;
-    UZU_REQUIRE(p.x && (p.router || p.logits) && p.ids && p.weights && p.d, "moe_route_groups: null argument");
+    UZU_REQUIRE(p.x && p.router && p.ids && p.weights && p.d, "moe_route_groups: null argument");
     UZU_UNSUPPORTED(p.outputs > kRouteMaxOutputs || p.top > 64 || !p.top, "moe_route_groups: at most %u router outputs and 64 winners (got %u, %u)", kRouteMaxOutputs, p.outputs, p.top);
     UZU_REQUIRE(p.groups && p.outputs % p.groups == 0 && p.keep && p.keep <= p.groups && p.top <= p.outputs / p.groups * p.keep, "moe_route_groups: %u winners among %u of %u groups of %u outputs",
                 p.top, p.keep, p.groups, p.outputs);
-    const uint32_t staged = !p.logits && (size_t)p.d * 4 <= 40 * 1024 ? 1u : 0u;
-    const size_t lds = ((size_t)2 * p.outputs + p.groups + (staged ? p.d : 0)) * 4;
-    // with the logits at hand one wave per row will do; without them the outputs' dot products are spread over sixteen
-    const uint32_t threads = p.logits ? 64 : p.outputs <= 4 ? 256 : 1024;
-    return launch_check([&] { hipLaunchKernelGGL(moe_route_groups_kernel, dim3(p.rows), dim3(threads), lds, s, p, staged); }, "moe_route_groups");
+    const uint32_t per_row = 2 * p.outputs + p.groups;
+    const uint32_t threads = p.outputs <= 4 ? 256 : p.outputs <= 8 ? 512 : 1024; // (no wave without an output; at least four)
+    if (p.rows > 64 && ((size_t)p.d + per_row) * 4 * 4 <= 60 * 1024)
+        return launch_check([&] { hipLaunchKernelGGL(moe_route_groups_kernel<4>, dim3((p.rows + 3) / 4), dim3(threads), ((size_t)p.d + per_row) * 4 * 4, s, p, 1u); }, "moe_route_groups");
+    const uint32_t staged = (size_t)p.d * 4 <= 40 * 1024 ? 1u : 0u;
+    return launch_check([&] { hipLaunchKernelGGL(moe_route_groups_kernel<1>, dim3(p.rows), dim3(threads), ((staged ? (size_t)p.d : 0) + per_row) * 4, s, p, staged); }, "moe_route_groups");
 }
 
 uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed,

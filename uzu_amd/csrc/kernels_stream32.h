@@ -133,10 +133,8 @@ uzu_status moe_route_topk(hipStream_t s, const float* x, const uint16_t* router,
 // Grouped sigmoid routing: per row s = sigmoid(router x) in f32 (bf16_products: x rounded to bf16 first), choice scores c = s + selection_bias (f32 [outputs] or null).  The outputs form
 // `groups` equal groups of neighbours; a group's strength is the sum of its two largest c (of its one, if it has one); only outputs of the `keep` strongest groups
 // can be chosen (ties: the lower group).  The `top` largest c among them win (ties: the lower index); weights = s / (sum of the winners' s + 1e-20) * scale.
-// logits (f32 [rows][outputs] or null): router x as the caller has computed it (many rows: one matrix product); null: the launch computes it.
 struct RouteGroupsParams {
     const float* x;
-    const float* logits;
     const uint16_t* router;
     const float* selection_bias;
     int32_t* ids;
