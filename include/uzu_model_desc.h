@@ -121,7 +121,19 @@ typedef enum {
      * a = exp(-lru_decay_rate r softplus(lru_lambda)) the state is S_t = a S_(t-1) + sqrt(1 - a^2) i u (f32 [lru_width], zero in front of position 0) and the
      * mixer's result out_projection(S_t * gelu_tanh(gate branch)) (k = lru_width).  Gates, decays and the state are f32 in both precisions; the sequence state
      * is S and the convolution's last taps - 1 inputs. */
-    UZU_MIXER_GATED_LRU = 4
+    UZU_MIXER_GATED_LRU = 4,
+    /* Gated linear attention (f32-stream designs): per head S_t = diag(a_t) S_(t-1) + k_t v_t^T (f32 [head_dim, value_head_dim], zero in front of position 0; the decay acts
+     * on the rows, one per key channel), o_t = attention_scale S_t^T q_t (attention_scale 0 = head_dim^(-1/2)).  qkv_projection rows: queries | keys | values | gate |
+     * decay down (n = 2 heads head_dim + 2 heads value_head_dim + dn_decay_rank), no biases; z = dn_decay_up (decay down) + its out_biases (n = heads head_dim),
+     * a_t = sigmoid(z)^(1 / decay_temperature).  Every head's o is divided by its root mean square (dn_norm_epsilon) and multiplied by dn_norm_scales [value_head_dim]; the
+     * concatenated heads times silu(gate) go through out_projection.  The up product of the decay, decays and the state are f32 in both precisions. */
+    UZU_MIXER_GATED_LINEAR_ATTENTION = 5,
+    /* State-space duality (Mamba-2), as the SECOND mixer of a pair (pair_mixer; f32-stream designs): dn_num_heads heads of dn_value_head_dim (inner = heads * width), state width
+     * dn_head_dim = N, B and C shared by the heads of each of dn_num_groups groups.  dn_in_proj rows: z (inner) | x (inner) | B (groups N) | C (groups N) | dt (heads);
+     * x, B, C pass a causal convolution per channel (dn_kernel_size taps, dn_conv_weights f32 [inner + 2 groups N, taps], dn_conv_biases) and silu;
+     * dt = softplus(dt + dn_dt_bias [heads]); per head S_t = exp(-exp(dn_a_log) dt) S_(t-1) + dt B_t x_t^T (f32 [N, width], zero in front of position 0),
+     * y_t = S_t^T C_t + ssd_skip x_t.  y * silu(z) is RMS-normed in ssd_norm_groups equal parts (dn_norm_epsilon), times dn_norm_scales [inner], then dn_out_proj. */
+    UZU_MIXER_STATE_SPACE = 6
 } uzu_mixer_kind;
 
 /* config/rope/*.rs -- every AnyRoPEConfig variant (encodable_block/mixer/attention/rope.rs:13-114) */
@@ -184,6 +196,8 @@ typedef struct {
     uint32_t router_groups;
     uint32_t router_groups_keep;
     float router_scale;
+    uint32_t router_raw;       /* ... the weights are the winners' s themselves (times router_scale), not divided by their sum (the field was `reserved`) */
+    uint32_t weight_on_input;  /* f32-stream designs: a winner's weight multiplies its expert's INPUT, y = sum_e expert_e(w_e x); no identity experts */
     uint32_t reserved;
 } uzu_moe_desc;
 typedef enum { UZU_MOE_ROUTE_TOPK_LOGITS = 0, UZU_MOE_ROUTE_SCORES = 1, UZU_MOE_ROUTE_SIGMOID_GROUPS = 2 } uzu_moe_routing;
@@ -340,7 +354,7 @@ typedef struct {
     /* has_gate on such a layer: num_heads more rows behind the packed projection's values; head a's result is multiplied by sigmoid(row a . h). */
     /* A second mixer beside the first (f32-stream designs): both read the same rows, the layer's mixer result is pair_scale_main * main + pair_scale_second *
      * second, each through its own out projection.  pair_mixer = 1 + uzu_mixer_kind of the second (0 = none); supported: attention with a channel-decay delta
-     * rule (UZU_MIXER_DELTA_NET) as the second. */
+     * rule (UZU_MIXER_DELTA_NET) or with a state-space mixer (UZU_MIXER_STATE_SPACE) as the second. */
     uint32_t pair_mixer;
     float pair_scale_main, pair_scale_second;
     /* UZU_MIXER_DELTA_NET in an f32-stream design: the gated delta rule with one decay per head and KEY CHANNEL.  dn_num_heads value heads of dn_value_head_dim on
@@ -368,6 +382,15 @@ typedef struct {
      * u = sum_a in[a] x_a; y = sublayer(norm(u)); then, all from the old ones, x_b <- sum_a mix[a, b] x_a + residual_mult out[b] y. */
     const float* hyper_mixer;
     const float* hyper_mlp; /* NULL on a layer without an MLP */
+    /* UZU_MIXER_ATTENTION in an f32-stream design: a causal convolution over positions on every channel of the packed projection's queries, keys and values (f32 [rows,
+     * qkv_conv_taps], no bias, no activation; the last tap weighs the current position) directly behind the projection, in front of norms and rotation; its last
+     * taps - 1 inputs are sequence state.  NULL = none. */
+    const float* qkv_conv;
+    uint32_t qkv_conv_taps;
+    float decay_temperature;  /* UZU_MIXER_GATED_LINEAR_ATTENTION */
+    const float* ssd_skip;    /* UZU_MIXER_STATE_SPACE: f32 [heads] */
+    uint32_t ssd_norm_groups; /* UZU_MIXER_STATE_SPACE */
+    uint32_t reserved_tail;
 } uzu_layer_desc;
 
 typedef struct {

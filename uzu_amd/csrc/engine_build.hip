@@ -341,7 +341,8 @@ uzu_status uzu_hip_model_create_tp(uzu_hip_context* ctx, const uzu_model_desc* d
                         desc->layers[l].ple_slice || desc->layers[l].input_conv_taps || desc->layers[l].qk_norm_whole || desc->layers[l].attention_chunk_size ||
                         desc->layers[l].values_are_keys || desc->layers[l].rel_bias_rows || desc->layers[l].head_temperature || desc->layers[l].pair_mixer ||
                         desc->layers[l].dn_channel_decay || desc->layers[l].latent_query_rank || desc->layers[l].gate_elementwise || desc->layers[l].hyper_mixer || desc->layers[l].hyper_mlp ||
-                        desc->layers[l].activation == UZU_ACT_XIELU || desc->layers[l].moe.plain_experts || desc->layers[l].post_mixer_norm.groups > 1 || desc->layers[l].post_mlp_norm.groups > 1,
+                        desc->layers[l].activation == UZU_ACT_XIELU || desc->layers[l].mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION || desc->layers[l].mixer_kind == UZU_MIXER_STATE_SPACE ||
+                        desc->layers[l].qkv_conv || desc->layers[l].moe.weight_on_input || desc->layers[l].moe.router_raw || desc->layers[l].moe.plain_experts || desc->layers[l].post_mixer_norm.groups > 1 || desc->layers[l].post_mlp_norm.groups > 1,
                         "model_create: layer %u uses a mechanism of the f32-stream designs (set uzu_model_desc::f32_stream)", l);
     UZU_UNSUPPORTED(desc->bigram_buckets || desc->output_norm.groups > 1 || desc->hyper_streams, "model_create: a hashed token-pair table, grouped norms and hyper-connections are mechanisms of the f32-stream designs");
     (void)hipSetDevice(ctx->device);

@@ -32,6 +32,11 @@
 // on one-row passes -- convolves the second one's row; k_hyper.hip), input convolutions BEHIND a pre norm, latent attention whose queries pass a normed latent of
 // their own and whose concatenated heads are gated coordinate by coordinate, a plain dense block with xIELU, and experts without a gate behind grouped sigmoid routing.
 //
+// A sixth family (Rilavik) adds: attention whose queries, keys and values pass a short causal convolution in front of the rotation, beside a state-space mixer (Mamba-2:
+// one decay and step size per head, grouped B / C, a skip, the gate in front of a norm in parts) -- a pair whose two projections, convolutions and out projections are
+// one launch each --, gated linear attention (a decay per head and key channel through a low-rank projection; both recurrences in k_decayed_state.hip), and experts that
+// read their input times the winner's raw sigmoid score behind a post norm.
+//
 // Precisions: `bf16_products` (default) rounds the activation operand of every matrix product to bf16 and keeps the latent cache in bf16; UZU_MODEL_FULL_F32
 // makes every product a true f32 product and the cache f32.  Everything else is f32 either way.
 #include <algorithm>
@@ -92,6 +97,12 @@ struct Stream32 {
         DNorm lat_q_norm;
         float act_a = 0.f, act_b = 0.f; // xIELU: softplus(p), 1 / 2 + softplus(q)
         float *hyper_mixer = nullptr, *hyper_mlp = nullptr; // f32 [in | out | mix]
+        // attention beside a state-space mixer: ONE projection (rows q | k | v | x | B | C | z | dt), ONE convolution over its first conv_channels columns (the shorter
+        // of the two filled up with zero taps in front; silu from conv_act_from on), ONE out projection over [attention | state-space] rows (W_left | W_right)
+        DLinear joint, joint_out;
+        float *conv_w = nullptr, *conv_b = nullptr; // f32 [conv_channels][conv_taps], f32 [conv_channels]; also: the convolution of an attention layer's q | k | v
+        uint32_t conv_channels = 0, conv_taps = 0, conv_act_from = 0;
+        float *ssd_skip = nullptr, *ssd_norm = nullptr;
     };
     std::vector<Layer> layers;
     float alpha_out = 0.f;
@@ -99,6 +110,9 @@ struct Stream32 {
     size_t ret_ws_bytes = 0;
     float* lru_ws = nullptr; // the recurrent unit in pieces: local state, decay product and carry per (piece of the pass, channel)
     size_t lru_ws_bytes = 0;
+    float* lin_ws = nullptr; // linear attention in chunks: one state block and its decay per (chunk of the pass, head)
+    size_t lin_ws_bytes = 0;
+    float* moe_pos_w = nullptr; // grouped experts whose weights multiply their inputs: the weight of a bucketed row
     float* att_ws = nullptr; // partial sums of the key-split attention of decode-sized passes
     size_t att_ws_bytes = 0;
     float* taps = nullptr; // UZU_MODEL_DEBUG_TAPS: f32 [layers][max_rows][d], what each layer handed on in the last pass
@@ -207,11 +221,11 @@ uzu_status s32_upload_tables(uzu_hip_model* m, const std::vector<PassSeq>& seqs,
             const size_t at = (size_t)l * S.max_seqs + i;
             if (h.mixer_kind == UZU_MIXER_ATTENTION) cache_ptrs[at] = own.cache_k, cache2_ptrs[at] = own.cache_v;
             else if (h.mixer_kind == UZU_MIXER_GATED_LRU) cache_ptrs[at] = own.ssm_state, cache2_ptrs[at] = own.conv_state;
-            else if (h.mixer_kind == UZU_MIXER_RETENTION) cache_ptrs[at] = own.ret_state;
+            else if (h.mixer_kind == UZU_MIXER_RETENTION || h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION) cache_ptrs[at] = own.ret_state;
             else cache_ptrs[at] = own.latent;
             shift_ptrs[at] = seqs[i].st->layers[l].shift_prev;
             inconv[at] = seqs[i].st->layers[l].in_conv;
-            if (h.pair_mixer) pair_state[at] = seqs[i].st->layers[l].ssm_state, pair_conv[at] = seqs[i].st->layers[l].conv_state;
+            if (h.pair_mixer || h.qkv_conv) pair_state[at] = seqs[i].st->layers[l].ssm_state, pair_conv[at] = seqs[i].st->layers[l].conv_state;
         }
     }
     // (pageable sources: the copies have left the host buffers when the calls return)
@@ -341,6 +355,26 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         }
         if (!hs && L.pre_mixer.present && X.in_conv_mixer) mix_in = conv_input(l, S.normed, X.in_conv_mixer, h.input_conv_taps, 0);
         const uint32_t H = h.num_heads, hd = h.head_dim, vd = h.value_head_dim, rank = h.latent_rank;
+        // attention's projected rows: S.q, or -- behind a convolution -- S.dn_cv.  Beside a state-space mixer the one projection and convolution serve both halves.
+        float* qkv_rows = S.q;
+        uint32_t ldqkv = L.qkv.n;
+        const bool joint = X.joint.w != nullptr;
+        auto mixer_conv = [&](uint32_t ldx) {
+            k::CausalConvParams cp{};
+            cp.x = S.q, cp.ldx = ldx, cp.out = S.dn_cv, cp.ldo = X.conv_channels, cp.w = X.conv_w, cp.bias = X.conv_b, cp.channels = X.conv_channels, cp.taps = X.conv_taps;
+            cp.act = X.conv_act_from < X.conv_channels ? 1 : 0, cp.act_from = X.conv_act_from;
+            cp.states = S.d_pair_conv_ptrs + (size_t)l * S.max_seqs, cp.spans = S.d_spans, cp.row_seq = S.d_row_seq, cp.nseq = nseq, cp.rows = rows, cp.max_count = max_count;
+            RUN("causal_conv_rows", (size_t)rows * cp.channels * 4 * (cp.taps + 1), k::causal_conv_rows(s, cp));
+            if (cp.taps > 1 && max_count > 1) RUN("causal_conv_commit", (size_t)nseq * cp.channels * 8 * (cp.taps - 1), k::causal_conv_commit(s, cp));
+            qkv_rows = S.dn_cv, ldqkv = X.conv_channels;
+        };
+        const uint32_t ldj = (X.joint.n + 3) / 4 * 4, ldo_joint = X.joint_out.k; // row pitches of the joint projection and of its halves' results
+        if (joint) {
+            k::LinearF32Params jp = lin(S, X.joint, mix_in, S.q, rows);
+            jp.ldy = ldj;
+            run_linear(e, jp);
+            mixer_conv(ldj);
+        }
         // prompt-sized pass over a pair of mixers: the first one's projection, rotation / append and attention core go to the side stream (they touch S.q, S.attn and
         // the caches; the second mixer touches its own rows); not while a launch is being timed or captured
         bool forked = false;
@@ -350,7 +384,10 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                 hipStreamWaitEvent(S.side, S.side_fork, 0) == hipSuccess)
                 forked = true, s = S.side, e.s = S.side;
         }
-        run_linear(e, lin(S, L.qkv, mix_in, S.q, rows)); // the packed projection of the mixer (queries first)
+        if (!joint) {
+            run_linear(e, lin(S, L.qkv, mix_in, S.q, rows)); // the packed projection of the mixer (queries first)
+            if (X.conv_w) mixer_conv(L.qkv.n);
+        }
         if (h.mixer_kind == UZU_MIXER_GATED_LRU) {
             const uint32_t w = h.lru_width, bw = w / h.lru_blocks;
             k::GatedLruParams gp{};
@@ -368,27 +405,44 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             }
             RUN("lru_scan", (size_t)rows * w * 20, k::lru_scan(s, gp));
         } else if (h.mixer_kind == UZU_MIXER_ATTENTION) {
-            const uint32_t G = h.num_groups, ldq = L.qkv.n;
+            const uint32_t G = h.num_groups, ldq = ldqkv;
             void* const* vcaches = S.d_cache2_ptrs + (size_t)l * S.max_seqs;
             k::RopeAppendParams rp{};
-            rp.qkv = S.q, rp.ld = ldq, rp.k_col = H * hd, rp.v_col = h.values_are_keys ? H * hd : H * hd + G * hd, rp.heads = H, rp.kv_heads = h.is_kv_sharing ? 0u : G, rp.dim = hd, rp.vdim = vd;
+            rp.qkv = qkv_rows, rp.ld = ldq, rp.k_col = H * hd, rp.v_col = h.values_are_keys ? H * hd : H * hd + G * hd, rp.heads = H, rp.kv_heads = h.is_kv_sharing ? 0u : G, rp.dim = hd, rp.vdim = vd;
             rp.rope_dim = h.use_rope ? L.rope_dim : 0u, rp.cosines = L.rope_cos, rp.sines = L.rope_sin, rp.key_scale = h.key_scale != 0.0f ? h.key_scale : 1.0f;
             rp.norm_whole = h.qk_norm_whole, rp.interleaved = h.rope_interleaved;
             rp.key_caches = caches, rp.value_caches = vcaches, rp.cache_bf16 = bf, rp.spans = S.d_spans, rp.row_seq = S.d_row_seq, rp.rows = rows;
             rp.q_norm = L.qn.present ? L.qn.scales : nullptr, rp.k_norm = L.kn.present && !h.is_kv_sharing ? L.kn.scales : nullptr, rp.norm_eps = L.qn.present ? L.qn.eps : L.kn.eps;
             RUN("rope_append", (size_t)rows * ldq * 8, k::rope_append(s, rp));
             k::WindowAttentionParams ap{};
-            ap.q = S.q, ap.ldq = ldq, ap.out = S.attn, ap.key_caches = caches, ap.value_caches = vcaches, ap.cache_bf16 = bf, ap.sinks = X.sinks, ap.spans = S.d_spans;
+            ap.q = qkv_rows, ap.ldq = ldq, ap.out = S.attn, ap.key_caches = caches, ap.value_caches = vcaches, ap.cache_bf16 = bf, ap.sinks = X.sinks, ap.spans = S.d_spans;
             ap.row_seq = S.d_row_seq, ap.rows = rows, ap.heads = H, ap.kv_heads = G, ap.dim = hd, ap.vdim = vd, ap.window = h.sliding_window_size;
             ap.scale = h.attention_scale != 0.0f ? h.attention_scale : 1.0f / sqrtf((float)hd), ap.soft_cap = h.score_soft_cap, ap.nseq = nseq;
             ap.chunk = h.attention_chunk_size, ap.head_scale = X.head_temp, ap.dist_bias = X.dist_bias, ap.dist_rows = X.dist_rows;
-            if (h.has_gate) ap.gate = S.q + H * hd + (h.is_kv_sharing ? 0u : G * hd + (h.values_are_keys ? 0u : G * vd)), ap.ldgate = ldq; // the gate rows stand behind the values
+            if (h.has_gate) ap.gate = S.q + H * hd + (h.is_kv_sharing ? 0u : G * hd + (h.values_are_keys ? 0u : G * vd)), ap.ldgate = L.qkv.n; // the gate rows stand behind the values
+            if (joint) ap.ldo = ldo_joint, ap.out_scale = h.pair_scale_main != 0.0f ? h.pair_scale_main : 1.0e-37f; // (a scale of exactly zero: a result that vanishes)
             for (uint32_t i = 0; i < nseq; ++i) ap.tiles += (counts[i] * (H / G) + 127) / 128;
             // decode-sized passes: spread a tile's key blocks over workgroups (a constant of the layer, so that a captured step stays valid as the context grows)
             uint32_t keys = h.sliding_window_size ? h.sliding_window_size : m->d.max_context_length;
             if (h.attention_chunk_size) keys = std::min(keys, h.attention_chunk_size);
             if (rows <= 4 * S.max_seqs && rows * H <= 4096) ap.splits = std::min<uint32_t>(16, (keys + 31) / 32), ap.split_ws = S.att_ws, ap.split_ws_bytes = S.att_ws_bytes;
             RUN("window_attention", (size_t)rows * H * (hd + vd) * 4, k::window_attention(s, ap));
+        } else if (h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION) { // queries | keys | values | gate | decay down
+            const uint32_t ldq = L.qkv.n, v_col = 2 * H * hd, g_col = v_col + H * vd, a_col = g_col + H * vd;
+            {   // the decay's second factor: what enters the recurrence is never rounded, a true f32 product in both precisions
+                k::LinearF32Params up = lin(S, X.decay_up, S.q + a_col, S.dn_decay, rows);
+                up.ldx = ldq, up.bf16_products = 0;
+                run_linear(e, up);
+            }
+            k::DecayedStateParams dp{};
+            dp.rows_in = S.q, dp.ld = ldq, dp.q_col = 0, dp.k_col = H * hd, dp.v_col = v_col, dp.decay = S.dn_decay, dp.lddecay = H * hd, dp.inv_temperature = 1.0f / h.decay_temperature;
+            dp.q_scale = h.attention_scale != 0.0f ? h.attention_scale : 1.0f / sqrtf((float)hd), dp.out = S.attn, dp.states = (float* const*)caches, dp.spans = S.d_spans, dp.nseq = nseq;
+            dp.rows = rows, dp.heads = H, dp.groups = H, dp.dim = hd, dp.vdim = vd, dp.chunk_ws = S.lin_ws, dp.chunk_ws_bytes = S.lin_ws_bytes;
+            for (uint32_t i = 0; i < nseq; ++i) dp.chunks += (counts[i] + 63) / 64;
+            RUN("decayed_state", (size_t)rows * H * (3 * hd + 2 * vd) * 4 + (size_t)nseq * H * hd * vd * 8, k::decayed_state(s, dp));
+            k::HeadNormGateParams np{};
+            np.x = S.attn, np.ldx = H * vd, np.weight = L.dn_norm, np.gate = S.q + g_col, np.ldgate = ldq, np.eps = h.dn_norm_epsilon, np.rows = rows, np.heads = H, np.width = vd;
+            RUN("head_norm_gate_rows", (size_t)rows * H * vd * 12, k::head_norm_gate_rows(s, np));
         } else if (h.mixer_kind == UZU_MIXER_RETENTION) {
             const uint32_t ldq = L.qkv.n; // queries | keys | values | gate
             k::RopeAppendParams rp{};
@@ -471,7 +525,24 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
             if (hipEventRecord(S.side_join, S.side) != hipSuccess && e.st == UZU_OK) set_error("engine: recording the side stream's join failed"), e.st = UZU_ERR_HIP;
             s = main_stream, e.s = main_stream;
         }
-        if (h.pair_mixer) { // the second mixer beside the first: a delta rule with a decay per head and key channel, reading the same rows
+        if (joint) { // the state-space mixer beside attention: x | B | C stand behind q | k | v in the convolved rows, z | dt behind all of them in the projected ones
+            const uint32_t Hs = h.dn_num_heads, Gs = h.dn_num_groups, N = h.dn_head_dim, pv = h.dn_value_head_dim, inner = Hs * pv, x_col = X.conv_act_from;
+            const uint32_t z_col = X.conv_channels, dt_col = z_col + inner;
+            k::DecayedStateParams dp{};
+            dp.rows_in = S.dn_cv, dp.ld = X.conv_channels, dp.q_col = x_col + inner + Gs * N, dp.k_col = x_col + inner, dp.v_col = x_col, dp.decay = S.q + dt_col, dp.lddecay = ldj, dp.per_head = 1;
+            dp.a_log = L.a_log, dp.dt_bias = L.dt_bias, dp.skip = X.ssd_skip, dp.q_scale = 1.0f, dp.out = S.dn_o, dp.states = S.d_pair_state_ptrs + (size_t)l * S.max_seqs, dp.spans = S.d_spans;
+            dp.nseq = nseq, dp.rows = rows, dp.heads = Hs, dp.groups = Gs, dp.dim = N, dp.vdim = pv, dp.chunk_ws = S.lin_ws, dp.chunk_ws_bytes = S.lin_ws_bytes;
+            for (uint32_t i = 0; i < nseq; ++i) dp.chunks += (counts[i] + 63) / 64;
+            RUN("decayed_state", (size_t)rows * (2 * inner + 2 * Gs * N) * 4 + (size_t)nseq * Hs * N * pv * 8, k::decayed_state(s, dp));
+            k::GatedNormParams np{};
+            np.y = S.dn_o, np.ldy = inner, np.gate = S.q + z_col, np.ldgate = ldj, np.weight = X.ssd_norm, np.out = S.attn + H * vd, np.ldo = ldo_joint, np.eps = h.dn_norm_epsilon;
+            np.out_scale = h.pair_scale_second != 0.0f ? h.pair_scale_second : 1.0e-37f, np.rows = rows, np.width = inner, np.parts = h.ssd_norm_groups ? h.ssd_norm_groups : 1;
+            RUN("gated_norm_rows", (size_t)rows * inner * 12, k::gated_norm_rows(s, np));
+            if (forked && hipStreamWaitEvent(main_stream, S.side_join, 0) != hipSuccess && e.st == UZU_OK) set_error("engine: waiting for the side stream failed"), e.st = UZU_ERR_HIP;
+            run_linear(e, lin(S, X.joint_out, S.attn, S.tmp, rows)); // both halves' out projections, summed
+            add_normed(S.tmp, cur, slot, L.post_mixer, X.ls1, pre_mlp_fused ? &L.pre_mlp : (h.no_mlp && !h.has_ple) ? next_pre : nullptr);
+            normed_ready = h.no_mlp && !h.has_ple && next_pre;
+        } else if (h.pair_mixer) { // the second mixer beside the first: a delta rule with a decay per head and key channel, reading the same rows
             const uint32_t Hd = h.dn_num_heads, Gd = h.dn_num_groups, dk = h.dn_head_dim, dv = h.dn_value_head_dim, taps = h.dn_kernel_size, ldi = L.in_proj.n;
             const uint32_t conv_dim = 2 * Gd * dk + Hd * dv, b_col = conv_dim, a_col = b_col + Hd, g_col = a_col + h.dn_decay_rank;
             run_linear(e, lin(S, L.in_proj, mix_in, S.dn_in, rows)); // q | k | v | beta | decay down | gate down
@@ -534,12 +605,15 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                 const uzu_moe_desc& M = h.moe;
                 const uint32_t E = M.num_routed_experts, top = M.num_active_experts, ff = M.expert_hidden_dim;
                 const k::ExpertAct act = expert_act(M);
-                const float* res = hs ? nullptr : slot; // (hyper-connections: the launch that follows joins the result)
+                // (hyper-connections, a post norm: the launch that follows joins the result)
+                const float* res = hs || L.post_mlp.present ? nullptr : slot;
+                float* moe_out = L.post_mlp.present ? S.tmp : slot;
+                const bool on_input = M.weight_on_input != 0;
                 if (M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS) {
                     k::RouteGroupsParams rp{};
                     rp.x = mlp_in, rp.router = L.moe.router_weights, rp.selection_bias = X.selection_bias, rp.ids = S.moe_ids, rp.weights = S.moe_w, rp.rows = rows, rp.d = d, rp.outputs = E;
                     rp.top = top, rp.groups = M.router_groups ? M.router_groups : 1, rp.keep = M.router_groups_keep ? M.router_groups_keep : rp.groups, rp.bf16_products = bf;
-                    rp.scale = M.router_scale != 0.0f ? M.router_scale : 1.0f;
+                    rp.scale = M.router_scale != 0.0f ? M.router_scale : 1.0f, rp.raw = M.router_raw;
                     RUN("moe_route_groups", (size_t)E * d * 2, k::moe_route_groups(s, rp));
                 } else if (M.routing == UZU_MOE_ROUTE_SCORES) {
                     RUN("moe_route_scores", (size_t)(E + M.num_identity_experts) * d * 2,
@@ -548,15 +622,19 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
                     RUN("moe_route_topk", (size_t)E * d * 2, k::moe_route_topk(s, mlp_in, L.moe.router_weights, L.moe.router_biases, S.moe_ids, S.moe_w, rows, d, E, top, M.router_renorm));
                 }
                 k::MoeGroupedParams gp{};
-                gp.x = mlp_in, gp.ids = S.moe_ids, gp.weights = S.moe_w, gp.w13 = L.moe.w13, gp.w2 = L.moe.w2, gp.residual = res, gp.y = slot, gp.y1 = S.moe_y1, gp.hidden = S.hid;
+                gp.x = mlp_in, gp.ids = S.moe_ids, gp.weights = S.moe_w, gp.w13 = L.moe.w13, gp.w2 = L.moe.w2, gp.residual = res, gp.y = moe_out, gp.y1 = S.moe_y1, gp.hidden = S.hid;
                 gp.y2 = S.moe_y2, gp.perm = S.moe_perm, gp.slot_pos = S.moe_slot_pos, gp.offsets = S.moe_offsets, gp.cursor = S.moe_cursor;
-                gp.rows = rows, gp.d = d, gp.ff = ff, gp.routed = E, gp.top = top, gp.act = act;
+                gp.rows = rows, gp.d = d, gp.ff = ff, gp.routed = E, gp.top = top, gp.act = act, gp.pos_weight = on_input ? S.moe_pos_w : nullptr;
                 if (bf && k::moe_experts_grouped_supported(gp)) { // prefill-sized: buckets per expert through the matrix-core linear
                     RUN("moe_experts_grouped", (size_t)E * (act.plain ? 2 : 3) * ff * d * 2 + (size_t)rows * top * ((act.plain ? 1 : 3) * ff + 2 * d) * 4, k::moe_experts_grouped(s, gp));
                 } else {
-                    RUN("moe_experts_gate_up", (size_t)rows * top * (act.plain ? 1 : 2) * ff * d * 2, k::moe_experts_gate_up(s, mlp_in, S.moe_ids, L.moe.w13, S.hid, rows, d, ff, E, top, bf, act));
+                    RUN("moe_experts_gate_up", (size_t)rows * top * (act.plain ? 1 : 2) * ff * d * 2, k::moe_experts_gate_up(s, mlp_in, S.moe_ids, L.moe.w13, S.hid, rows, d, ff, E, top, bf, act, on_input ? S.moe_w : nullptr));
                     RUN("moe_experts_down_combine", (size_t)rows * top * ff * d * 2,
-                        k::moe_experts_down_combine(s, S.hid, mlp_in, S.moe_ids, S.moe_w, L.moe.w2, res, slot, rows, d, ff, E, top, bf));
+                        k::moe_experts_down_combine(s, S.hid, mlp_in, S.moe_ids, on_input ? nullptr : S.moe_w, L.moe.w2, res, moe_out, rows, d, ff, E, top, bf));
+                }
+                if (L.post_mlp.present) {
+                    add_normed(S.tmp, slot, slot, L.post_mlp, X.ls2, h.has_ple ? nullptr : next_pre);
+                    normed_ready = !h.has_ple && next_pre;
                 }
             } else {
                 if (h.mlp_plain) {
@@ -710,11 +788,12 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     auto full = [](const uzu_linear_desc& L, uint32_t n, uint32_t kk) { return L.weights && L.method == UZU_QUANT_NONE && L.n == n && L.k == kk && !L.input_signs && !L.output_signs && !L.lora_rank; };
     for (uint32_t l = 0; l < nl; ++l) {
         const uzu_layer_desc& h = desc->layers[l];
-        UZU_UNSUPPORTED(h.mixer_kind != UZU_MIXER_LATENT_ATTENTION && h.mixer_kind != UZU_MIXER_ATTENTION && h.mixer_kind != UZU_MIXER_RETENTION && h.mixer_kind != UZU_MIXER_GATED_LRU,
-                        "model_create: layer %u: an f32-stream design's mixer is latent attention, attention over cached keys and values, retention, or a gated linear recurrent unit "
-                        "(a channel-decay delta rule rides beside attention as the second mixer of a pair)", l);
-        UZU_UNSUPPORTED(h.mixer_kind != UZU_MIXER_ATTENTION && (h.qk_norm_whole || h.attention_chunk_size || h.values_are_keys || h.rel_bias_rows || h.head_temperature || h.pair_mixer),
-                        "model_create: layer %u: chunks, a distance bias, head temperatures, values that are keys, a whole-projection norm and a second mixer are options of attention", l);
+        UZU_UNSUPPORTED(h.mixer_kind != UZU_MIXER_LATENT_ATTENTION && h.mixer_kind != UZU_MIXER_ATTENTION && h.mixer_kind != UZU_MIXER_RETENTION && h.mixer_kind != UZU_MIXER_GATED_LRU &&
+                            h.mixer_kind != UZU_MIXER_GATED_LINEAR_ATTENTION,
+                        "model_create: layer %u: an f32-stream design's mixer is latent attention, attention over cached keys and values, retention, gated linear attention, or a gated "
+                        "linear recurrent unit (a channel-decay delta rule or a state-space mixer rides beside attention as the second mixer of a pair)", l);
+        UZU_UNSUPPORTED(h.mixer_kind != UZU_MIXER_ATTENTION && (h.qk_norm_whole || h.attention_chunk_size || h.values_are_keys || h.rel_bias_rows || h.head_temperature || h.pair_mixer || h.qkv_conv),
+                        "model_create: layer %u: convolved queries, keys and values, chunks, a distance bias, head temperatures, values that are keys, a whole-projection norm and a second mixer are options of attention", l);
         UZU_REQUIRE(!h.pre_mixer_norm.present || norm_ok(h.pre_mixer_norm), "model_create: layer %u: a pre-mixer norm is a dynamic-tanh or RMS norm (absent: the mixer reads the stream)", l);
         UZU_REQUIRE(groups_ok(h.pre_mixer_norm, d) && groups_ok(h.post_mixer_norm, d) && groups_ok(h.pre_mlp_norm, d) && groups_ok(h.post_mlp_norm, d),
                     "model_create: layer %u: a norm in parts is an RMS norm with a weight vector over model_dim %% groups == 0 coordinates", l);
@@ -730,15 +809,15 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
         UZU_UNSUPPORTED(!h.pre_mixer_norm.present && h.stream_reentry.weights, "model_create: layer %u: a re-entry projection in front of a mixer without a pre norm", l);
         UZU_UNSUPPORTED(h.token_shift && h.pre_mixer_norm.kind != UZU_NORM_DYNAMIC_TANH, "model_create: layer %u: the token shift follows a dynamic-tanh norm", l);
         UZU_REQUIRE(!h.post_mixer_norm.present || rms_vec(h.post_mixer_norm), "model_create: layer %u: a post-mixer norm is an RMS norm with a weight vector", l);
-        UZU_REQUIRE(!h.post_mlp_norm.present || (rms_vec(h.post_mlp_norm) && !h.no_mlp && h.mlp_kind != UZU_MLP_MOE && !h.parallel_block),
-                    "model_create: layer %u: a post-MLP norm is an RMS norm with a weight vector behind a dense block", l);
+        UZU_REQUIRE(!h.post_mlp_norm.present || (rms_vec(h.post_mlp_norm) && !h.no_mlp && !h.parallel_block),
+                    "model_create: layer %u: a post-MLP norm is an RMS norm with a weight vector behind an MLP of its own", l);
         UZU_REQUIRE((!h.layer_scale_mixer || h.post_mixer_norm.present) && (!h.layer_scale_mlp || h.post_mlp_norm.present), "model_create: layer %u: a layer scale follows a post norm", l);
         UZU_UNSUPPORTED(h.has_post_layer_scalar || h.normalize_values || h.is_non_causal, "model_create: layer %u: layer options of the bf16-stream families", l);
         if (h.weights_of_layer) {
             UZU_REQUIRE(h.weights_of_layer - 1 < l, "model_create: layer %u uses the tensors of run %u, which does not precede it", l, h.weights_of_layer - 1);
             const uzu_layer_desc& src = desc->layers[h.weights_of_layer - 1];
             UZU_REQUIRE(!src.weights_of_layer && src.mixer_kind == h.mixer_kind && src.qkv_projection.n == h.qkv_projection.n && src.out_projection.k == h.out_projection.k &&
-                        src.hidden_dim == h.hidden_dim && src.no_mlp == h.no_mlp && src.mlp_kind == h.mlp_kind && src.has_ple == h.has_ple && !h.is_kv_sharing && !src.is_kv_sharing &&
+                        src.pair_mixer == h.pair_mixer && src.qkv_conv_taps == h.qkv_conv_taps && src.hidden_dim == h.hidden_dim && src.no_mlp == h.no_mlp && src.mlp_kind == h.mlp_kind && src.has_ple == h.has_ple && !h.is_kv_sharing && !src.is_kv_sharing &&
                         (src.stream_reentry.weights != nullptr) == (h.stream_reentry.weights != nullptr),
                         "model_create: layer %u: a run that shares tensors has the shapes and options of the run that owns them", l);
         }
@@ -802,10 +881,25 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             UZU_REQUIRE(!h.values_are_keys || (h.value_head_dim == h.head_dim && !h.is_kv_sharing), "model_create: layer %u: values that are the key rows have the keys' width and a cache of their own", l);
             if (h.rel_bias_rows)
                 UZU_REQUIRE(h.rel_bias && (h.rel_bias_rows == 1 || h.rel_bias_max > (float)(h.rel_bias_rows / 2)), "model_create: layer %u: a distance bias [rows, heads] whose last bucket starts beyond rows / 2", l);
+            if (h.qkv_conv) {
+                UZU_REQUIRE(h.qkv_conv_taps >= 1 && h.qkv_conv_taps <= 64, "model_create: layer %u: a convolution of 1 .. 64 taps on queries, keys and values", l);
+                UZU_UNSUPPORTED(h.is_kv_sharing, "model_create: layer %u: convolved queries on another layer's cache", l);
+            }
             if (h.pair_mixer) {
-                const uint32_t Hd = h.dn_num_heads, Gd = h.dn_num_groups, dk = h.dn_head_dim, dv = h.dn_value_head_dim;
-                UZU_UNSUPPORTED(h.pair_mixer != 1 + UZU_MIXER_DELTA_NET || !h.dn_channel_decay, "model_create: layer %u: the second mixer of a pair is a delta rule with channel decays", l);
+                UZU_UNSUPPORTED(h.pair_mixer != 1 + UZU_MIXER_STATE_SPACE && (h.pair_mixer != 1 + UZU_MIXER_DELTA_NET || !h.dn_channel_decay),
+                                "model_create: layer %u: the second mixer of a pair is a delta rule with channel decays or a state-space mixer", l);
                 UZU_REQUIRE(h.post_mixer_norm.present && !h.parallel_block, "model_create: layer %u: a pair of mixers joins the stream behind a post-mixer norm", l);
+            }
+            if (h.pair_mixer == 1 + UZU_MIXER_STATE_SPACE) {
+                const uint32_t Hs = h.dn_num_heads, Gs = h.dn_num_groups, N = h.dn_head_dim, inner = Hs * h.dn_value_head_dim, parts = h.ssd_norm_groups ? h.ssd_norm_groups : 1;
+                UZU_REQUIRE(Hs && Gs && Hs % Gs == 0 && N && inner && h.dn_kernel_size >= 1 && h.dn_kernel_size <= 64 && inner % parts == 0,
+                            "model_create: layer %u: the state-space mixer's %u heads on %u groups, 1 .. 64 taps, %u coordinates normed in %u equal parts", l, Hs, Gs, inner, parts);
+                UZU_UNSUPPORTED(!k::decayed_state_supported(N, h.dn_value_head_dim), "model_create: layer %u: state-space heads of %u x %u", l, N, h.dn_value_head_dim);
+                UZU_REQUIRE(full(h.dn_in_proj, 2 * inner + 2 * Gs * N + Hs, d) && !h.dn_in_proj.out_biases && full(h.dn_out_proj, d, inner) && !h.dn_out_proj.out_biases && h.dn_conv_weights && h.dn_a_log &&
+                            h.dn_dt_bias && h.ssd_skip && h.dn_norm_scales, "model_create: layer %u: the state-space mixer's projection z | x | B | C | dt, out projection, convolution, a_log, dt_bias, skip and norm", l);
+                UZU_UNSUPPORTED(h.has_gate || h.is_kv_sharing || h.out_projection.out_biases, "model_create: layer %u: head gates, a shared cache and out-projection biases on attention beside a state-space mixer", l);
+            } else if (h.pair_mixer) {
+                const uint32_t Hd = h.dn_num_heads, Gd = h.dn_num_groups, dk = h.dn_head_dim, dv = h.dn_value_head_dim;
                 UZU_REQUIRE(Hd && Gd && Hd % Gd == 0 && dk && dv && h.dn_kernel_size >= 1 && h.dn_kernel_size <= 64 && h.dn_decay_rank && h.dn_gate_rank,
                             "model_create: layer %u: the delta rule's %u value heads on %u query / key heads, 1 .. 64 taps, low-rank decay and gate", l, Hd, Gd);
                 UZU_UNSUPPORTED(!k::channel_delta_supported(dk, dv), "model_create: layer %u: delta-rule heads of %u x %u (keys up to 256)", l, dk, dv);
@@ -824,6 +918,12 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                 UZU_REQUIRE(full(h.qkv_projection, h.num_heads * h.head_dim + h.num_groups * (h.head_dim + (h.values_are_keys ? 0 : h.value_head_dim)) + (h.has_gate ? h.num_heads : 0), d),
                             "model_create: layer %u: the packed projection must be a full-precision matrix [heads head_dim + groups (head_dim + value_head_dim) (+ heads gate rows), model_dim]", l);
             }
+        } else if (h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION) {
+            UZU_REQUIRE(h.dn_decay_rank && full(h.qkv_projection, 2 * h.num_heads * h.head_dim + 2 * h.num_heads * h.value_head_dim + h.dn_decay_rank, d) && !h.qkv_projection.out_biases &&
+                        full(h.dn_decay_up, h.num_heads * h.head_dim, h.dn_decay_rank) && h.dn_norm_scales && h.decay_temperature > 0.0f,
+                        "model_create: layer %u: gated linear attention's packed projection q | k | v | gate | decay down, decay up product, temperature and norm", l);
+            UZU_UNSUPPORTED(!k::decayed_state_supported(h.head_dim, h.value_head_dim), "model_create: layer %u: gated linear attention heads of %u x %u", l, h.head_dim, h.value_head_dim);
+            UZU_UNSUPPORTED(h.is_kv_sharing || h.sliding_window_size || h.has_sinks || h.unit_sink || h.score_soft_cap != 0.0f || h.use_rope, "model_create: layer %u: attention options on gated linear attention", l);
         } else if (h.mixer_kind == UZU_MIXER_RETENTION) {
             UZU_REQUIRE(full(h.qkv_projection, 2 * h.num_heads * h.head_dim + 2 * h.num_heads * h.value_head_dim, d) && !h.qkv_projection.out_biases,
                         "model_create: layer %u: a retention layer's packed projection is queries | keys | values | gate without biases", l);
@@ -844,6 +944,8 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                             M.num_active_experts <= M.num_routed_experts + M.num_identity_experts && M.router_weights &&
                             (M.num_routed_experts == 0 || (M.expert_hidden_dim && M.w13 && M.w2)) && M.gating_sel == 2 && !M.up_biases && !M.down_biases,
                             "model_create: layer %u: routed SiLU-gated experts without biases, with their router and expert tensors", l);
+                UZU_UNSUPPORTED(M.weight_on_input && (M.plain_experts || M.num_identity_experts), "model_create: layer %u: weights on the inputs of ungated or identity experts", l);
+                UZU_REQUIRE(!M.router_raw || M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS, "model_create: layer %u: raw scores as weights belong to sigmoid routing", l);
                 if (M.routing == UZU_MOE_ROUTE_SIGMOID_GROUPS) {
                     const uint32_t G = M.router_groups ? M.router_groups : 1, keep = M.router_groups_keep ? M.router_groups_keep : G;
                     UZU_REQUIRE(!M.num_identity_experts && !M.router_biases && M.num_routed_experts % G == 0 && keep <= G && M.num_active_experts <= M.num_routed_experts / G * keep,
@@ -884,15 +986,16 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     S.layers.resize(nl);
     uint32_t w_q = 0, w_rank = 0, w_lat = 0, w_attn = 0, w_hid = 0, w_top = 1, w_moe = 0, w_routed = 0, w_lru = 0, w_side = 0, w_y1 = 0;
     uint32_t w_dn_in = 0, w_dn_cv = 0, w_dn_k = 0, w_dn_v = 0;
-    bool any_pair = false, any_inconv = false, any_normed_conv = false;
-    uint32_t w_latq = 0;
+    bool any_pair = false, any_inconv = false, any_normed_conv = false, any_conv = false;
+    uint32_t w_latq = 0, w_pos = 0;
     for (uint32_t l = 0; l < nl; ++l) {
         const uzu_layer_desc& h = desc->layers[l];
         DLayer& L = m->layers[l];
         Stream32::Layer& X = S.layers[l];
         uint32_t kw_l = h.latent_rank + h.latent_rope_dim;
-        w_q = std::max(w_q, h.qkv_projection.n), w_rank = std::max({w_rank, h.latent_down.n ? h.latent_down.n : kw_l, h.latent_query_rank}), w_lat = std::max(w_lat, h.num_heads * kw_l);
-        w_attn = std::max(w_attn, std::max(h.num_heads * h.value_head_dim, h.lru_width)), w_lru = std::max(w_lru, h.lru_width), w_side = std::max(w_side, h.has_ple ? h.ple_dim : 0u);
+        const bool joint = h.pair_mixer == 1 + UZU_MIXER_STATE_SPACE;
+        w_q = std::max(w_q, (h.qkv_projection.n + (joint ? h.dn_in_proj.n : 0u) + 3) / 4 * 4), w_rank = std::max({w_rank, h.latent_down.n ? h.latent_down.n : kw_l, h.latent_query_rank}), w_lat = std::max(w_lat, h.num_heads * kw_l);
+        w_attn = std::max(w_attn, std::max(h.num_heads * h.value_head_dim + (joint ? h.dn_out_proj.k : 0u), h.lru_width)), w_lru = std::max(w_lru, h.lru_width), w_side = std::max(w_side, h.has_ple ? h.ple_dim : 0u);
         if (!h.no_mlp && h.mlp_kind != UZU_MLP_MOE) w_hid = std::max(w_hid, h.hidden_dim), w_y1 = std::max(w_y1, h.mlp_plain ? 0u : 2 * h.hidden_dim);
         if (h.weights_of_layer) { // the tensors of an earlier run: its device pointers, this run's own scalars; nothing is uploaded twice
             L = m->layers[h.weights_of_layer - 1];
@@ -902,7 +1005,7 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             any_normed_conv |= (h.pre_mixer_norm.present && h.input_conv_mixer) || (h.pre_mlp_norm.present && h.input_conv_mlp);
             if (!h.no_mlp && h.mlp_kind == UZU_MLP_MOE) {
                 const uzu_moe_desc& M = h.moe;
-                w_hid = std::max<uint32_t>(w_hid, M.num_active_experts * M.expert_hidden_dim), w_top = std::max(w_top, M.num_active_experts);
+                w_hid = std::max<uint32_t>(w_hid, M.num_active_experts * M.expert_hidden_dim), w_top = std::max(w_top, M.num_active_experts), w_pos = std::max(w_pos, M.weight_on_input ? M.num_active_experts : 0u);
                 w_moe = std::max(w_moe, M.num_active_experts * 2 * M.expert_hidden_dim), w_routed = std::max(w_routed, M.num_routed_experts);
             }
             continue;
@@ -952,7 +1055,45 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                 X.dist_rows = far + 1;
                 TRY(upload(m, tab.data(), tab.size() * 4, &X.dist_bias));
             }
-            if (h.pair_mixer) {
+            if (joint || h.qkv_conv) { // the convolution of q | k | v, and the state-space mixer's x | B | C behind it
+                const uint32_t nqkv = h.qkv_projection.n - (h.has_gate ? h.num_heads : 0), inner = joint ? h.dn_out_proj.k : 0, mixed = joint ? inner + 2 * h.dn_num_groups * h.dn_head_dim : 0;
+                const uint32_t C = nqkv + mixed, tl = h.qkv_conv ? h.qkv_conv_taps : 1, tr = joint ? h.dn_kernel_size : 1, taps = std::max(tl, tr);
+                std::vector<float> w((size_t)C * taps, 0.0f), b(C, 0.0f); // (a shorter filter: zero taps in front; no filter: the row itself)
+                for (uint32_t c = 0; c < nqkv; ++c)
+                    for (uint32_t j = 0; j < tl; ++j) w[(size_t)c * taps + taps - tl + j] = h.qkv_conv ? h.qkv_conv[(size_t)c * tl + j] : 1.0f;
+                for (uint32_t c = 0; c < mixed; ++c) {
+                    for (uint32_t j = 0; j < tr; ++j) w[((size_t)nqkv + c) * taps + taps - tr + j] = h.dn_conv_weights[(size_t)c * tr + j];
+                    if (h.dn_conv_biases) b[nqkv + c] = h.dn_conv_biases[c];
+                }
+                X.conv_channels = C, X.conv_taps = taps, X.conv_act_from = nqkv;
+                TRY(upload(m, w.data(), w.size() * 4, &X.conv_w));
+                if (joint && h.dn_conv_biases) TRY(upload(m, b.data(), b.size() * 4, &X.conv_b));
+                w_dn_cv = std::max(w_dn_cv, C);
+                any_conv = true;
+            }
+            if (joint) {
+                const uint32_t nqkv = h.qkv_projection.n, inner = h.dn_out_proj.k, mixed = inner + 2 * h.dn_num_groups * h.dn_head_dim, ni = h.dn_in_proj.n, ko = h.out_projection.k;
+                const uint16_t *in = (const uint16_t*)h.dn_in_proj.weights, *wl = (const uint16_t*)h.out_projection.weights, *wr = (const uint16_t*)h.dn_out_proj.weights;
+                std::vector<uint16_t> w((size_t)(nqkv + ni) * d), o((size_t)d * (ko + inner)), bias;
+                memcpy(w.data(), h.qkv_projection.weights, (size_t)nqkv * d * 2);
+                memcpy(&w[(size_t)nqkv * d], in + (size_t)inner * d, (size_t)mixed * d * 2);                                             // x | B | C
+                memcpy(&w[(size_t)(nqkv + mixed) * d], in, (size_t)inner * d * 2);                                                        // z
+                memcpy(&w[(size_t)(nqkv + mixed + inner) * d], in + (size_t)(inner + mixed) * d, (size_t)(ni - inner - mixed) * d * 2); // dt
+                for (uint32_t n = 0; n < d; ++n) {
+                    memcpy(&o[(size_t)n * (ko + inner)], wl + (size_t)n * ko, (size_t)ko * 2);
+                    memcpy(&o[(size_t)n * (ko + inner) + ko], wr + (size_t)n * inner, (size_t)inner * 2);
+                }
+                if (h.qkv_projection.out_biases) bias.assign((size_t)nqkv + ni, 0), memcpy(bias.data(), h.qkv_projection.out_biases, (size_t)nqkv * 2);
+                X.joint.n = nqkv + ni, X.joint.k = d, X.joint_out.n = d, X.joint_out.k = ko + inner;
+                TRY(upload(m, w.data(), w.size() * 2, &X.joint.w));
+                if (!bias.empty()) TRY(upload(m, bias.data(), bias.size() * 2, &X.joint.out_biases));
+                TRY(upload(m, o.data(), o.size() * 2, &X.joint_out.w));
+                TRY(upload(m, h.dn_a_log, (size_t)h.dn_num_heads * 4, &L.a_log));
+                TRY(upload(m, h.dn_dt_bias, (size_t)h.dn_num_heads * 4, &L.dt_bias));
+                TRY(upload(m, h.ssd_skip, (size_t)h.dn_num_heads * 4, &X.ssd_skip));
+                TRY(upload(m, h.dn_norm_scales, (size_t)inner * 4, &X.ssd_norm));
+                w_dn_v = std::max(w_dn_v, inner);
+            } else if (h.pair_mixer) {
                 const size_t conv_dim = 2 * (size_t)h.dn_num_groups * h.dn_head_dim + (size_t)h.dn_num_heads * h.dn_value_head_dim;
                 TRY(upload_linear(m, h.dn_in_proj, &L.in_proj));
                 TRY(upload_linear(m, h.dn_out_proj, &L.out_proj));
@@ -982,8 +1123,15 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             TRY(upload(m, h.lru_lambda, w * 4, &X.lru_lambda));
         }
         X.alpha1 = h.pre_mixer_norm.alpha;
-        TRY(upload_linear(m, h.qkv_projection, &L.qkv));
-        TRY(upload_linear(m, h.out_projection, &L.out));
+        if (!joint) {
+            TRY(upload_linear(m, h.qkv_projection, &L.qkv));
+            TRY(upload_linear(m, h.out_projection, &L.out));
+        }
+        if (h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION) {
+            TRY(upload_linear(m, h.dn_decay_up, &X.decay_up));
+            TRY(upload(m, h.dn_norm_scales, (size_t)h.value_head_dim * 4, &L.dn_norm));
+            w_dn_k = std::max(w_dn_k, h.num_heads * h.head_dim);
+        }
         if (h.mixer_kind == UZU_MIXER_RETENTION) TRY(upload(m, h.retention_decay, (size_t)h.num_heads * 4, &X.decay));
         if (h.unit_sink) { // a sink of logit 0 per head
             std::vector<float> f(h.num_heads, 0.0f);
@@ -1032,7 +1180,7 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
                 }
                 if (M.selection_bias) TRY(upload(m, M.selection_bias, (E + M.num_identity_experts) * 4, &X.selection_bias));
                 w_hid = std::max<uint32_t>(w_hid, M.num_active_experts * M.expert_hidden_dim);
-                w_top = std::max(w_top, M.num_active_experts);
+                w_top = std::max(w_top, M.num_active_experts), w_pos = std::max(w_pos, M.weight_on_input ? M.num_active_experts : 0u);
                 w_moe = std::max(w_moe, M.num_active_experts * 2 * M.expert_hidden_dim), w_routed = std::max(w_routed, M.num_routed_experts);
             } else {
                 if (h.activation == UZU_ACT_XIELU) {
@@ -1095,11 +1243,12 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     if (w_side) TRY(need_f32(m, R * w_side, &S.side_g));
     if (w_dn_in) {
         TRY(need_f32(m, R * w_dn_in, &S.dn_in));
-        TRY(need_f32(m, R * w_dn_cv, &S.dn_cv));
-        TRY(need_f32(m, R * w_dn_k, &S.dn_decay));
         TRY(need_f32(m, R * w_dn_v, &S.dn_gate));
-        TRY(need_f32(m, R * w_dn_v, &S.dn_o));
     }
+    if (w_dn_cv) TRY(need_f32(m, R * w_dn_cv, &S.dn_cv));
+    if (w_dn_k) TRY(need_f32(m, R * w_dn_k, &S.dn_decay));
+    if (w_dn_v) TRY(need_f32(m, R * w_dn_v, &S.dn_o));
+    if (w_pos && !S.full_f32) TRY(need_f32(m, R * w_pos, &S.moe_pos_w));
     TRY(need_f32(m, R * w_top, &S.moe_w));
     if (w_moe && !S.full_f32) { // workspaces of the grouped expert form (bf16 products only)
         void* q = nullptr;
@@ -1118,14 +1267,16 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
     TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(void*), &p)); S.d_cache_ptrs = (void**)p;
     TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(void*), &p)); S.d_cache2_ptrs = (void**)p;
     TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_shift_ptrs = (float**)p;
+    if (any_pair || any_conv) {
+        TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_pair_state_ptrs = (float**)p;
+        TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_pair_conv_ptrs = (float**)p;
+    }
     if (any_pair) {
         if (hipStreamCreateWithFlags(&S.side, hipStreamNonBlocking) != hipSuccess || hipEventCreateWithFlags(&S.side_fork, hipEventDisableTiming) != hipSuccess ||
             hipEventCreateWithFlags(&S.side_join, hipEventDisableTiming) != hipSuccess) {
             set_error("model_create: the side stream of a pair of mixers could not be created");
             return fail(UZU_ERR_HIP);
         }
-        TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_pair_state_ptrs = (float**)p;
-        TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_pair_conv_ptrs = (float**)p;
     }
     if (any_inconv) { TRY(dev_alloc(m, (size_t)nl * S.max_seqs * sizeof(float*), &p)); S.d_inconv_ptrs = (float**)p; }
     if (desc->bigram_buckets) { TRY(dev_alloc(m, S.max_seqs * sizeof(uint32_t*), &p)); S.d_prev_tok_ptrs = (uint32_t**)p; }
@@ -1145,6 +1296,14 @@ uzu_status s32_create(uzu_hip_context* ctx, const uzu_model_desc* desc, uint32_t
             S.ret_ws_bytes = std::max(S.ret_ws_bytes, k::retention_chunk_ws_bytes(S.max_rows / 64 + S.max_seqs, h.num_heads, h.head_dim, h.value_head_dim));
     }
     if (S.ret_ws_bytes) TRY(need_f32(m, S.ret_ws_bytes / 4, &S.ret_ws));
+    for (uint32_t l = 0; l < nl; ++l) {
+        const uzu_layer_desc& h = desc->layers[l];
+        if (h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION)
+            S.lin_ws_bytes = std::max(S.lin_ws_bytes, k::decayed_state_chunk_ws_bytes(S.max_rows / 64 + S.max_seqs, h.num_heads, h.head_dim, h.value_head_dim));
+        if (h.pair_mixer == 1 + UZU_MIXER_STATE_SPACE)
+            S.lin_ws_bytes = std::max(S.lin_ws_bytes, k::decayed_state_chunk_ws_bytes(S.max_rows / 64 + S.max_seqs, h.dn_num_heads, h.dn_head_dim, h.dn_value_head_dim));
+    }
+    if (S.lin_ws_bytes) TRY(need_f32(m, S.lin_ws_bytes / 4, &S.lin_ws));
     if (w_lru) {
         S.lru_ws_bytes = k::lru_piece_ws_bytes(S.max_rows / 32 + S.max_seqs, w_lru);
         TRY(need_f32(m, S.lru_ws_bytes / 4, &S.lru_ws));
@@ -1184,7 +1343,7 @@ uzu_status s32_state_layer(uzu_hip_model* m, uzu_hip_state* st, uint32_t l) {
     const uzu_layer_desc& h = m->layers[l].d;
     void* p = nullptr;
     const size_t elem = m->s32->full_f32 ? 4 : 2;
-    if (h.mixer_kind == UZU_MIXER_RETENTION) { // read only behind position 0, where the kernel starts from zeros: no fill needed
+    if (h.mixer_kind == UZU_MIXER_RETENTION || h.mixer_kind == UZU_MIXER_GATED_LINEAR_ATTENTION) { // read only behind position 0, where the kernel starts from zeros: no fill needed
         UZU_PROPAGATE(state_alloc(st, (size_t)h.num_heads * h.head_dim * h.value_head_dim * 4, &p, false));
         st->layers[l].ret_state = (float*)p;
     } else if (h.mixer_kind == UZU_MIXER_GATED_LRU) { // the state and the convolution's last taps - 1 inputs; both read only behind position 0
@@ -1210,8 +1369,12 @@ uzu_status s32_state_layer(uzu_hip_model* m, uzu_hip_state* st, uint32_t l) {
     if (h.pair_mixer) { // the second mixer's state and convolution window; both read only behind position 0
         UZU_PROPAGATE(state_alloc(st, (size_t)h.dn_num_heads * h.dn_head_dim * h.dn_value_head_dim * 4, &p, false));
         st->layers[l].ssm_state = (float*)p;
-        const size_t conv_dim = 2 * (size_t)h.dn_num_groups * h.dn_head_dim + (size_t)h.dn_num_heads * h.dn_value_head_dim;
-        UZU_PROPAGATE(state_alloc(st, conv_dim * (h.dn_kernel_size > 1 ? h.dn_kernel_size - 1 : 1) * 4, &p, false));
+    }
+    const Stream32::Layer& X = m->s32->layers[l];
+    if (h.pair_mixer || X.conv_w) { // (attention's own convolution and a state-space mixer's share one window)
+        const size_t conv_dim = X.conv_w ? X.conv_channels : 2 * (size_t)h.dn_num_groups * h.dn_head_dim + (size_t)h.dn_num_heads * h.dn_value_head_dim;
+        const uint32_t taps = X.conv_w ? X.conv_taps : h.dn_kernel_size;
+        UZU_PROPAGATE(state_alloc(st, conv_dim * (taps > 1 ? taps - 1 : 1) * 4, &p, false));
         st->layers[l].conv_state = (float*)p;
     }
     if ((h.input_conv_mixer || h.input_conv_mlp) && h.input_conv_taps > 1) { // the mixer's window, then the MLP's; read only behind position 0

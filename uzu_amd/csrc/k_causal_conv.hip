@@ -43,7 +43,7 @@ __global__ void __launch_bounds__(256) causal_conv_rows_kernel(CausalConvParams 
         else if (back <= t) xin = state[(size_t)(p.taps - 1 - (back - i)) * p.channels + c]; // in front of the pass: the state's rows are positions start - (taps - 1) .. start - 1
         acc = fmaf(p.w[(size_t)c * p.taps + j], xin, acc);
     }
-    if (p.act == 1) acc = acc / (1.0f + expf(-acc));
+    if (p.act == 1 && c >= p.act_from) acc = acc / (1.0f + expf(-acc));
     if (p.add_input) acc = own + acc;
     p.out[(size_t)r * p.ldo + p.o_col + c] = acc;
     if (sp.count == 1 && p.taps > 1) window_update(p, sp, z, c);
@@ -86,7 +86,7 @@ __global__ void __launch_bounds__(256) causal_conv_block_kernel(CausalConvParams
         }
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-            if (p.act == 1) acc[q] = acc[q] / (1.0f + expf(-acc[q]));
+            if (p.act == 1 && c + q >= p.act_from) acc[q] = acc[q] / (1.0f + expf(-acc[q]));
             if (p.add_input) acc[q] = past[0][q] + acc[q];
         }
         *(f32x4_v*)(p.out + (size_t)r * p.ldo + p.o_col + c) = acc;
@@ -125,7 +125,47 @@ __global__ void __launch_bounds__(256) head_norm_gate_kernel(HeadNormGateParams 
     }
 }
 
+// a workgroup per (row, part): the gated values stay in registers where a part is at most kGatedKeep steps of the workgroup; 256 strided partial sums, a fixed tree
+constexpr uint32_t kGatedKeep = 8;
+__global__ void __launch_bounds__(256) gated_norm_rows_kernel(GatedNormParams p) {
+    __shared__ float s_red[256];
+    const uint32_t r = blockIdx.x, w = p.width / p.parts, c0 = blockIdx.y * w, tid = threadIdx.x;
+    const float *y = p.y + (size_t)r * p.ldy + c0, *g = p.gate + (size_t)r * p.ldgate + c0, *wt = p.weight + c0;
+    float* out = p.out + (size_t)r * p.ldo + c0;
+    auto gated = [&](uint32_t i) { return y[i] * (g[i] / (1.0f + expf(-g[i]))); };
+    float keep[kGatedKeep], ss = 0.0f;
+#pragma unroll
+    for (uint32_t u = 0; u < kGatedKeep; ++u) {
+        const uint32_t i = tid + u * 256;
+        keep[u] = i < w ? gated(i) : 0.0f;
+        ss = fmaf(keep[u], keep[u], ss);
+    }
+    for (uint32_t i = tid + kGatedKeep * 256; i < w; i += 256) {
+        const float v = gated(i);
+        ss = fmaf(v, v, ss);
+    }
+    s_red[tid] = ss;
+    __syncthreads();
+    for (uint32_t h = 128; h > 0; h >>= 1) {
+        if (tid < h) s_red[tid] += s_red[tid + h];
+        __syncthreads();
+    }
+    const float inv = p.out_scale / sqrtf(s_red[0] / (float)w + p.eps);
+    for (uint32_t i = tid + kGatedKeep * 256; i < w; i += 256) out[i] = gated(i) * inv * wt[i]; // (out may be y: a thread replaces what it alone reads)
+#pragma unroll
+    for (uint32_t u = 0; u < kGatedKeep; ++u) {
+        const uint32_t i = tid + u * 256;
+        if (i < w) out[i] = keep[u] * inv * wt[i];
+    }
+}
+
 } // namespace
+
+uzu_status gated_norm_rows(hipStream_t s, const GatedNormParams& p) {
+    if (!p.rows) return UZU_OK;
+    UZU_REQUIRE(p.y && p.gate && p.weight && p.out && p.width && p.parts && p.parts <= 65535 && p.width % p.parts == 0, "gated_norm: %u coordinates in %u equal parts", p.width, p.parts);
+    return launch_check([&] { hipLaunchKernelGGL(gated_norm_rows_kernel, dim3(p.rows, p.parts), dim3(256), 0, s, p); }, "gated_norm_rows");
+}
 
 uzu_status causal_conv_rows(hipStream_t s, const CausalConvParams& p) {
     if (!p.rows) return UZU_OK;

@@ -523,12 +523,12 @@ __global__ void __launch_bounds__(1024) moe_route_groups_kernel(RouteGroupsParam
         sum += sc;
         if (t == lane) my_s = sc, my_id = (int32_t)best_e;
     }
-    if (lane < p.top) p.ids[out] = my_id, p.weights[out] = my_s / (sum + 1e-20f) * p.scale;
+    if (lane < p.top) p.ids[out] = my_id, p.weights[out] = (p.raw ? my_s : my_s / (sum + 1e-20f)) * p.scale;
 }
 
 // a workgroup per (row, slot): the row once into LDS, then a wave per hidden unit (gate and up rows of the unit in the same pass)
 __global__ void __launch_bounds__(256) moe_experts_gate_up_kernel(const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t d, uint32_t ff, uint32_t routed,
-                                                                  uint32_t top, uint32_t bf16_products, ExpertAct act) {
+                                                                  uint32_t top, uint32_t bf16_products, ExpertAct act, const float* in_weights) {
     extern __shared__ float s_x[];
     const uint32_t slot = blockIdx.x, r = slot / top;
     const int32_t e = ids[slot];
@@ -537,16 +537,17 @@ __global__ void __launch_bounds__(256) moe_experts_gate_up_kernel(const float* x
     __syncthreads();
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nw = blockDim.x >> 6;
     const uint16_t* base = w13 + (size_t)e * (act.plain ? 1 : 2) * ff * d;
+    const float wt = in_weights ? in_weights[slot] : 1.0f;
     for (uint32_t f = blockIdx.y * nw + wave; f < ff; f += gridDim.y * nw) {
         if (act.plain) { // no gate rows
-            const float v = fmaxf(wave_sum(lane_dot(s_x, base + (size_t)f * d, d, lane)), 0.0f);
+            const float v = fmaxf(wt * wave_sum(lane_dot(s_x, base + (size_t)f * d, d, lane)), 0.0f);
             if (lane == 0) hidden[(size_t)slot * ff + f] = v * v;
             continue;
         }
         const uint16_t* wu = base + (size_t)f * d;
         const uint16_t* wg = base + (size_t)(ff + f) * d;
         const float au = wave_sum(lane_dot(s_x, wu, d, lane)), ag = wave_sum(lane_dot(s_x, wg, d, lane));
-        if (lane == 0) hidden[(size_t)slot * ff + f] = expert_act(ag, au, act);
+        if (lane == 0) hidden[(size_t)slot * ff + f] = expert_act(wt * ag, wt * au, act);
     }
 }
 
@@ -568,7 +569,7 @@ __global__ void __launch_bounds__(256) moe_experts_down_kernel(const float* hidd
         float total = residual ? residual[(size_t)r * d + n] : 0.0f;
         for (uint32_t j = 0; j < top; ++j) {
             const int32_t e = ids[(size_t)r * top + j];
-            const float wt = weights[(size_t)r * top + j];
+            const float wt = weights ? weights[(size_t)r * top + j] : 1.0f;
             if (e < 0) continue;
             if ((uint32_t)e >= routed) { // identity expert: the block's input itself
                 total = fmaf(wt, x[(size_t)r * d + n], total);
@@ -591,7 +592,7 @@ __global__ void __launch_bounds__(256) moe_experts_down_rows_kernel(const float*
     float acc = 0.0f, same = 0.0f; // same: identity experts
     for (uint32_t j = 0; j < top; ++j) {
         const int32_t e = ids[(size_t)r * top + j];
-        const float wt = weights[(size_t)r * top + j];
+        const float wt = weights ? weights[(size_t)r * top + j] : 1.0f;
         if (e < 0) continue;
         if ((uint32_t)e >= routed) same = fmaf(wt, x[(size_t)r * d + n], same);
         else acc = fmaf(wt, lane_dot(hidden + ((size_t)r * top + j) * ff, w2 + ((size_t)e * d + n) * ff, ff, lane, bf16_products), acc);
@@ -621,7 +622,7 @@ __global__ void __launch_bounds__(1024) moe_bucket_kernel(const int32_t* ids, ui
 }
 // a pair's place inside its expert's bucket: the order of arrival (any order gives the same numbers: a row's product does not depend on its place in a tile)
 __global__ void __launch_bounds__(256) moe_scatter_kernel(const int32_t* ids, uint32_t slots, uint32_t routed, uint32_t top, const uint32_t* offsets, uint32_t* cursor, uint32_t* perm,
-                                                         uint32_t* slot_pos) {
+                                                         uint32_t* slot_pos, const float* weights, float* pos_weight) {
     const uint32_t i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= slots) return;
     const int32_t e = ids[i];
@@ -632,14 +633,16 @@ __global__ void __launch_bounds__(256) moe_scatter_kernel(const int32_t* ids, ui
     const uint32_t pos = offsets[e] + atomicAdd(&cursor[e], 1u);
     perm[pos] = i / top;
     slot_pos[i] = pos;
+    if (pos_weight) pos_weight[pos] = weights[i];
 }
-__global__ void __launch_bounds__(256) moe_act_mul_kernel(const float* y1, float* hidden, const uint32_t* offsets, uint32_t routed, uint32_t ff, ExpertAct act) {
+__global__ void __launch_bounds__(256) moe_act_mul_kernel(const float* y1, float* hidden, const uint32_t* offsets, uint32_t routed, uint32_t ff, ExpertAct act, const float* pos_weight) {
     const uint32_t pos = blockIdx.x;
     if (pos >= offsets[routed]) return;
     const float* src = y1 + (size_t)pos * 2 * ff;
+    const float wt = pos_weight ? pos_weight[pos] : 1.0f;
     for (uint32_t f = threadIdx.x; f < ff; f += blockDim.x) {
         const float g = src[ff + f];
-        hidden[(size_t)pos * ff + f] = expert_act(g, src[f], act);
+        hidden[(size_t)pos * ff + f] = expert_act(wt * g, wt * src[f], act);
     }
 }
 __global__ void __launch_bounds__(256) moe_combine_kernel(const float* y2, const float* x, const int32_t* ids, const float* weights, const uint32_t* slot_pos, const float* residual,
@@ -651,7 +654,7 @@ __global__ void __launch_bounds__(256) moe_combine_kernel(const float* y2, const
             const int32_t e = ids[(size_t)r * top + j];
             if (e < 0) continue;
             const float src = (uint32_t)e >= routed ? x[(size_t)r * d + n] : y2[(size_t)slot_pos[(size_t)r * top + j] * d + n];
-            total = fmaf(weights[(size_t)r * top + j], src, total);
+            total = fmaf(weights ? weights[(size_t)r * top + j] : 1.0f, src, total);
         }
         y[(size_t)r * d + n] = total;
     }
@@ -672,9 +675,10 @@ bool moe_experts_grouped_supported(const MoeGroupedParams& p) {
 
 uzu_status moe_experts_grouped(hipStream_t s, const MoeGroupedParams& p) {
     UZU_REQUIRE(moe_experts_grouped_supported(p), "moe_experts_grouped: shape not covered");
+    UZU_REQUIRE(!p.pos_weight || !p.act.plain, "moe_experts_grouped: weights on the inputs of plain experts");
     const uint32_t slots = p.rows * p.top;
     UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_bucket_kernel, dim3(1), dim3(1024), (size_t)p.routed * 4, s, p.ids, slots, p.routed, p.offsets, p.cursor); }, "moe_bucket"));
-    UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_scatter_kernel, dim3((slots + 255) / 256), dim3(256), 0, s, p.ids, slots, p.routed, p.top, p.offsets, p.cursor, p.perm, p.slot_pos); },
+    UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_scatter_kernel, dim3((slots + 255) / 256), dim3(256), 0, s, p.ids, slots, p.routed, p.top, p.offsets, p.cursor, p.perm, p.slot_pos, p.weights, p.pos_weight); },
                                "moe_scatter"));
     LinearF32Params q{};
     const uint32_t n1 = p.act.plain ? p.ff : 2 * p.ff;
@@ -682,12 +686,12 @@ uzu_status moe_experts_grouped(hipStream_t s, const MoeGroupedParams& p) {
     q.bf16_products = 1, q.row_offsets = p.offsets, q.row_map = p.perm;
     if (p.act.plain) q.y = p.hidden, q.act = 1; // no gate: the activation rides in the product's epilogue
     UZU_PROPAGATE(linear_mfma(s, q));
-    if (!p.act.plain) UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_act_mul_kernel, dim3(slots), dim3(256), 0, s, p.y1, p.hidden, p.offsets, p.routed, p.ff, p.act); }, "moe_act_mul"));
+    if (!p.act.plain) UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_act_mul_kernel, dim3(slots), dim3(256), 0, s, p.y1, p.hidden, p.offsets, p.routed, p.ff, p.act, p.pos_weight); }, "moe_act_mul"));
     LinearF32Params r{};
     r.x = p.hidden, r.w = p.w2, r.y = p.y2, r.rows = slots, r.n = p.d, r.k = p.ff, r.ldx = p.ff, r.ldy = p.d, r.batch = p.routed, r.w_batch = (size_t)p.d * p.ff;
     r.bf16_products = 1, r.row_offsets = p.offsets;
     UZU_PROPAGATE(linear_mfma(s, r));
-    return launch_check([&] { hipLaunchKernelGGL(moe_combine_kernel, dim3(p.rows), dim3(256), 0, s, p.y2, p.x, p.ids, p.weights, p.slot_pos, p.residual, p.y, p.d, p.routed, p.top); },
+    return launch_check([&] { hipLaunchKernelGGL(moe_combine_kernel, dim3(p.rows), dim3(256), 0, s, p.y2, p.x, p.ids, p.pos_weight ? nullptr : p.weights, p.slot_pos, p.residual, p.y, p.d, p.routed, p.top); },
                         "moe_combine");
 }
 
@@ -808,13 +812,13 @@ uzu_status moe_route_groups(hipStream_t s, const RouteGroupsParams& p) {
 }
 
 uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed,
-                               uint32_t top, uint32_t bf16_products, const ExpertAct& act) {
+                               uint32_t top, uint32_t bf16_products, const ExpertAct& act, const float* in_weights) {
     if (!rows || !routed) return UZU_OK;
     UZU_UNSUPPORTED((size_t)d * 4 > 48 * 1024, "moe_experts_gate_up: model_dim %u does not fit the workgroup's LDS row", d);
     // few (row, slot) pairs (decode): the hidden units of a pair are spread over more workgroups, so that the expert's rows stream through many CUs
     const uint32_t want = (1024 + rows * top - 1) / (rows * top), most = (ff + 3) / 4;
     const uint32_t gy = want < 1 ? 1 : (want > most ? most : want);
-    return launch_check([&] { hipLaunchKernelGGL(moe_experts_gate_up_kernel, dim3(rows * top, gy), dim3(256), (size_t)d * 4, s, x, ids, w13, hidden, d, ff, routed, top, bf16_products, act); },
+    return launch_check([&] { hipLaunchKernelGGL(moe_experts_gate_up_kernel, dim3(rows * top, gy), dim3(256), (size_t)d * 4, s, x, ids, w13, hidden, d, ff, routed, top, bf16_products, act, in_weights); },
                         "moe_experts_gate_up");
 }
 

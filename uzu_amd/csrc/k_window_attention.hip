@@ -172,13 +172,13 @@ __global__ void __launch_bounds__(64) window_attention_simple_kernel(WindowAtten
             acc[i] = sum;
         }
     }
-    float* o = p.out + ((size_t)r * p.heads + a) * p.vdim;
-    const float og = p.gate ? 1.0f / (1.0f + expf(-p.gate[(size_t)r * p.ldgate + a])) : 1.0f;
+    float* o = p.out + (size_t)r * p.ldo + (size_t)a * p.vdim;
+    const float og = p.gate ? p.out_scale / (1.0f + expf(-p.gate[(size_t)r * p.ldgate + a])) : p.out_scale;
 #pragma unroll
     for (uint32_t i = 0; i < kMaxVecPerLane; ++i) {
         const uint32_t c = lane + 64 * i;
         if (c >= p.vdim) break;
-        o[c] = p.gate ? acc[i] / l * og : acc[i] / l;
+        o[c] = acc[i] / l * og; // (og = 1: the value itself)
     }
 }
 
@@ -195,8 +195,12 @@ uzu_status rope_append(hipStream_t s, const RopeAppendParams& p) {
 
 uzu_status window_attention_mfma(hipStream_t s, const WindowAttentionParams& p); // k_window_attention_mfma.hip
 
-uzu_status window_attention(hipStream_t s, const WindowAttentionParams& p) {
+uzu_status window_attention(hipStream_t s, const WindowAttentionParams& params) {
+    WindowAttentionParams p = params;
     if (!p.rows) return UZU_OK;
+    if (!p.ldo) p.ldo = p.heads * p.vdim;
+    if (p.out_scale == 0.0f) p.out_scale = 1.0f;
+    UZU_REQUIRE(p.ldo >= p.heads * p.vdim, "window_attention: result rows of pitch %u", p.ldo);
     UZU_REQUIRE(p.q && p.out && p.key_caches && p.value_caches && p.spans && p.row_seq, "window_attention: null argument");
     UZU_REQUIRE(p.heads && p.kv_heads && p.heads % p.kv_heads == 0 && p.dim && p.vdim, "window_attention: %u query heads on %u key / value heads", p.heads, p.kv_heads);
     UZU_UNSUPPORTED(p.vdim > 64 * kMaxVecPerLane || p.dim > 8192, "window_attention: value width %u (at most %u)", p.vdim, 64 * kMaxVecPerLane);

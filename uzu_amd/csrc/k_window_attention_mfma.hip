@@ -180,9 +180,9 @@ __global__ void __launch_bounds__(256) window_attention_mfma_kernel(WindowAttent
         if (half == 0) ws[RP] = m_run, ws[RP + 1] = l_run;
         return;
     }
-    float inv = 1.0f / l_run;
+    float inv = p.out_scale / l_run;
     if (p.gate) inv *= 1.0f / (1.0f + expf(-p.gate[(size_t)(sp.row0 + row) * p.ldgate + head]));
-    float* out = p.out + ((size_t)(sp.row0 + row) * p.heads + head) * p.vdim;
+    float* out = p.out + (size_t)(sp.row0 + row) * p.ldo + (size_t)head * p.vdim;
 #pragma unroll
     for (int b = 0; b < NB; ++b)
 #pragma unroll
@@ -195,7 +195,7 @@ __global__ void __launch_bounds__(256) window_attention_mfma_kernel(WindowAttent
 // a workgroup per item: out = sum_s e^(m_s - M) O_s / sum_s e^(m_s - M) l_s over the splits, in split order (a split that saw no key has l = 0 and m = -1e30)
 // (gate: the item's result times sigmoid(gate[row, head]), item = row * heads + head)
 __global__ void __launch_bounds__(128) window_attention_merge_kernel(const float* ws, float* out, uint32_t splits, uint32_t vdim, uint32_t rp, const float* gate, uint32_t ldgate,
-                                                                     uint32_t heads) {
+                                                                     uint32_t heads, uint32_t ldo, float out_scale) {
     const uint32_t item = blockIdx.x, tid = threadIdx.x;
     const float* base = ws + (size_t)item * splits * (rp + 4);
     // the splits' weights once, a lane per split (at most 64 splits); the sums over the splits run in split order
@@ -213,7 +213,7 @@ __global__ void __launch_bounds__(128) window_attention_merge_kernel(const float
         float acc = 0.0f;
 #pragma unroll 8
         for (uint32_t s = 0; s < splits; ++s) acc = fmaf(s_w[s], base[(size_t)s * (rp + 4) + c], acc);
-        out[(size_t)item * vdim + c] = acc / den;
+        out[(size_t)(item / heads) * ldo + (size_t)(item % heads) * vdim + c] = acc / den * out_scale;
     }
 }
 
@@ -234,7 +234,7 @@ static bool use_split(const WindowAttentionParams& p) {
 
 bool window_attention_mfma_supported(const WindowAttentionParams& p) {
     const bool split = use_split(p);
-    return p.cache_bf16 && blocks_of(p) && p.dim % 8 == 0 && p.vdim % 8 == 0 && p.ldq % 4 == 0 && p.kv_heads && p.heads % p.kv_heads == 0 && p.nseq && p.tiles &&
+    return p.cache_bf16 && blocks_of(p) && p.dim % 8 == 0 && p.vdim % 8 == 0 && p.ldq % 4 == 0 && p.ldo % 4 == 0 && p.kv_heads && p.heads % p.kv_heads == 0 && p.nseq && p.tiles &&
            (split || p.rows >= 16 * p.nseq) && p.kv_heads <= 65535 && ((uintptr_t)p.q & 15) == 0 && ((uintptr_t)p.out & 15) == 0;
 }
 
@@ -249,7 +249,7 @@ uzu_status window_attention_mfma(hipStream_t s, const WindowAttentionParams& p) 
         else if (nb == 2) UZU_WA(2);
         else UZU_WA(4);
 #undef UZU_WA
-        return launch_check([&] { hipLaunchKernelGGL(window_attention_merge_kernel, dim3(p.rows * p.heads), dim3(128), 0, s, (const float*)p.split_ws, p.out, p.splits, p.vdim, 32 * nb, p.gate, p.ldgate, p.heads); },
+        return launch_check([&] { hipLaunchKernelGGL(window_attention_merge_kernel, dim3(p.rows * p.heads), dim3(128), 0, s, (const float*)p.split_ws, p.out, p.splits, p.vdim, 32 * nb, p.gate, p.ldgate, p.heads, p.ldo, p.out_scale); },
                             "window_attention_merge");
     }
     const dim3 grid(p.tiles, p.kv_heads);

@@ -9,6 +9,7 @@
 //   k_gated_lru.hip          the gated linear recurrent unit: short causal convolution over a carried window, gates / decays / state update
 //   k_causal_conv.hip        a causal per-channel convolution of row blocks over a carried window (sublayer inputs, the delta rule's q / k / v), per-head norm + gate
 //   k_channel_delta.hip      the gated delta rule with a decay per head and key channel
+//   k_decayed_state.hip      linear attention over a decayed outer-product state with decays from the data (per key channel, or per head with a step size)
 //   k_hyper.hip              hyper-connections: join a sublayer's result to the copies of the stream, read + norm (+ input convolution) the next sublayer's row
 #pragma once
 
@@ -132,14 +133,14 @@ uzu_status moe_route_topk(hipStream_t s, const float* x, const uint16_t* router,
                           uint32_t outputs, uint32_t top, uint32_t renorm);
 // Grouped sigmoid routing: per row s = sigmoid(router x) in f32 (bf16_products: x rounded to bf16 first), choice scores c = s + selection_bias (f32 [outputs] or null).  The outputs form
 // `groups` equal groups of neighbours; a group's strength is the sum of its two largest c (of its one, if it has one); only outputs of the `keep` strongest groups
-// can be chosen (ties: the lower group).  The `top` largest c among them win (ties: the lower index); weights = s / (sum of the winners' s + 1e-20) * scale.
+// can be chosen (ties: the lower group).  The `top` largest c among them win (ties: the lower index); weights = s / (sum of the winners' s + 1e-20) * scale, or (raw) s * scale.
 struct RouteGroupsParams {
     const float* x;
     const uint16_t* router;
     const float* selection_bias;
     int32_t* ids;
     float* weights;
-    uint32_t rows, d, outputs, top, groups, keep, bf16_products;
+    uint32_t rows, d, outputs, top, groups, keep, bf16_products, raw;
     float scale;
 };
 uzu_status moe_route_groups(hipStream_t s, const RouteGroupsParams& p);
@@ -155,15 +156,18 @@ struct ExpertAct {
 uzu_status gated_act_rows(hipStream_t s, const float* y1, float* hidden, uint32_t rows, uint32_t ff, const ExpertAct& act);
 
 // hidden[r * top + j, f] = act(gate_e x_r, up_e x_r) for e = ids[r, j] < routed; w13 bf16 [routed][2 ff][d], rows [0, ff) of an expert = up, [ff, 2 ff) = gate
+// in_weights (f32 [rows, top] or null): the expert reads in_weights[r, j] * x_r instead (both products are multiplied by it in front of the activation)
 uzu_status moe_experts_gate_up(hipStream_t s, const float* x, const int32_t* ids, const uint16_t* w13, float* hidden, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed,
-                               uint32_t top, uint32_t bf16_products, const ExpertAct& act = ExpertAct());
+                               uint32_t top, uint32_t bf16_products, const ExpertAct& act = ExpertAct(), const float* in_weights = nullptr);
 // y[r, :] = residual[r, :] + sum_j weights[r, j] * (ids[r, j] < routed ? down_e hidden[r * top + j] : x[r, :])   in slot order; w2 bf16 [routed][d][ff]; y may alias residual
+// (weights null: 1)
 uzu_status moe_experts_down_combine(hipStream_t s, const float* hidden, const float* x, const int32_t* ids, const float* weights, const uint16_t* w2, const float* residual,
                                     float* y, uint32_t rows, uint32_t d, uint32_t ff, uint32_t routed, uint32_t top, uint32_t bf16_products);
 
 // The same block for prefill-sized row counts with bf16 products: the (row, slot) pairs are bucketed by expert (counts -> offsets -> positions), every expert runs
 // its bucket through the matrix-core linear as one grouped launch (gate | up, then down), and the rows are combined in slot order.  Workspaces: y1
 // [rows * top][2 ff], hidden [rows * top][ff], y2 [rows * top][d] f32; perm / slot_pos [rows * top], offsets [routed + 1], cursor [routed] u32.
+// pos_weight (f32 [rows * top] or null): the winners' weights multiply the experts' inputs instead of their results (not with plain experts).
 struct MoeGroupedParams {
     const float* x;
     const int32_t* ids;
@@ -171,7 +175,7 @@ struct MoeGroupedParams {
     const uint16_t *w13, *w2;
     const float* residual;
     float* y;
-    float *y1, *hidden, *y2;
+    float *y1, *hidden, *y2, *pos_weight;
     uint32_t *perm, *slot_pos, *offsets, *cursor;
     uint32_t rows, d, ff, routed, top;
     ExpertAct act;
@@ -301,6 +305,9 @@ struct WindowAttentionParams {
     uint32_t dist_rows;
     const float* gate;
     uint32_t ldgate;
+    // ldo: row pitch of `out` (0 = heads * vdim); out_scale: everything above times it (0 = 1)
+    uint32_t ldo;
+    float out_scale;
     uint32_t form;  // 0: chosen by shape; 1: the simple form (a wave per row and head); 2: the matrix-core form
     uint32_t nseq;  // entries of `spans`
     uint32_t tiles; // sum over the sequences of ceil(count * (heads / kv_heads) / 128): the matrix-core form's item tiles (the caller knows the counts)
@@ -412,7 +419,7 @@ uzu_status lru_scan(hipStream_t s, const GatedLruParams& p);
 //   out[r, o_col + c] = act(bias[c] + sum_j w[c, j] * xin(t - (taps - 1) + j, c))  (+ x[r, x_col + c] with add_input: a sublayer that reads h + conv(h))
 // xin = channel c of the sequence's input rows `x` (f32, pitch ldx, column x_col): of this pass, or (in front of the pass) the taps - 1 inputs the state keeps
 // (states[z] + state_offset: f32 [taps - 1][channels], oldest first), or zero in front of position 0.  w f32 [channels][taps]: the last tap weighs the row itself.
-// act: 0 none, 1 silu.  `out` is another block of rows than `x`.  causal_conv_commit leaves the last taps - 1 inputs behind the pass in the state; it reads the
+// act: 0 none, 1 silu, on the channels from act_from on.  `out` is another block of rows than `x`.  causal_conv_commit leaves the last taps - 1 inputs behind the pass in the state; it reads the
 // same `x`, which must still hold the pass's inputs.  A sequence that brings one row has its window replaced by causal_conv_rows itself; max_count (the longest
 // share of the pass, 0 = unknown) == 1 makes causal_conv_commit a no-op.
 struct CausalConvParams {
@@ -421,7 +428,7 @@ struct CausalConvParams {
     float* out;
     uint32_t ldo, o_col;
     const float *w, *bias;
-    uint32_t channels, taps, add_input, act;
+    uint32_t channels, taps, add_input, act, act_from;
     float* const* states; // device array [nseq]
     size_t state_offset;  // floats
     const SeqSpan* spans;
@@ -443,6 +450,19 @@ struct HeadNormGateParams {
     uint32_t rows, heads, width;
 };
 uzu_status head_norm_gate_rows(hipStream_t s, const HeadNormGateParams& p);
+
+// The gate in front of the norm, the norm in `parts` equal consecutive parts of the row:  u = y * silu(gate),  out[r, i] = u[i] / sqrt(mean over i's part of u^2 + eps) *
+// weight[i] * out_scale   (y / gate / out: f32 rows of pitch ldy / ldgate / ldo, `width` used; weight f32 [width]; out may be y)
+struct GatedNormParams {
+    const float* y;
+    const float* gate;
+    const float* weight;
+    float* out;
+    uint32_t ldy, ldgate, ldo;
+    float eps, out_scale;
+    uint32_t rows, width, parts;
+};
+uzu_status gated_norm_rows(hipStream_t s, const GatedNormParams& p);
 
 // The gated delta rule with a decay per head and key channel (k_channel_delta.hip).  Row r (sequence z) of `qkv` (f32, pitch ld) holds queries [groups][dim] at
 // q_col, keys [groups][dim] at k_col and values [heads][vdim] at v_col (behind their convolution and silu); value head a reads group a / (heads / groups).
@@ -468,6 +488,35 @@ struct ChannelDeltaParams {
 bool channel_delta_supported(uint32_t dim, uint32_t vdim);
 uzu_status channel_delta_prep(hipStream_t s, const ChannelDeltaParams& p);
 uzu_status channel_delta(hipStream_t s, const ChannelDeltaParams& p);
+
+// Linear attention over a decayed outer-product state, decays from the data (k_decayed_state.hip).  Row r (sequence z) of `rows_in` (f32, pitch ld) holds queries
+// [groups][dim] at q_col, keys [groups][dim] at k_col and values [heads][vdim] at v_col; head a reads group a / (heads / groups).  Row after row, per head:
+//   S <- diag(decay) S + step k v^T  (S [dim][vdim], rows = key channels),   out[r, a, :] = q_scale S^T q + skip[a] v       (skip f32 [heads] or null)
+// per_head == 0:  decay[c] = sigmoid(pre[r, a dim + c])^inv_temperature, step = 1                     pre = `decay`, f32 rows of pitch lddecay
+// per_head != 0:  step = softplus(pre[r, a] + dt_bias[a]), decay = exp(-exp(a_log[a]) step) for every channel
+// states: device array [nseq] of pointers to f32 [heads][dim][vdim], read at the pass's first row (zeros instead when the span starts at position 0) and left
+// behind its last.  All f32.  form 0: chosen by the row count; 1: token by token; 2: in chunks of 64 rows (differs from form 1 by f32 rounding only; needs
+// chunks = sum over the sequences of ceil(count / 64) and a workspace of decayed_state_chunk_ws_bytes(chunks, heads, dim, vdim) bytes, without which form 0 goes
+// token by token).
+struct DecayedStateParams {
+    const float* rows_in;
+    uint32_t ld, q_col, k_col, v_col;
+    const float* decay;
+    uint32_t lddecay, per_head;
+    float inv_temperature;
+    const float *a_log, *dt_bias, *skip;
+    float q_scale;
+    float* out; // [rows][heads * vdim]
+    float* const* states;
+    const SeqSpan* spans;
+    uint32_t nseq, rows, heads, groups, dim, vdim;
+    uint32_t form, chunks;
+    float* chunk_ws;
+    size_t chunk_ws_bytes;
+};
+size_t decayed_state_chunk_ws_bytes(uint32_t chunks, uint32_t heads, uint32_t dim, uint32_t vdim);
+bool decayed_state_supported(uint32_t dim, uint32_t vdim);
+uzu_status decayed_state(hipStream_t s, const DecayedStateParams& p);
 
 } // namespace k
 } // namespace uzu

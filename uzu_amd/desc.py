@@ -18,7 +18,7 @@ import numpy as np
 # enums (uzu_model_desc.h)
 QUANT_SCALE_BIAS, QUANT_SCALE_ZERO_POINT, QUANT_SCALE_SYMMETRIC, QUANT_NONE = 0, 1, 2, 3
 ACT_SILU, ACT_GELU_APPROX, ACT_GELU_EXACT, ACT_IDENTITY, ACT_SOFTPLUS, ACT_RELU_SQUARED, ACT_XIELU = 0, 1, 2, 3, 4, 5, 6
-MIXER_ATTENTION, MIXER_DELTA_NET, MIXER_LATENT_ATTENTION, MIXER_RETENTION, MIXER_GATED_LRU = 0, 1, 2, 3, 4
+MIXER_ATTENTION, MIXER_DELTA_NET, MIXER_LATENT_ATTENTION, MIXER_RETENTION, MIXER_GATED_LRU, MIXER_GATED_LINEAR_ATTENTION, MIXER_STATE_SPACE = 0, 1, 2, 3, 4, 5, 6
 NORM_STATISTICS, NORM_DYNAMIC_TANH, NORM_RMS_SCALAR = 0, 1, 2
 MOE_ROUTE_TOPK_LOGITS, MOE_ROUTE_SCORES, MOE_ROUTE_SIGMOID_GROUPS = 0, 1, 2
 ROPE_NONE, ROPE_UNSCALED, ROPE_LLAMA, ROPE_LINEAR, ROPE_YARN, ROPE_LONGROPE = 0, 1, 2, 3, 4, 5
@@ -64,7 +64,8 @@ class MoeDesc(C.Structure):
         ("router_weights", C.c_void_p), ("router_biases", C.c_void_p), ("w13", C.c_void_p), ("w2", C.c_void_p), ("up_biases", C.c_void_p), ("down_biases", C.c_void_p),
         ("routing", C.c_uint32), ("num_identity_experts", C.c_uint32), ("selection_bias", C.c_void_p),
         ("up_offset", C.c_float), ("plain_experts", C.c_uint32),
-        ("router_groups", C.c_uint32), ("router_groups_keep", C.c_uint32), ("router_scale", C.c_float), ("reserved", C.c_uint32),
+        ("router_groups", C.c_uint32), ("router_groups_keep", C.c_uint32), ("router_scale", C.c_float), ("router_raw", C.c_uint32),
+        ("weight_on_input", C.c_uint32), ("reserved", C.c_uint32),
     ]
 
 
@@ -112,6 +113,7 @@ class LayerDesc(C.Structure):
         ("dn_channel_decay", C.c_uint32), ("dn_decay_rank", C.c_uint32), ("dn_gate_rank", C.c_uint32), ("dn_decay_up", LinearDesc), ("dn_gate_up", LinearDesc),
         ("latent_query_rank", C.c_uint32), ("gate_elementwise", C.c_uint32), ("latent_query_norm", NormDesc), ("latent_query_up", LinearDesc),
         ("xielu_p", C.c_float), ("xielu_q", C.c_float), ("hyper_mixer", C.c_void_p), ("hyper_mlp", C.c_void_p),
+        ("qkv_conv", C.c_void_p), ("qkv_conv_taps", C.c_uint32), ("decay_temperature", C.c_float), ("ssd_skip", C.c_void_p), ("ssd_norm_groups", C.c_uint32), ("reserved_tail", C.c_uint32),
     ]
 
 
@@ -256,12 +258,15 @@ class MoeWeights:
     router_groups: int = 1
     router_groups_keep: int = 1
     router_scale: float = 1.0
+    router_raw: bool = False       # ... weights = the winners' scores themselves (times router_scale)
+    weight_on_input: bool = False  # a winner's weight multiplies its expert's input instead of its output
 
     def desc(self) -> MoeDesc:
         return MoeDesc(self.num_routed_experts, self.num_active_experts, self.expert_hidden_dim, int(self.router_renorm), self.gating_sel, self.silu_alpha,
                        self.gate_clip[0], self.gate_clip[1], self.up_clip[0], self.up_clip[1], _ptr(self.router_weights), _ptr(self.router_biases), _ptr(self.w13),
                        _ptr(self.w2), _ptr(self.up_biases), _ptr(self.down_biases), int(self.routing), int(self.num_identity_experts), _ptr(self.selection_bias),
-                       float(self.up_offset), int(self.plain_experts), int(self.router_groups), int(self.router_groups_keep), float(self.router_scale), 0)
+                       float(self.up_offset), int(self.plain_experts), int(self.router_groups), int(self.router_groups_keep), float(self.router_scale), int(self.router_raw),
+                       int(self.weight_on_input), 0)
 
     def nbytes_active(self) -> int:
         """bytes one decoded token streams: the router + the k active experts' matrices and biases"""
@@ -382,13 +387,19 @@ class LayerWeights:
     # hyper-connections (ModelBundle.hyper_streams = s): f32 [s + s + s s] = in | out | mix[from, to] of each sublayer
     hyper_mixer: Optional[np.ndarray] = None
     hyper_mlp: Optional[np.ndarray] = None
+    # attention: a causal convolution over positions on the packed queries, keys and values, f32 [rows, taps], in front of norms and rotation
+    qkv_conv: Optional[np.ndarray] = None
+    decay_temperature: float = 0.0                 # gated linear attention (MIXER_GATED_LINEAR_ATTENTION): decay = sigmoid(.)^(1 / temperature)
+    # state-space mixer (MIXER_STATE_SPACE as pair_mixer; the dn_* fields: dn_head_dim = state width, dn_norm_scales [heads width], dn_dt_bias [heads])
+    ssd_skip: Optional[np.ndarray] = None          # f32 [heads]
+    ssd_norm_groups: int = 0
 
     def _moe_desc(self) -> MoeDesc:
         if self.moe is not None:
             return self.moe.desc()
         if self.gated_act is not None:
             slope, gate, up, off = self.gated_act
-            return MoeDesc(0, 0, 0, 0, 2, float(slope), float(gate[0]), float(gate[1]), float(up[0]), float(up[1]), None, None, None, None, None, None, 0, 0, None, float(off), 0, 0, 0, 0.0, 0)
+            return MoeDesc(0, 0, 0, 0, 2, float(slope), float(gate[0]), float(gate[1]), float(up[0]), float(up[1]), None, None, None, None, None, None, 0, 0, None, float(off), 0, 0, 0, 0.0, 0, 0, 0)
         return MoeDesc()
 
     def desc(self) -> LayerDesc:
@@ -429,6 +440,7 @@ class LayerWeights:
             ld(self.dn_decay_up), ld(self.dn_gate_up),
             0 if self.latent_query_up is None else int(self.latent_query_up.k), int(self.gate_elementwise), self.latent_query_norm.desc(), ld(self.latent_query_up),
             float(self.xielu[0]), float(self.xielu[1]), _ptr(self.hyper_mixer), _ptr(self.hyper_mlp),
+            _ptr(self.qkv_conv), 0 if self.qkv_conv is None else int(self.qkv_conv.shape[1]), float(self.decay_temperature), _ptr(self.ssd_skip), int(self.ssd_norm_groups), 0,
         )
 
     def linears(self):
@@ -657,11 +669,13 @@ class ModelBundle:
                 if l.attention_chunk_size:  # at most the row's own chunk
                     rows = min(rows, l.attention_chunk_size)
                 total += rows * l.num_groups * (l.head_dim + (l.value_head_dim or l.head_dim)) * 2  # K and V rows, bf16 (a sharing layer reads its source's)
-                if l.pair_mixer is not None:  # the delta rule beside it: f32 state read + write, the convolution's window and taps
+                if l.pair_mixer is not None:  # the recurrent mixer beside it: f32 state read + write, the convolution's window and taps
                     total += 2 * l.dn_num_heads * l.dn_value_head_dim * l.dn_head_dim * 4
                     conv_dim = 2 * l.dn_num_groups * l.dn_head_dim + l.dn_num_heads * l.dn_value_head_dim
                     total += conv_dim * (3 * l.dn_kernel_size - 2) * 4
-            elif l.mixer_kind == MIXER_RETENTION:
+                if l.qkv_conv is not None:
+                    total += l.qkv_conv.shape[0] * (3 * l.qkv_conv.shape[1] - 2) * 4
+            elif l.mixer_kind in (MIXER_RETENTION, MIXER_GATED_LINEAR_ATTENTION):
                 total += 2 * l.num_heads * l.head_dim * l.value_head_dim * 4  # f32 state read + write
             elif l.mixer_kind == MIXER_LATENT_ATTENTION:
                 rows = min(context, l.sliding_window_size) if l.sliding_window_size else context
@@ -699,11 +713,11 @@ class ModelBundle:
                 if l.attention_chunk_size:  # a row sees (chunk + 1) / 2 keys of its own chunk on average
                     vis = min(vis, tokens * (l.attention_chunk_size + 1) / 2.0)
                 flops += 2.0 * vis * l.num_heads * (l.head_dim + l.value_head_dim)
-                if l.pair_mixer is not None:  # the delta rule beside it: ~6 flops per state element per token (decay, S k, rank-1 update, S q)
-                    flops += 6.0 * tokens * l.dn_num_heads * l.dn_value_head_dim * l.dn_head_dim
+                if l.pair_mixer is not None:  # the recurrent mixer beside it: ~6 flops per state element per token for a delta rule (decay, S k, rank-1 update, S q), 4 without S k
+                    flops += (4.0 if l.pair_mixer == MIXER_STATE_SPACE else 6.0) * tokens * l.dn_num_heads * l.dn_value_head_dim * l.dn_head_dim
             elif l.mixer_kind == MIXER_ATTENTION:
                 flops += 4.0 * pairs * l.num_heads * l.head_dim
-            elif l.mixer_kind == MIXER_RETENTION:  # per token and head: the outer-product update and the read-out of the state
+            elif l.mixer_kind in (MIXER_RETENTION, MIXER_GATED_LINEAR_ATTENTION):  # per token and head: the outer-product update and the read-out of the state
                 flops += 4.0 * tokens * l.num_heads * l.head_dim * l.value_head_dim
             elif l.mixer_kind == MIXER_LATENT_ATTENTION:  # scores and weighted sum in latent space, over the window
                 w = l.sliding_window_size

@@ -1,4 +1,4 @@
-"""What the readers of designs with their own ``config.json`` schema (uzu_amd.lazolix, relulix, begasun, zovolorn, dironex) share: bf16 tensors of a safetensors file by name with
+"""What the readers of designs with their own ``config.json`` schema (uzu_amd.lazolix, relulix, begasun, zovolorn, dironex, rilavik) share: bf16 tensors of a safetensors file by name with
 shape checks, bf16 bit patterns, and a full-precision linear of the engine's description."""
 from __future__ import annotations
 
