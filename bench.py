@@ -12,7 +12,7 @@ Prints ONE JSON line on rank 0 with two extra o
   roofline     -- the dominant kernel (the int4 GEMV family) : algorithmic bytes / HIP-event time, vs 8 TB/s HBM
   cpu_baseline -- the CPU oracle (port of the reference's single-threaded CPU backend) timed on this host
 
-Side runs (their own JSON line, never the headline): --config c3|c4|c5, --exact, and --design lazolix | relulix | begasun | zovolorn | dironex (prefill / chained decode / batched
+Side runs (their own JSON line, never the headline): --config c3|c4|c5, --exact, and --design lazolix | relulix | begasun | zovolorn | dironex | rilavik (prefill / chained decode / batched
 decode of an f32-stream design at real layer sizes beside the engine's closest existing model at equal sizes).
 """
 import argparse
@@ -59,13 +59,14 @@ def parse_args():
                     help="BASELINE.json configs[1..4]: c2 (default, the headline) Qwen3.5-0.8B int4 ctx-2048 decode; c3 Llama-3-8B int4, 4k prefill x 8 "
                          "sequences in batched passes (prefill tokens/s, MFMA roofline); c4 Llama-3-8B int8 decode (TP = --gpus); c5 Qwen3-14B-class int4 at "
                          "ctx 8192, one sequence decoding while another is prefilled (TP = --gpus)")
-    ap.add_argument("--design", choices=["", "lazolix", "relulix", "begasun", "zovolorn", "dironex"], default="", help="side runs of a design outside BASELINE.json (never the headline): `lazolix` times prefill, "
+    ap.add_argument("--design", choices=["", "lazolix", "relulix", "begasun", "zovolorn", "dironex", "rilavik"], default="", help="side runs of a design outside BASELINE.json (never the headline): `lazolix` times prefill, "
                     "chained decode and batched decode of the f32-stream design at layer sizes of real models (random weights), beside the closest "
                     "bf16-stream model of the engine at equal sizes (windowed attention with sinks + int4 dense / bf16 expert MLPs); `relulix` does the same for the "
                     "design of parallel blocks with rotated attention, retention layers and clamped experts, beside Lazolix with experts at equal sizes; `begasun` for the looped stack of recurrent units, latent attention with a rotated key part "
                     "and grouped attention, beside Lazolix with dense blocks at equal sizes; `zovolorn` for the pairs of chunked attention + channel-decay delta rule alternating with grouped attention, "
                     "beside Begasun's recurrent units alternating with grouped attention at equal sizes; `dironex` for hyper-connected latent attention (a query latent, a rotated key part) and windowed grouped "
-                    "attention with xIELU dense blocks and ungated experts, beside Lazolix with the same pattern of dense blocks and experts at equal sizes")
+                    "attention with xIELU dense blocks and ungated experts, beside Lazolix with the same pattern of dense blocks and experts at equal sizes; `rilavik` for convolved windowed attention beside a "
+                    "state-space mixer and gated linear attention with score-scaled experts, beside Relulix (attention, retention, experts) and Zovolorn's pairs at equal sizes")
     ap.add_argument("--design-sizes", default="w1024,w2048", help="--design: comma-separated size presets")
     ap.add_argument("--sequences", type=int, default=8, help="c3: sequences per batched prefill pass")
     ap.add_argument("--prompt", type=int, default=4096, help="c3: prompt tokens per sequence")
@@ -716,8 +717,57 @@ def bench_dironex(args):
     print(json.dumps(out), flush=True)
 
 
+def rilavik_bundles(z, context):
+    """a Rilavik model and the two existing models closest to it at the sizes `z` (see bench_rilavik)"""
+    import tempfile
+    from uzu_amd import loader, relulix, rilavik, zovolorn
+    H, G, dim, vd, window = z["heads"], max(1, z["heads"] // 4), z["dim"], z["vdim"], z["window"]
+
+    def bundle(design, cfg):
+        with tempfile.TemporaryDirectory() as tmp:
+            design.save(tmp, cfg, design.random_tensors(cfg, seed=1))
+            return loader.load_model_dir(tmp, max_context_length=context)
+    mlp = rilavik.moe_mlp(z["experts"], z["top"], z["eff"])
+    par = rilavik.parallel_layer(rilavik.attention_half(H, G, dim, vd, window, conv=4, rot_dims=dim, rot_base=500000.0, factor=8.0),
+                                 rilavik.state_space_half(z["width"] // 64, 64, 128, groups=2, norm_groups=2, conv=4), 0.8, 1.1, mlp=mlp)
+    gla = rilavik.gla_layer(H, dim, vd, rank=16, mlp=mlp)
+    out = {"rilavik": bundle(rilavik, rilavik.config(z["vocab"], z["width"], ([par, par, par, gla] * ((z["layers"] + 3) // 4))[:z["layers"]]))}
+    rmlp = relulix.moe_mlp(z["experts"], z["top"], z["eff"], limit=7.0)
+    att = relulix.attention_layer(H, G, dim, vd, relulix.rotation(dim, 500000.0), window=window, softcap=30.0, mlp=rmlp)
+    ret = relulix.retention_layer(H, dim, vd, relulix.rotation(dim, 1e6), [1.0 - 2.0 ** -(5 + (a % 6)) for a in range(H)], mlp=rmlp)
+    out["closest"] = bundle(relulix, relulix.config(z["vocab"], z["width"], ([att, att, att, ret] * ((z["layers"] + 3) // 4))[:z["layers"]]))
+    zmlp = zovolorn.dense_mlp(z["top"] * z["eff"])  # the active experts' width
+    zpar = zovolorn.parallel_layer(H, G, dim, window, 32, 2048.0, z["width"] // 64, 2, 128, 64, 4, rank=16, left_scale=0.8, right_scale=1.1, mlp=zmlp)
+    out["closest_pairs"] = bundle(zovolorn, zovolorn.config(z["vocab"], z["width"], [zpar] * z["layers"], taps=4))
+    return out
+
+
+def bench_rilavik(args):
+    """Prefill / decode throughput of Rilavik models (three layers of convolved windowed attention beside a state-space mixer, one of gated linear attention; experts that
+    read their input times the router's score) beside the closest existing models at equal size: Relulix (three windowed attention layers, one of retention; clamped routed
+    experts; same width / heads / head widths / window / experts / vocabulary / layer count -- its layers have no second mixer) and Zovolorn (pairs of attention and a
+    channel-decay delta rule with heads and state of the state-space mixer's sizes, dense blocks as wide as the active experts).  One JSON line."""
+    from uzu_amd import synthetic as S
+    from uzu_amd.backend import Context
+    ctx = Context.new(0)
+    prompt_len, steps, warm, nbatch = 2048, max(8, min(args.steps, 128)), max(2, min(args.warmup, 8)), 8
+    out = {"metric": "rilavik_side_run", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16 products, f32 stream", "data": "synthetic (random weights, synthetic token ids)",
+           "prompt_tokens": prompt_len, "decode_steps": steps, "batched_decode_sequences": nbatch, "sizes": {}}
+    for size in [s for s in args.design_sizes.split(",") if s]:
+        z = LAZOLIX_SIZES[size]
+        prompt = S.synthetic_prompt(prompt_len, z["vocab"]).astype(np.uint32)
+        rec = {name: _time_f32_stream(ctx, b, prompt, steps, warm, nbatch) for name, b in rilavik_bundles(z, prompt_len + steps + warm + 64).items()}
+        out["sizes"][size] = {"shape": dict(z, kv_heads=max(1, z["heads"] // 4), ssd_heads=z["width"] // 64, ssd_vdim=64, ssd_state=128, ssd_groups=2, conv=4, rank=16,
+                                            pattern="3 x (convolved windowed attention + state-space mixer), gated linear attention; experts everywhere",
+                                            closest="Relulix: 3 x windowed attention, retention; experts", closest_pairs="Zovolorn: attention + channel-decay delta rule; dense"), **rec}
+    ctx.close()
+    print(json.dumps(out), flush=True)
+
+
 def main():
     args = parse_args()
+    if args.design == "rilavik":
+        return bench_rilavik(args)
     if args.design == "dironex":
         return bench_dironex(args)
     if args.design == "zovolorn":

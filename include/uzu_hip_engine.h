@@ -159,6 +159,14 @@ uzu_status uzu_hip_s32_latent_rope_append(uzu_hip_context* ctx, const float* x, 
 uzu_status uzu_hip_s32_gated_lru(uzu_hip_context* ctx, const float* branches, const float* conv_w, const float* conv_b, const uint16_t* gate_w, const float* gate_b,
                                  const float* lambda, float rate, float* state_inout, float* conv_state_inout, float* out, uint32_t rows, uint32_t start, uint32_t width,
                                  uint32_t blocks, uint32_t taps, uint32_t form);
+/*   decayed_state: S <- decay S + step k v^T, out = q_scale S^T q + skip v per head; decay = sigmoid(pre)^(1 / temperature) per head and key channel (per_head == 0,
+ *   step 1), or step = softplus(pre + dt_bias), decay = exp(-exp(a_log) step) (per_head); state in and out (ignored at start 0); form 0 dispatch, 1 token by token,
+ *   2 chunks; pitch_pad unused floats behind every packed row.   gated_norm: y silu(gate), RMS-normed in equal parts, times weight and out_scale. */
+uzu_status uzu_hip_s32_decayed_state(uzu_hip_context* ctx, const float* q, const float* k, const float* v, const float* decay, uint32_t per_head, float temperature, const float* a_log,
+                                     const float* dt_bias, const float* skip, float q_scale, float* state_inout, float* out, uint32_t rows, uint32_t start, uint32_t heads, uint32_t groups,
+                                     uint32_t dim, uint32_t vdim, uint32_t form, uint32_t pitch_pad);
+uzu_status uzu_hip_s32_gated_norm(uzu_hip_context* ctx, const float* y, const float* gate, const float* weight, float* out, float eps, float out_scale, uint32_t rows, uint32_t width,
+                                  uint32_t parts);
 /* 1: the full library.  0: the `stream32` flavor (make -C uzu_amd/csrc stream32 -> libuzu_hip_stream32.so), built without the fused decode kernels of the
  * bf16-stream models -- four minutes of compile time that a first use serving only an f32-stream design does not need; it refuses bf16-stream models at creation. */
 int uzu_hip_decode_kernels_present(void);

@@ -2,6 +2,7 @@
 // They exist so that every mechanism can be held to an independent statement of its equations on its own (tests/test_gpu_lazolix_kernels.py) and so that two
 // forms of one kernel can be compared on the same inputs; the engine calls the kernels directly (engine_stream32.hip).
 #include <algorithm>
+#include <cmath>
 #include <vector>
 
 #include "device_utils.h"
@@ -358,6 +359,69 @@ uzu_status uzu_hip_s32_retention(uzu_hip_context* ctx, const float* q, const flo
     UZU_PROPAGATE(finish(ctx));
     UZU_HIP_TRY(hipMemcpy(out, dout, (size_t)rows * heads * vdim * 4, hipMemcpyDeviceToHost));
     UZU_HIP_TRY(hipMemcpy(state_inout, dst, (size_t)heads * dim * vdim * 4, hipMemcpyDeviceToHost));
+    return UZU_OK;
+}
+
+// Linear attention with decays from the data, rows at positions start ..: q, k [rows][groups * dim], v [rows][heads * vdim]; decay [rows][heads * dim] (per_head == 0) or
+// [rows][heads]; a_log / dt_bias [heads] (per_head), skip [heads] or null; state_inout [heads][dim][vdim] is the state in front of the rows (ignored when start == 0) and
+// behind them.  form 0 dispatch, 1 token by token, 2 in chunks.  pitch_pad: that many unused floats behind every packed row (which moves columns off 16-byte borders).
+uzu_status uzu_hip_s32_decayed_state(uzu_hip_context* ctx, const float* q, const float* kk, const float* v, const float* decay, uint32_t per_head, float temperature, const float* a_log,
+                                     const float* dt_bias, const float* skip, float q_scale, float* state_inout, float* out, uint32_t rows, uint32_t start, uint32_t heads, uint32_t groups,
+                                     uint32_t dim, uint32_t vdim, uint32_t form, uint32_t pitch_pad) {
+    UZU_REQUIRE(ctx && q && kk && v && decay && state_inout && out && heads && groups && (!per_head || (a_log && dt_bias)), "s32_decayed_state: null argument");
+    (void)hipSetDevice(ctx->device);
+    Scratch S;
+    const uint32_t nq = groups * dim, ld = 2 * nq + heads * vdim + pitch_pad, nd = per_head ? heads : heads * dim;
+    std::vector<float> packed((size_t)rows * ld, NAN);
+    for (uint32_t r = 0; r < rows; ++r) {
+        float* row = packed.data() + (size_t)r * ld;
+        std::copy(q + (size_t)r * nq, q + (size_t)(r + 1) * nq, row);
+        std::copy(kk + (size_t)r * nq, kk + (size_t)(r + 1) * nq, row + nq);
+        std::copy(v + (size_t)r * heads * vdim, v + (size_t)(r + 1) * heads * vdim, row + 2 * nq);
+    }
+    float *dx, *dd, *dst, *dout, *dws = nullptr, *da = nullptr, *db = nullptr, *dk = nullptr;
+    float** dsp;
+    k::SeqSpan* spans;
+    uint32_t* row_seq;
+    UZU_PROPAGATE(S.up(packed.data(), packed.size(), &dx));
+    UZU_PROPAGATE(S.up(decay, (size_t)rows * nd, &dd));
+    if (per_head) {
+        UZU_PROPAGATE(S.up(a_log, heads, &da));
+        UZU_PROPAGATE(S.up(dt_bias, heads, &db));
+    }
+    if (skip) UZU_PROPAGATE(S.up(skip, heads, &dk));
+    UZU_PROPAGATE(S.up((const float*)state_inout, (size_t)heads * dim * vdim, &dst));
+    UZU_PROPAGATE(S.up((const float*)nullptr, (size_t)rows * heads * vdim, &dout));
+    UZU_PROPAGATE(S.up((float* const*)&dst, 1, &dsp));
+    UZU_PROPAGATE(one_sequence(S, rows, start, &spans, &row_seq));
+    k::DecayedStateParams p{};
+    p.rows_in = dx, p.ld = ld, p.q_col = 0, p.k_col = nq, p.v_col = 2 * nq, p.decay = dd, p.lddecay = nd, p.per_head = per_head, p.inv_temperature = temperature > 0.0f ? 1.0f / temperature : 0.0f;
+    p.a_log = da, p.dt_bias = db, p.skip = dk, p.q_scale = q_scale, p.out = dout, p.states = dsp, p.spans = spans, p.nseq = 1, p.rows = rows, p.heads = heads, p.groups = groups;
+    p.dim = dim, p.vdim = vdim, p.form = form, p.chunks = (rows + 63) / 64, p.chunk_ws_bytes = k::decayed_state_chunk_ws_bytes(p.chunks, heads, dim, vdim);
+    UZU_PROPAGATE(S.up((const float*)nullptr, p.chunk_ws_bytes / 4, &dws));
+    p.chunk_ws = dws;
+    UZU_PROPAGATE(k::decayed_state(ctx->stream, p));
+    UZU_PROPAGATE(finish(ctx));
+    UZU_HIP_TRY(hipMemcpy(out, dout, (size_t)rows * heads * vdim * 4, hipMemcpyDeviceToHost));
+    UZU_HIP_TRY(hipMemcpy(state_inout, dst, (size_t)heads * dim * vdim * 4, hipMemcpyDeviceToHost));
+    return UZU_OK;
+}
+
+// The gate in front of a norm in parts: out = rms in parts (y * silu(gate)) * weight * out_scale.  Host arrays y, gate, out [rows][width], weight [width].
+uzu_status uzu_hip_s32_gated_norm(uzu_hip_context* ctx, const float* y, const float* gate, const float* weight, float* out, float eps, float out_scale, uint32_t rows, uint32_t width, uint32_t parts) {
+    UZU_REQUIRE(ctx && y && gate && weight && out, "s32_gated_norm: null argument");
+    (void)hipSetDevice(ctx->device);
+    Scratch S;
+    float *dy, *dg, *dw, *dout;
+    UZU_PROPAGATE(S.up(y, (size_t)rows * width, &dy));
+    UZU_PROPAGATE(S.up(gate, (size_t)rows * width, &dg));
+    UZU_PROPAGATE(S.up(weight, width, &dw));
+    UZU_PROPAGATE(S.up((const float*)nullptr, (size_t)rows * width, &dout));
+    k::GatedNormParams p{};
+    p.y = dy, p.gate = dg, p.weight = dw, p.out = dout, p.ldy = p.ldgate = p.ldo = width, p.eps = eps, p.out_scale = out_scale, p.rows = rows, p.width = width, p.parts = parts;
+    UZU_PROPAGATE(k::gated_norm_rows(ctx->stream, p));
+    UZU_PROPAGATE(finish(ctx));
+    UZU_HIP_TRY(hipMemcpy(out, dout, (size_t)rows * width * 4, hipMemcpyDeviceToHost));
     return UZU_OK;
 }
 

@@ -125,38 +125,37 @@ __global__ void __launch_bounds__(256) head_norm_gate_kernel(HeadNormGateParams 
     }
 }
 
-// a workgroup per (row, part): the gated values stay in registers where a part is at most kGatedKeep steps of the workgroup; 256 strided partial sums, a fixed tree
-constexpr uint32_t kGatedKeep = 8;
+// a workgroup per (row, part): the first kGatedKeep coordinates travel in registers, their weights too (every load in front of the sum of squares), wider parts go over
+// the rest in further steps
+constexpr uint32_t kGatedUnroll = 4, kGatedKeep = 256 * kGatedUnroll;
 __global__ void __launch_bounds__(256) gated_norm_rows_kernel(GatedNormParams p) {
-    __shared__ float s_red[256];
+    __shared__ float s_red[16];
     const uint32_t r = blockIdx.x, w = p.width / p.parts, c0 = blockIdx.y * w, tid = threadIdx.x;
     const float *y = p.y + (size_t)r * p.ldy + c0, *g = p.gate + (size_t)r * p.ldgate + c0, *wt = p.weight + c0;
     float* out = p.out + (size_t)r * p.ldo + c0;
-    auto gated = [&](uint32_t i) { return y[i] * (g[i] / (1.0f + expf(-g[i]))); };
-    float keep[kGatedKeep], ss = 0.0f;
+    auto gated = [](float v, float z) { return v * (z / (1.0f + expf(-z))); };
+    float yv[kGatedUnroll], gv[kGatedUnroll], wv[kGatedUnroll], ss = 0.0f;
 #pragma unroll
-    for (uint32_t u = 0; u < kGatedKeep; ++u) {
+    for (uint32_t u = 0; u < kGatedUnroll; ++u) {
         const uint32_t i = tid + u * 256;
-        keep[u] = i < w ? gated(i) : 0.0f;
-        ss = fmaf(keep[u], keep[u], ss);
+        yv[u] = i < w ? y[i] : 0.0f, gv[u] = i < w ? g[i] : 0.0f, wv[u] = i < w ? wt[i] : 0.0f;
     }
-    for (uint32_t i = tid + kGatedKeep * 256; i < w; i += 256) {
-        const float v = gated(i);
+#pragma unroll
+    for (uint32_t u = 0; u < kGatedUnroll; ++u) {
+        yv[u] = gated(yv[u], gv[u]);
+        ss = fmaf(yv[u], yv[u], ss);
+    }
+    for (uint32_t i = tid + kGatedKeep; i < w; i += 256) {
+        const float v = gated(y[i], g[i]);
         ss = fmaf(v, v, ss);
     }
-    s_red[tid] = ss;
-    __syncthreads();
-    for (uint32_t h = 128; h > 0; h >>= 1) {
-        if (tid < h) s_red[tid] += s_red[tid + h];
-        __syncthreads();
-    }
-    const float inv = p.out_scale / sqrtf(s_red[0] / (float)w + p.eps);
-    for (uint32_t i = tid + kGatedKeep * 256; i < w; i += 256) out[i] = gated(i) * inv * wt[i]; // (out may be y: a thread replaces what it alone reads)
+    const float inv = p.out_scale / sqrtf(block_sum(ss, s_red) / (float)w + p.eps);
 #pragma unroll
-    for (uint32_t u = 0; u < kGatedKeep; ++u) {
+    for (uint32_t u = 0; u < kGatedUnroll; ++u) {
         const uint32_t i = tid + u * 256;
-        if (i < w) out[i] = keep[u] * inv * wt[i];
+        if (i < w) out[i] = yv[u] * inv * wv[u];
     }
+    for (uint32_t i = tid + kGatedKeep; i < w; i += 256) out[i] = gated(y[i], g[i]) * inv * wt[i]; // (out may be y: a thread replaces what it alone reads)
 }
 
 } // namespace

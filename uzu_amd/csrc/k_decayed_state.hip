@@ -18,15 +18,13 @@ namespace k {
 
 namespace {
 
-__device__ __forceinline__ float log_sigmoid_f32(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
 
-// one decay per head: the step size of a row (it multiplies the key) and the row's log decay
+// one decay per head: the step size of a row (it multiplies the key); the row's log decay is -exp(a_log) times it
 __device__ __forceinline__ float head_step(const DecayedStateParams& p, uint32_t r, uint32_t a) { return softplus_f32(p.decay[(size_t)r * p.lddecay + a] + p.dt_bias[a]); }
-// a decay per key channel
-__device__ __forceinline__ float channel_log_decay(const DecayedStateParams& p, uint32_t r, uint32_t a, uint32_t c) {
-    return log_sigmoid_f32(p.decay[(size_t)r * p.lddecay + (size_t)a * p.dim + c]) * p.inv_temperature;
-}
+// a decay per key channel: sigmoid(z)^inv_temperature by way of its logarithm, min(z, 0) - ln(1 + e^(-|z|)) (an absolute error of one rounding of 1: what the decay
+// itself is rounded to)
+__device__ __forceinline__ float channel_decay(float z, float inv_temperature) { return fast_exp((fminf(z, 0.0f) - fast_log(1.0f + fast_exp(-fabsf(z)))) * inv_temperature); }
 
 // ---- token by token.  grid (sequence * heads, ceil(vdim / 16)); thread = (column tid % 16, part tid / 16 of the key channels): it owns S[i][column] for
 // i = part, part + 16, ...; a token's partial sums meet by lane exchange and then over the four waves in LDS, in a fixed order
@@ -55,7 +53,7 @@ __global__ void __launch_bounds__(256) decayed_state_steps_kernel(DecayedStatePa
             const bool in = c < p.dim;
             s_q[c] = in ? row[p.q_col + (size_t)g * p.dim + c] * p.q_scale : 0.0f;
             s_k[c] = in ? row[p.k_col + (size_t)g * p.dim + c] * step : 0.0f;
-            if (CHANNEL) s_e[c] = in ? expf(channel_log_decay(p, r, a, c)) : 0.0f;
+            if (CHANNEL) s_e[c] = in ? channel_decay(p.decay[(size_t)r * p.lddecay + (size_t)a * p.dim + c], p.inv_temperature) : 0.0f;
         }
         if (tid < 16) s_v[tid] = live ? row[p.v_col + (size_t)a * p.vdim + col] : 0.0f;
         __syncthreads();
@@ -120,84 +118,113 @@ __device__ __forceinline__ float suffix_after(float v, uint32_t lane) {
     }
     return s;
 }
+// the sum over a quad of lanes, left in every one of them
+__device__ __forceinline__ float quad_sum(float v) {
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true)); // quad_perm [1, 0, 3, 2]
+    v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true)); // quad_perm [2, 3, 0, 1]
+    return v;
+}
+// four neighbouring floats of a row, those from `left` on zero; aligned: one 16-byte load (the host has checked pitch, columns and widths)
+__device__ __forceinline__ f32x4_m load4(const float* at, uint32_t left, bool aligned) {
+    f32x4_m v{0.f, 0.f, 0.f, 0.f};
+    if (aligned) {
+        if (left) v = *(const f32x4_m*)at;
+    } else {
+#pragma unroll
+        for (uint32_t u = 0; u < 4; ++u)
+            if (u < left) v[u] = at[u];
+    }
+    return v;
+}
 
-// a workgroup per (chunk, head, tile of 64 key channels x 128 value columns): v_mfma_f32_32x32x2_f32, lane l feeds A[l % 32][k = l / 32], B[k = l / 32][l % 32] and holds
-// rows 8 (r / 4) + 4 (l / 32) + r % 4 of column l % 32
-template <bool CHANNEL>
-__global__ void __launch_bounds__(256) decayed_state_local_kernel(DecayedStateParams p, float* ws) {
-    constexpr uint32_t KW = 64, VW = 128;
-    __shared__ float s_k[kChunk][KW], s_v[kChunk][VW], s_tot[4][KW]; // s_k: a decay per channel -- first the log decays
-    __shared__ float s_e[kChunk];                                    // one decay per head: a row's step size times the decay behind it
+// a workgroup per (chunk, head, tile of 64 key channels x 64 NQ value columns): v_mfma_f32_32x32x2_f32, lane l feeds A[l % 32][k = l / 32], B[k = l / 32][l % 32] and
+// holds rows 8 (r / 4) + 4 (l / 32) + r % 4 of column l % 32
+template <bool CHANNEL, int NQ>
+__global__ void __launch_bounds__(256) decayed_state_local_kernel(DecayedStateParams p, float* ws, uint32_t aligned) {
+    constexpr uint32_t KW = 64, VW = 64 * NQ;
+    __shared__ __attribute__((aligned(16))) float s_k[kChunk][KW], s_v[kChunk][VW];
+    __shared__ float s_tot[4][KW]; // a decay per channel: a block's whole decay
+    __shared__ float s_e[kChunk];  // one decay per head: a row's step size times the decay behind it
     uint32_t z, c;
     SeqSpan sp;
     if (!find_chunk(p, blockIdx.x, z, c, sp)) return;
     const uint32_t a = blockIdx.y, g = a / (p.heads / p.groups), tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l32 = lane & 31, half = lane >> 5;
     const uint32_t vtiles = (p.vdim + VW - 1) / VW, i0 = blockIdx.z / vtiles * KW, j0 = blockIdx.z % vtiles * VW;
     const uint32_t r0 = sp.row0 + c * kChunk, n = sp.count - c * kChunk < kChunk ? sp.count - c * kChunk : kChunk;
-    if (!CHANNEL && wave == 0) { // lane = row: the decay of everything behind it
-        const float dt = lane < n ? head_step(p, r0 + lane, a) : 0.0f;
-        const float e = -expf(p.a_log[a]) * dt, behind = suffix_after(e, lane);
-        s_e[lane] = dt * expf(behind);
-        if (lane == 0 && blockIdx.z == 0) ws[decay_at(p, blockIdx.x, a, false)] = expf(e + behind);
-    }
-    if (CHANNEL)
-        for (uint32_t e = tid; e < kChunk * KW; e += 256) {
-            const uint32_t t = e / KW, i = e % KW;
-            s_k[t][i] = (t < n && i0 + i < p.dim) ? channel_log_decay(p, r0 + t, a, i0 + i) : 0.0f;
-        }
-    for (uint32_t e = tid; e < kChunk * VW; e += 256) {
-        const uint32_t t = e / VW, j = e % VW;
-        s_v[t][j] = (t < n && j0 + j < p.vdim) ? p.rows_in[(size_t)(r0 + t) * p.ld + p.v_col + (size_t)a * p.vdim + j0 + j] : 0.0f;
-    }
-    __syncthreads();
-    if (CHANNEL) { // thread = (channel, block of 16 rows)
-        const uint32_t i = tid & 63, b = tid >> 6;
-        float tot = 0.0f;
+    // thread = (channel i of the tile, block b of 16 rows): its keys (and decays) in registers, every load in front of the first use
+    const uint32_t i = lane, b = wave;
+    const bool in = i0 + i < p.dim;
+    const float* kcol = p.rows_in + (size_t)r0 * p.ld + p.k_col + (size_t)g * p.dim + i0 + i;
+    float key[kBlock], dec[CHANNEL ? kBlock : 1];
 #pragma unroll
-        for (uint32_t t = 0; t < kBlock; ++t) tot += s_k[b * kBlock + t][i];
-        s_tot[b][i] = tot;
-        __syncthreads();
-        float behind = 0.0f;
-        for (uint32_t o = 3; o > b; --o) behind += s_tot[o][i];
-        if (b == 0 && j0 == 0 && i0 + i < p.dim) ws[decay_at(p, blockIdx.x, a, true) + i0 + i] = expf(behind + s_tot[0][i]);
-        const float* kcol = p.rows_in + p.k_col + (size_t)g * p.dim + i0 + i;
-#pragma unroll 4
+    for (uint32_t t = 0; t < kBlock; ++t) {
+        const uint32_t row = b * kBlock + t;
+        key[t] = row < n && in ? kcol[(size_t)row * p.ld] : 0.0f;
+        if (CHANNEL) dec[CHANNEL ? t : 0] = row < n && in ? p.decay[(size_t)(r0 + row) * p.lddecay + (size_t)a * p.dim + i0 + i] : 0.0f;
+    }
+    {   // values: thread = (rows tid / (16 NQ) + .., four columns)
+        constexpr uint32_t TPR = 16 * NQ, RPP = 256 / TPR;
+        const uint32_t col = (tid % TPR) * 4, left = j0 + col < p.vdim ? p.vdim - j0 - col : 0;
+        const float* vb = p.rows_in + (size_t)r0 * p.ld + p.v_col + (size_t)a * p.vdim + j0 + col;
+        f32x4_m v[kChunk / RPP];
+#pragma unroll
+        for (uint32_t u = 0; u < kChunk / RPP; ++u) {
+            const uint32_t t = tid / TPR + u * RPP;
+            v[u] = load4(vb + (size_t)t * p.ld, t < n ? left : 0, aligned);
+        }
+#pragma unroll
+        for (uint32_t u = 0; u < kChunk / RPP; ++u) *(f32x4_m*)&s_v[tid / TPR + u * RPP][col] = v[u];
+    }
+    if (CHANNEL) {
+        float run = 1.0f; // the decay of the rows behind t inside the block
+#pragma unroll
         for (int t = kBlock - 1; t >= 0; --t) {
-            const uint32_t row = b * kBlock + t;
-            const float e = s_k[row][i];
-            s_k[row][i] = (row < n && i0 + i < p.dim) ? kcol[(size_t)(r0 + row) * p.ld] * expf(behind) : 0.0f;
-            behind += e;
+            key[t] *= run;
+            run *= b * kBlock + t < n ? channel_decay(dec[CHANNEL ? t : 0], p.inv_temperature) : 1.0f;
         }
+        s_tot[b][i] = run;
+        __syncthreads();
+        float behind = 1.0f;
+        for (uint32_t o = b + 1; o < 4; ++o) behind *= s_tot[o][i];
+        if (b == 0 && j0 == 0 && in) ws[decay_at(p, blockIdx.x, a, true) + i0 + i] = run * behind;
+#pragma unroll
+        for (uint32_t t = 0; t < kBlock; ++t) s_k[b * kBlock + t][i] = key[t] * behind;
     } else {
-        for (uint32_t e = tid; e < kChunk * KW; e += 256) {
-            const uint32_t t = e / KW, i = e % KW;
-            s_k[t][i] = (t < n && i0 + i < p.dim) ? p.rows_in[(size_t)(r0 + t) * p.ld + p.k_col + (size_t)g * p.dim + i0 + i] * s_e[t] : 0.0f;
+        if (wave == 0) { // lane = row: its step size and the decay of everything behind it
+            const float dt = lane < n ? head_step(p, r0 + lane, a) : 0.0f;
+            const float e = -expf(p.a_log[a]) * dt, behind = suffix_after(e, lane);
+            s_e[lane] = dt * expf(behind);
+            if (lane == 0 && blockIdx.z == 0) ws[decay_at(p, blockIdx.x, a, false)] = expf(e + behind);
         }
+        __syncthreads();
+#pragma unroll
+        for (uint32_t t = 0; t < kBlock; ++t) s_k[b * kBlock + t][i] = key[t] * s_e[b * kBlock + t];
     }
     __syncthreads();
-    // eight 32 x 32 tiles: wave w owns channel half w / 2 and column tiles 2 (w % 2), 2 (w % 2) + 1
-    f32x16_m acc[2];
+    // 32 x 32 tiles: wave w owns channel half w / 2 and column tiles NQ (w % 2) ..
+    f32x16_m acc[NQ];
 #pragma unroll
-    for (int q = 0; q < 2; ++q)
+    for (int q = 0; q < NQ; ++q)
 #pragma unroll
         for (int r = 0; r < 16; ++r) acc[q][r] = 0.0f;
-    const uint32_t ti = (wave >> 1) * 32, tj = (wave & 1) * 64, steps = (n + 1) / 2;
-    if (i0 + ti < p.dim && j0 + tj < p.vdim) {
-        for (uint32_t t2 = 0; t2 < steps; ++t2) {
-            const uint32_t t = 2 * t2 + half;
+    const uint32_t ti = (wave >> 1) * 32, tj = (wave & 1) * 32 * NQ;
+    if (i0 + ti >= p.dim || j0 + tj >= p.vdim) return;
+    for (uint32_t t0 = 0; t0 < n; t0 += 8) // (rows beyond the chunk's: zero keys and values)
+#pragma unroll
+        for (uint32_t u = 0; u < 4; ++u) {
+            const uint32_t t = t0 + 2 * u + half;
             const float ka = s_k[t][ti + l32];
 #pragma unroll
-            for (int q = 0; q < 2; ++q) acc[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(ka, s_v[t][tj + 32 * q + l32], acc[q], 0, 0, 0);
+            for (int q = 0; q < NQ; ++q) acc[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(ka, s_v[t][tj + 32 * q + l32], acc[q], 0, 0, 0);
         }
-        float* dst = ws + ((size_t)blockIdx.x * p.heads + a) * p.dim * p.vdim;
+    float* dst = ws + ((size_t)blockIdx.x * p.heads + a) * p.dim * p.vdim;
 #pragma unroll
-        for (int q = 0; q < 2; ++q) {
-            const uint32_t j = j0 + tj + 32 * q + l32;
+    for (int q = 0; q < NQ; ++q) {
+        const uint32_t j = j0 + tj + 32 * q + l32;
 #pragma unroll
-            for (int r = 0; r < 16; ++r) {
-                const uint32_t i = i0 + ti + 8 * (r >> 2) + 4 * half + (r & 3);
-                if (i < p.dim && j < p.vdim) dst[(size_t)i * p.vdim + j] = acc[q][r];
-            }
+        for (int r = 0; r < 16; ++r) {
+            const uint32_t row = i0 + ti + 8 * (r >> 2) + 4 * half + (r & 3);
+            if (row < p.dim && j < p.vdim) dst[(size_t)row * p.vdim + j] = acc[q][r];
         }
     }
 }
@@ -234,16 +261,17 @@ template <bool CHANNEL> __global__ void __launch_bounds__(256) decayed_state_sca
     *state = S;
 }
 
-// a workgroup per (chunk, head, 128 value columns).  Key channels in slabs of 32: raw and decayed queries / keys in LDS; a wave owns the block of 16 x 16 scores on
-// the diagonal that bears its number (running products, lane = (key row, quarter of the slab)), up to two of the six blocks below it (v_mfma_f32_16x16x4_f32) and,
-// for the carried state, 32 rows x 64 columns of the result.
-template <bool CHANNEL>
-__global__ void __launch_bounds__(256) decayed_state_out_kernel(DecayedStateParams p, const float* ws) {
-    constexpr uint32_t SW = 32, PW = SW + 4, VW = 128; // a slab row's pitch: 16-byte aligned, rows on distinct banks
-    constexpr uint32_t ROWS = kChunk * PW;
-    __shared__ __attribute__((aligned(16))) float s_buf[CHANNEL ? 5 * ROWS : (2 * ROWS + kChunk * PW > kChunk * VW ? 2 * ROWS + kChunk * PW : kChunk * VW)];
+// a workgroup per (chunk, head, 64 NQ value columns).  Key channels in slabs of 32; the next slab's rows travel from memory into registers while the current one is
+// worked on, the carried state's rows go from memory straight into the products.  One decay per head: scores as two 32 x 32 tiles per wave row, times a table of decays.
+// A decay per channel: a wave owns the block of 16 x 16 scores on the diagonal that bears its number (running products, lane = (key row, quarter of the slab)) and up to
+// two of the six blocks below it (v_mfma_f32_16x16x4_f32).  Results: wave w has rows 32 (w / 2) .., column tiles NQ (w % 2) ..
+template <bool CHANNEL, int NQ>
+__global__ void __launch_bounds__(256, CHANNEL ? 2 : 3) decayed_state_out_kernel(DecayedStateParams p, const float* ws, uint32_t aligned) {
+    constexpr uint32_t SW = 32, PW = SW + 4, VW = 64 * NQ, ROWS = kChunk * PW; // a slab row's pitch: 16-byte aligned, rows on distinct banks
+    constexpr uint32_t BUF = CHANNEL ? 5 * ROWS : 2 * ROWS;
+    __shared__ __attribute__((aligned(16))) float s_buf[BUF > kChunk * VW ? BUF : kChunk * VW];
     __shared__ float s_p[kChunk][kChunk + 1], s_tot[4][SW]; // s_tot: a block's whole decay per channel of the slab
-    __shared__ float s_h[3][kChunk]; // one decay per head: log decays, step sizes, the decay from the chunk's start up to and including a row
+    __shared__ float s_h[6][kChunk]; // one decay per head, by row: log decay, step size, decay from the chunk's start, sums of log decays up to the row / behind it in its block, blocks' sums
     uint32_t z, c;
     SeqSpan sp;
     if (!find_chunk(p, blockIdx.x, z, c, sp)) return;
@@ -251,99 +279,139 @@ __global__ void __launch_bounds__(256) decayed_state_out_kernel(DecayedStatePara
     const uint32_t j0 = blockIdx.z * VW, dim = p.dim, vdim = p.vdim;
     const uint32_t r0 = sp.row0 + c * kChunk, n = sp.count - c * kChunk < kChunk ? sp.count - c * kChunk : kChunk;
     const float* base = p.rows_in + (size_t)r0 * p.ld;
-    const float *qb = base + p.q_col + (size_t)g * dim, *kb = base + p.k_col + (size_t)g * dim;
-    const bool carried = sp.start || c;
+    const float *qb = base + p.q_col + (size_t)g * dim, *kb = base + p.k_col + (size_t)g * dim, *eb = p.decay + (size_t)r0 * p.lddecay + (size_t)a * dim;
     const float* S = ws + ((size_t)blockIdx.x * p.heads + a) * dim * vdim + j0;
-    float *s_q = s_buf, *s_k = s_buf + ROWS, *s_x = s_buf + 2 * ROWS; // s_x: one decay per head -- queries decayed from the chunk's start
+    float *s_q = s_buf, *s_k = s_buf + ROWS;
     float *s_e = s_buf + 2 * ROWS, *s_qd = s_buf + 3 * ROWS, *s_kd = s_buf + 4 * ROWS; // a decay per channel: decays; queries decayed from their block's start; keys decayed to its end
-    for (uint32_t e = tid; e < kChunk * (kChunk + 1); e += 256) (&s_p[0][0])[e] = 0.0f;
+    const uint32_t pi = wave >> 1, pj = wave & 1;
+    const bool out_on = j0 + pj * 32 * NQ < vdim, carried = (sp.start || c) && out_on;
+    // a slab's loads: thread = (rows tid / 8, tid / 8 + 32, four channels)
+    const uint32_t lr = tid >> 3, lc = (tid & 7) * 4;
+    f32x4_m fq[2], fk[2], fe[CHANNEL ? 2 : 1];
+    auto fetch = [&](uint32_t d0) {
+        const uint32_t left = d0 + lc < dim ? dim - d0 - lc : 0;
+#pragma unroll
+        for (uint32_t u = 0; u < 2; ++u) {
+            const uint32_t r = lr + 32 * u, m = r < n ? left : 0;
+            fq[u] = load4(qb + (size_t)r * p.ld + d0 + lc, m, aligned);
+            fk[u] = load4(kb + (size_t)r * p.ld + d0 + lc, m, aligned);
+            if (CHANNEL) fe[CHANNEL ? u : 0] = load4(eb + (size_t)r * p.lddecay + d0 + lc, m, aligned);
+        }
+    };
+    fetch(0);
     if (!CHANNEL) {
+        for (uint32_t e = tid; e < kChunk * (kChunk + 1); e += 256) (&s_p[0][0])[e] = 0.0f;
         if (wave == 0) {
             const float dt = lane < n ? head_step(p, r0 + lane, a) : 0.0f, e = -expf(p.a_log[a]) * dt;
-            float upto = e; // the sum over lanes 0 .. lane
+            float upto = e, behind = __shfl_down(e, 1, 16); // inside the row's block of 16
+            behind = l16 < 15 ? behind : 0.0f;
 #pragma unroll
-            for (int off = 1; off < 64; off <<= 1) {
-                const float o = __shfl_up(upto, off, 64);
-                upto += lane >= (uint32_t)off ? o : 0.0f;
+            for (int off = 1; off < 16; off <<= 1) {
+                const float o = __shfl_up(upto, off, 16), q = __shfl_down(behind, off, 16);
+                upto += l16 >= (uint32_t)off ? o : 0.0f;
+                behind += l16 + off < 16 ? q : 0.0f;
             }
-            s_h[0][lane] = e, s_h[1][lane] = dt, s_h[2][lane] = expf(upto);
+            const float tot = __shfl(upto, 15, 16);
+            float before = 0.0f; // the blocks in front
+#pragma unroll
+            for (uint32_t o = 0; o < 3; ++o) {
+                const float t = __shfl(tot, (int)(o * kBlock), 64);
+                before += o < quarter ? t : 0.0f;
+            }
+            s_h[0][lane] = e, s_h[1][lane] = dt, s_h[2][lane] = expf(before + upto), s_h[3][lane] = upto, s_h[4][lane] = behind, s_h[5][quarter] = tot;
         }
         __syncthreads();
-        // thread = (key row j, block of 16 query rows): e^(the log decays of rows j + 1 .. i), summed from j on
-        const uint32_t j = lane, b = wave;
-        float sum = 0.0f;
-        const uint32_t i_lo = b * kBlock;
-        for (uint32_t t = j + 1; t < i_lo; ++t) sum += s_h[0][t];
+        // thread = (key row j, block of 16 query rows): step_j e^(the log decays of rows j + 1 .. i)
+        const uint32_t j = lane, b = wave, jb = j / kBlock;
         const float dt = s_h[1][j];
-        for (uint32_t i = i_lo; i < i_lo + kBlock; ++i) {
-            if (i < j) continue;
-            if (i > j) sum += s_h[0][i];
-            s_p[i][j] = i < n ? expf(sum) * dt : 0.0f;
+        if (b > jb) {
+            float sum = s_h[4][j];
+            for (uint32_t o = jb + 1; o < b; ++o) sum += s_h[5][o];
+#pragma unroll 4
+            for (uint32_t i = b * kBlock; i < b * kBlock + kBlock; ++i) s_p[i][j] = i < n ? expf(sum + s_h[3][i]) * dt : 0.0f;
+        } else if (b == jb) {
+            float sum = 0.0f;
+#pragma unroll 4
+            for (uint32_t i = b * kBlock; i < b * kBlock + kBlock; ++i) {
+                sum += i > j ? s_h[0][i] : 0.0f;
+                if (i >= j) s_p[i][j] = i < n ? expf(sum) * dt : 0.0f;
+            }
         }
+    } else {
+        for (uint32_t e = tid; e < kChunk * (kChunk + 1); e += 256) (&s_p[0][0])[e] = 0.0f;
     }
-    const uint32_t pi = wave >> 1, pj = wave & 1; // 32-row half of the result; one decay per head: 32-column half of the scores; result column tiles 2 pj, 2 pj + 1
-    f32x16_m sc, o[2];
+    f32x16_m sc, o[NQ];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) sc[r] = 0.0f, o[0][r] = 0.0f, o[1][r] = 0.0f;
+    for (int r = 0; r < 16; ++r) sc[r] = 0.0f;
+#pragma unroll
+    for (int q = 0; q < NQ; ++q)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[q][r] = 0.0f;
     // the six pairs of blocks below the diagonal: (1, 0), (2, 0), (2, 1), (3, 0), (3, 1), (3, 2)
     auto below_i = [](uint32_t pair) { return pair < 1 ? 1u : pair < 3 ? 2u : 3u; };
     auto below_j = [&](uint32_t pair) { const uint32_t i = below_i(pair); return pair - i * (i - 1) / 2; };
     f32x4_m lower[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-    float diag[kBlock];
-#pragma unroll
-    for (uint32_t i = 0; i < kBlock; ++i) diag[i] = 0.0f;
-    const bool out_on = j0 + pj * 64 < vdim;
+    const uint32_t row = pi * 32 + l32; // this lane's row of the query operand
+    float from_start = 1.0f;
     for (uint32_t d0 = 0; d0 < dim; d0 += SW) {
+        float sv[SW / 2][NQ]; // the carried state's rows of the slab
+#pragma unroll
+        for (uint32_t d = 0; d < SW / 2; ++d)
+#pragma unroll
+            for (int q = 0; q < NQ; ++q) {
+                const uint32_t dg = d0 + 2 * d + half, col = pj * 32 * NQ + 32 * q + l32;
+                sv[d][q] = carried && dg < dim && j0 + col < vdim ? S[(size_t)dg * vdim + col] : 0.0f;
+            }
         __syncthreads(); // the slab before has been read
-        for (uint32_t e = tid; e < kChunk * SW; e += 256) {
-            const uint32_t r = e / SW, dd = e % SW, d = d0 + dd;
-            const bool ok = r < n && d < dim;
-            const float q = ok ? qb[(size_t)r * p.ld + d] * p.q_scale : 0.0f;
-            s_q[r * PW + dd] = q;
-            s_k[r * PW + dd] = ok ? kb[(size_t)r * p.ld + d] : 0.0f;
-            if (CHANNEL) s_e[r * PW + dd] = ok ? channel_log_decay(p, r0 + r, a, d) : 0.0f;
-            else s_x[r * PW + dd] = q * s_h[2][r];
+#pragma unroll
+        for (uint32_t u = 0; u < 2; ++u) {
+            const uint32_t at = (lr + 32 * u) * PW + lc;
+            *(f32x4_m*)(s_q + at) = fq[u] * p.q_scale;
+            *(f32x4_m*)(s_k + at) = fk[u];
+            if (CHANNEL) { // (rows and channels beyond the chunk: their queries and keys are zeros)
+                f32x4_m e;
+#pragma unroll
+                for (int v = 0; v < 4; ++v) e[v] = channel_decay(fe[CHANNEL ? u : 0][v], p.inv_temperature);
+                *(f32x4_m*)(s_e + at) = e;
+            }
         }
         __syncthreads();
-        if (CHANNEL) { // thread = (channel, block, direction): prefixes onto the queries, suffixes onto the keys; the log decays become decays behind them
-            const uint32_t dd = tid & 31, b = (tid >> 5) & 3, first = b * kBlock;
-            float sum = 0.0f;
+        if (d0 + SW < dim) fetch(d0 + SW);
+        if (CHANNEL) { // thread = (channel, block, direction): running products onto the queries from the block's start, onto the keys from its end
+            const uint32_t dd = tid & 31, first = ((tid >> 5) & 3) * kBlock;
+            float run = 1.0f;
             if (tid < 128) {
-#pragma unroll 4
+#pragma unroll
                 for (uint32_t t = 0; t < kBlock; ++t) {
-                    sum += s_e[(first + t) * PW + dd];
-                    s_qd[(first + t) * PW + dd] = s_q[(first + t) * PW + dd] * expf(sum);
+                    run *= s_e[(first + t) * PW + dd];
+                    s_qd[(first + t) * PW + dd] = s_q[(first + t) * PW + dd] * run;
                 }
-                s_tot[b][dd] = expf(sum);
+                s_tot[first / kBlock][dd] = run;
             } else {
-#pragma unroll 4
+#pragma unroll
                 for (int t = kBlock - 1; t >= 0; --t) {
-                    s_kd[(first + t) * PW + dd] = s_k[(first + t) * PW + dd] * expf(sum);
-                    sum += s_e[(first + t) * PW + dd];
+                    s_kd[(first + t) * PW + dd] = s_k[(first + t) * PW + dd] * run;
+                    run *= s_e[(first + t) * PW + dd];
                 }
             }
             __syncthreads();
-            for (uint32_t e = tid; e < kChunk * SW; e += 256) s_e[e / SW * PW + e % SW] = expf(s_e[e / SW * PW + e % SW]);
-            __syncthreads();
-            {   // the diagonal block `wave`: key row l16, channels 8 quarter .. 8 quarter + 7 of the slab
-                const uint32_t first_row = wave * kBlock, ch = quarter * 8;
-                float w[8];
-                const f32x4_m k0 = *(const f32x4_m*)(s_k + (first_row + l16) * PW + ch), k1 = *(const f32x4_m*)(s_k + (first_row + l16) * PW + ch + 4);
-#pragma unroll
-                for (int u = 0; u < 4; ++u) w[u] = k0[u], w[u + 4] = k1[u];
-#pragma unroll
+            {   // the diagonal block `wave`: four lanes share a key row, channels 8 quad .. 8 quad + 7 of the slab each; the sums gather in s_p
+                const uint32_t first_row = wave * kBlock, j = lane >> 2, ch = (lane & 3) * 8;
+                const f32x4_m k0 = *(const f32x4_m*)(s_k + (first_row + j) * PW + ch), k1 = *(const f32x4_m*)(s_k + (first_row + j) * PW + ch + 4);
+                f32x4_m w0{0.f, 0.f, 0.f, 0.f}, w1 = w0; // the key as row i sees it: nothing in front of its own row
+#pragma unroll 2
                 for (uint32_t i = 0; i < kBlock; ++i) {
-                    const float* er = s_e + (first_row + i) * PW + ch;
-                    const float* qr = s_q + (first_row + i) * PW + ch;
+                    const float *er = s_e + (first_row + i) * PW + ch, *qr = s_q + (first_row + i) * PW + ch;
                     const f32x4_m e0 = *(const f32x4_m*)er, e1 = *(const f32x4_m*)(er + 4), q0 = *(const f32x4_m*)qr, q1 = *(const f32x4_m*)(qr + 4);
-                    float dot = 0.0f;
+                    const bool own = i == j;
+                    float d0v = 0.0f, d1v = 0.0f;
 #pragma unroll
-                    for (int u = 0; u < 8; ++u) {
-                        const float ev = u < 4 ? e0[u] : e1[u - 4], qv = u < 4 ? q0[u] : q1[u - 4];
-                        w[u] = i > l16 ? w[u] * ev : w[u];
-                        dot = fmaf(qv, w[u], dot);
+                    for (int u = 0; u < 4; ++u) {
+                        w0[u] = own ? k0[u] : w0[u] * e0[u], w1[u] = own ? k1[u] : w1[u] * e1[u];
+                        d0v = fmaf(q0[u], w0[u], d0v), d1v = fmaf(q1[u], w1[u], d1v);
                     }
-                    diag[i] += i >= l16 ? dot : 0.0f;
+                    const float dot = quad_sum(d0v + d1v);
+                    if ((lane & 3) == 0) s_p[first_row + i][first_row + j] += dot;
                 }
             }
 #pragma unroll
@@ -355,43 +423,41 @@ __global__ void __launch_bounds__(256) decayed_state_out_kernel(DecayedStatePara
                 for (uint32_t k4 = 0; k4 < SW; k4 += 4) {
                     const uint32_t ch = k4 + quarter;
                     float qa = s_qd[(bi * kBlock + l16) * PW + ch];
-                    for (uint32_t b = bj + 1; b < bi; ++b) qa *= s_tot[b][ch];
+                    if (bi - bj > 1) qa *= s_tot[bj + 1][ch];
+                    if (bi - bj > 2) qa *= s_tot[bj + 2][ch];
                     lower[q] = __builtin_amdgcn_mfma_f32_16x16x4f32(qa, s_kd[(bj * kBlock + l16) * PW + ch], lower[q], 0, 0, 0);
                 }
             }
-        } else {
-#pragma unroll 4
-            for (uint32_t d = 0; d < SW; d += 2) sc = __builtin_amdgcn_mfma_f32_32x32x2f32(s_q[(pi * 32 + l32) * PW + d + half], s_k[(pj * 32 + l32) * PW + d + half], sc, 0, 0, 0);
-        }
-        if (carried && out_on) { // + sum_d (query decayed from the chunk's start) S[d][column], the state's rows straight from memory
-#pragma unroll 4
-            for (uint32_t d = 0; d < SW; d += 2) {
-                const uint32_t dl = d + half, dg = d0 + dl, row = pi * 32 + l32;
-                float qa;
-                if (CHANNEL) {
-                    qa = s_qd[row * PW + dl];
-                    for (uint32_t b = 0; b < row / kBlock; ++b) qa *= s_tot[b][dl];
-                } else {
-                    qa = s_x[row * PW + dl];
-                }
+            if (carried) { // + sum_d (query decayed from the chunk's start) S[d][column]
+                const uint32_t rb = row / kBlock;
 #pragma unroll
-                for (int q = 0; q < 2; ++q) {
-                    const uint32_t col = pj * 64 + 32 * q + l32;
-                    const float sv = (dg < dim && j0 + col < vdim) ? S[(size_t)dg * vdim + col] : 0.0f;
-                    o[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(qa, sv, o[q], 0, 0, 0);
+                for (uint32_t d = 0; d < SW / 2; ++d) {
+                    const uint32_t dl = 2 * d + half;
+                    float qa = s_qd[row * PW + dl];
+                    const float t0 = s_tot[0][dl], t1 = s_tot[1][dl], t2 = s_tot[2][dl];
+                    qa *= rb > 0 ? t0 : 1.0f;
+                    qa *= rb > 1 ? t1 : 1.0f;
+                    qa *= rb > 2 ? t2 : 1.0f;
+#pragma unroll
+                    for (int q = 0; q < NQ; ++q) o[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(qa, sv[d][q], o[q], 0, 0, 0);
+                    if ((d & 3) == 3) __builtin_amdgcn_sched_barrier(0);
+                }
+            }
+        } else {
+            if (d0 == 0) from_start = s_h[2][row];
+#pragma unroll
+            for (uint32_t d = 0; d < SW / 2; ++d) {
+                const float qv = s_q[row * PW + 2 * d + half];
+                sc = __builtin_amdgcn_mfma_f32_32x32x2f32(qv, s_k[(pj * 32 + l32) * PW + 2 * d + half], sc, 0, 0, 0);
+                if (carried) {
+#pragma unroll
+                    for (int q = 0; q < NQ; ++q) o[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(qv * from_start, sv[d][q], o[q], 0, 0, 0);
                 }
             }
         }
     }
     __syncthreads(); // the slabs are done with
     if (CHANNEL) {
-#pragma unroll
-        for (uint32_t i = 0; i < kBlock; ++i) {
-            float v = diag[i];
-            v += __shfl_xor(v, 16, 64);
-            v += __shfl_xor(v, 32, 64);
-            if (quarter == 0 && i >= l16) s_p[wave * kBlock + i][wave * kBlock + l16] = v;
-        }
 #pragma unroll
         for (int q = 0; q < 2; ++q) {
             const uint32_t pair = wave + 4 * q;
@@ -407,23 +473,31 @@ __global__ void __launch_bounds__(256) decayed_state_out_kernel(DecayedStatePara
         }
     }
     float* s_v = s_buf; // [64][VW]
-    for (uint32_t e = tid; e < kChunk * VW; e += 256) {
-        const uint32_t t = e / VW, j = e % VW;
-        s_v[e] = (t < n && j0 + j < vdim) ? base[(size_t)t * p.ld + p.v_col + (size_t)a * vdim + j0 + j] : 0.0f;
+    {
+        constexpr uint32_t TPR = 16 * NQ, RPP = 256 / TPR;
+        const uint32_t col = (tid % TPR) * 4, left = j0 + col < vdim ? vdim - j0 - col : 0;
+        const float* vb = base + p.v_col + (size_t)a * vdim + j0 + col;
+#pragma unroll
+        for (uint32_t u = 0; u < kChunk / RPP; ++u) {
+            const uint32_t t = tid / TPR + u * RPP;
+            *(f32x4_m*)(s_v + t * VW + col) = load4(vb + (size_t)t * p.ld, t < n ? left : 0, aligned);
+        }
     }
     __syncthreads();
     if (!out_on) return;
-    const uint32_t last = n < pi * 32 + 32 ? n : pi * 32 + 32, steps = (last + 1) / 2; // keys up to this half's last row
-    for (uint32_t t2 = 0; t2 < steps; ++t2) {
-        const uint32_t t = 2 * t2 + half;
-        const float pa = s_p[pi * 32 + l32][t];
+    const uint32_t last = n < pi * 32 + 32 ? n : pi * 32 + 32; // keys up to this half's last row (beyond the chunk's rows: zero scores and values)
+    for (uint32_t t0 = 0; t0 < last; t0 += 8)
 #pragma unroll
-        for (int q = 0; q < 2; ++q) o[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(pa, s_v[t * VW + pj * 64 + 32 * q + l32], o[q], 0, 0, 0);
-    }
+        for (uint32_t u = 0; u < 4; ++u) {
+            const uint32_t t = t0 + 2 * u + half;
+            const float pa = s_p[row][t];
+#pragma unroll
+            for (int q = 0; q < NQ; ++q) o[q] = __builtin_amdgcn_mfma_f32_32x32x2f32(pa, s_v[t * VW + pj * 32 * NQ + 32 * q + l32], o[q], 0, 0, 0);
+        }
     const float skip = p.skip ? p.skip[a] : 0.0f;
 #pragma unroll
-    for (int q = 0; q < 2; ++q) {
-        const uint32_t col = pj * 64 + 32 * q + l32;
+    for (int q = 0; q < NQ; ++q) {
+        const uint32_t col = pj * 32 * NQ + 32 * q + l32;
         if (j0 + col >= vdim) continue;
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
@@ -447,18 +521,25 @@ uzu_status decayed_state(hipStream_t s, const DecayedStateParams& p) {
     UZU_REQUIRE((size_t)p.nseq * p.heads <= 0x7FFFFFFFu && p.heads <= 65535 && p.nseq <= 65535, "decayed_state: too many heads for one launch");
     if (p.form == 2 || (p.form == 0 && p.chunk_ws && p.rows > 16 * p.nseq)) { // prompt-sized: in chunks
         UZU_REQUIRE(p.chunk_ws && p.chunks && p.chunk_ws_bytes >= decayed_state_chunk_ws_bytes(p.chunks, p.heads, p.dim, p.vdim), "decayed_state: the chunked form needs its workspace");
-        const uint32_t vt = (p.vdim + 127) / 128, kt = (p.dim + 63) / 64;
+        const uint32_t vw = p.vdim <= 64 ? 64 : 128, vt = (p.vdim + vw - 1) / vw, kt = (p.dim + 63) / 64;
+        const uint32_t aligned = p.ld % 4 == 0 && p.q_col % 4 == 0 && p.k_col % 4 == 0 && p.v_col % 4 == 0 && p.dim % 4 == 0 && p.vdim % 4 == 0 && (uintptr_t)p.rows_in % 16 == 0 &&
+                                 (p.per_head || (p.lddecay % 4 == 0 && (uintptr_t)p.decay % 16 == 0)) ? 1u : 0u;
         UZU_REQUIRE((size_t)vt * kt <= 65535 && ((size_t)p.dim * p.vdim + 255) / 256 <= 65535, "decayed_state: head widths %u x %u", p.dim, p.vdim);
         const dim3 lgrid(p.chunks, p.heads, vt * kt), sgrid(p.nseq, p.heads, (uint32_t)(((size_t)p.dim * p.vdim + 255) / 256)), ogrid(p.chunks, p.heads, vt);
         float* ws = p.chunk_ws;
+#define UZU_DC(CH, NQ)                                                                                                                                                             \
+    do {                                                                                                                                                                           \
+        UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL((decayed_state_local_kernel<CH, NQ>), lgrid, dim3(256), 0, s, p, ws, aligned); }, "decayed_state_local"));             \
+        UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(decayed_state_scan_kernel<CH>, sgrid, dim3(256), 0, s, p, ws); }, "decayed_state_scan"));                              \
+        return launch_check([&] { hipLaunchKernelGGL((decayed_state_out_kernel<CH, NQ>), ogrid, dim3(256), 0, s, p, (const float*)ws, aligned); }, "decayed_state_out");           \
+    } while (0)
         if (p.per_head) {
-            UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(decayed_state_local_kernel<false>, lgrid, dim3(256), 0, s, p, ws); }, "decayed_state_local"));
-            UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(decayed_state_scan_kernel<false>, sgrid, dim3(256), 0, s, p, ws); }, "decayed_state_scan"));
-            return launch_check([&] { hipLaunchKernelGGL(decayed_state_out_kernel<false>, ogrid, dim3(256), 0, s, p, (const float*)ws); }, "decayed_state_out");
+            if (vw == 64) UZU_DC(false, 1);
+            UZU_DC(false, 2);
         }
-        UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(decayed_state_local_kernel<true>, lgrid, dim3(256), 0, s, p, ws); }, "decayed_state_local"));
-        UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(decayed_state_scan_kernel<true>, sgrid, dim3(256), 0, s, p, ws); }, "decayed_state_scan"));
-        return launch_check([&] { hipLaunchKernelGGL(decayed_state_out_kernel<true>, ogrid, dim3(256), 0, s, p, (const float*)ws); }, "decayed_state_out");
+        if (vw == 64) UZU_DC(true, 1);
+        UZU_DC(true, 2);
+#undef UZU_DC
     }
     const dim3 grid(p.nseq * p.heads, (p.vdim + 15) / 16);
 #define UZU_DS(N)                                                                                                                                                     \

@@ -90,109 +90,94 @@ __global__ void __launch_bounds__(64) embed_pair_commit_kernel(EmbedPairParams p
     if (sp.count > 1) *p.prev[z] = p.tokens[sp.row0 + sp.count - 1];
 }
 
+// A workgroup per row (or part of a row): the first kNormKeep coordinates of the row travel in registers -- every load of the launch is issued before the sum of squares
+// is known (a one-row decode step's launch consists of memory round trips: one is enough) --, wider rows go over the rest in further steps.  The sum of squares:
+// strided partial sums per thread, a fixed exchange inside the wave, the four waves in order.
 constexpr int kNormUnroll = 8;
-// a workgroup per row: the sum of squares as 256 strided partial sums folded in a fixed tree, then the scaled row
+constexpr uint32_t kNormKeep = 256 * kNormUnroll;
+
 // (blockIdx.y = the part of a row that is normed in gridDim.y equal consecutive parts: `d` is the part's width, `ld` the row's)
 __global__ void __launch_bounds__(256) rms_norm_rows_kernel(const float* x, float* out, const float* scales, float gain, float eps, const uint32_t* row_index, uint32_t d,
                                                             float offset, uint32_t ld) {
-    __shared__ float s_red[256];
+    __shared__ float s_red[16];
     const uint32_t r = blockIdx.x, part0 = blockIdx.y * d;
     const float* xr = x + (size_t)(row_index ? row_index[r] : r) * ld + part0;
     if (scales) scales += part0;
-    float acc = 0.0f;
-    for (uint32_t i = threadIdx.x; i < d; i += 256) acc = fmaf(xr[i], xr[i], acc);
-    s_red[threadIdx.x] = acc;
-    __syncthreads();
-    for (uint32_t w = 128; w > 0; w >>= 1) {
-        if (threadIdx.x < w) s_red[threadIdx.x] += s_red[threadIdx.x + w];
-        __syncthreads();
-    }
-    const float inv = 1.0f / sqrtf(s_red[0] / (float)d + eps);
     float* o = out + (size_t)r * ld + part0;
-    // kNormUnroll elements per thread and step, every load of a step in front of its stores (out may alias x for the compiler: a loop of load -> store pairs would
-    // pay one memory round trip per element, which is what a one-row decode step's launch consists of)
-    for (uint32_t i0 = threadIdx.x; i0 < d; i0 += 256 * kNormUnroll) {
-        float xv[kNormUnroll], sv[kNormUnroll];
+    float xv[kNormUnroll], sv[kNormUnroll], acc = 0.0f;
 #pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            xv[u] = i < d ? xr[i] : 0.0f;
-            sv[u] = (i < d && scales) ? scales[i] : 0.0f;
-        }
+    for (int u = 0; u < kNormUnroll; ++u) {
+        const uint32_t i = threadIdx.x + u * 256;
+        xv[u] = i < d ? xr[i] : 0.0f;
+        sv[u] = (i < d && scales) ? scales[i] : 0.0f;
+    }
 #pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            if (i >= d) break;
-            const float v = xv[u] * inv * gain;
-            o[i] = scales ? v * (sv[u] + offset) : v;
-        }
+    for (int u = 0; u < kNormUnroll; ++u) acc = fmaf(xv[u], xv[u], acc);
+    for (uint32_t i = threadIdx.x + kNormKeep; i < d; i += 256) acc = fmaf(xr[i], xr[i], acc);
+    const float inv = 1.0f / sqrtf(block_sum(acc, s_red) / (float)d + eps);
+#pragma unroll
+    for (int u = 0; u < kNormUnroll; ++u) {
+        const uint32_t i = threadIdx.x + u * 256;
+        if (i >= d) break;
+        const float v = xv[u] * inv * gain;
+        o[i] = scales ? v * (sv[u] + offset) : v;
+    }
+    for (uint32_t i = threadIdx.x + kNormKeep; i < d; i += 256) {
+        const float v = xr[i] * inv * gain;
+        o[i] = scales ? v * (scales[i] + offset) : v;
     }
 }
 
-// the same sum of squares over a sublayer's result y; the normed row joins the stream: out = residual + y * inv * (scales + offset) * layer_scale
+// the same over a sublayer's result y; the normed row joins the stream: out = residual + y * inv * (scales + offset) * layer_scale
 // ... and, with `next`, the norm of the new row for the sublayer that follows (its own weights, offset and epsilon): next[r] = rms(out[r]) * (next_scales + next_offset)
 __global__ void __launch_bounds__(256) rms_norm_add_rows_kernel(const float* y, const float* residual, float* out, const float* scales, float offset, const float* layer_scale,
                                                                 float eps, uint32_t d, float* next, const float* next_scales, float next_offset, float next_eps, uint32_t ld) {
-    __shared__ float s_red[256];
+    __shared__ float s_red[16];
     const uint32_t r = blockIdx.x, part0 = blockIdx.y * d; // (a row normed in gridDim.y parts of width d; `next` only with one part)
     const float* yr = y + (size_t)r * ld + part0;
     scales += part0;
     if (layer_scale) layer_scale += part0;
-    float acc = 0.0f;
-    for (uint32_t i = threadIdx.x; i < d; i += 256) acc = fmaf(yr[i], yr[i], acc);
-    s_red[threadIdx.x] = acc;
-    __syncthreads();
-    for (uint32_t w = 128; w > 0; w >>= 1) {
-        if (threadIdx.x < w) s_red[threadIdx.x] += s_red[threadIdx.x + w];
-        __syncthreads();
-    }
-    const float inv = 1.0f / sqrtf(s_red[0] / (float)d + eps);
     const float* res = residual + (size_t)r * ld + part0;
     float* o = out + (size_t)r * ld + part0;
-    float acc2 = 0.0f;
-    for (uint32_t i0 = threadIdx.x; i0 < d; i0 += 256 * kNormUnroll) { // (loads of a step in front of its stores, as in rms_norm_rows_kernel; sums in the same order)
-        float yv[kNormUnroll], rv[kNormUnroll], sv[kNormUnroll], lv[kNormUnroll];
+    float yv[kNormUnroll], rv[kNormUnroll], sv[kNormUnroll], lv[kNormUnroll], nv[kNormUnroll], acc = 0.0f, acc2 = 0.0f;
 #pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            const bool ok = i < d;
-            yv[u] = ok ? yr[i] : 0.0f, rv[u] = ok ? res[i] : 0.0f, sv[u] = ok ? scales[i] : 0.0f, lv[u] = (ok && layer_scale) ? layer_scale[i] : 1.0f;
-        }
+    for (int u = 0; u < kNormUnroll; ++u) {
+        const uint32_t i = threadIdx.x + u * 256;
+        const bool ok = i < d;
+        yv[u] = ok ? yr[i] : 0.0f, rv[u] = ok ? res[i] : 0.0f, sv[u] = ok ? scales[i] : 0.0f, lv[u] = (ok && layer_scale) ? layer_scale[i] : 1.0f;
+        nv[u] = (ok && next) ? next_scales[i] : 0.0f;
+    }
 #pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            if (i >= d) break;
-            float v = yv[u] * inv * (sv[u] + offset);
-            if (layer_scale) v *= lv[u];
-            v = rv[u] + v;
-            o[i] = v;
-            acc2 = fmaf(v, v, acc2);
-        }
+    for (int u = 0; u < kNormUnroll; ++u) acc = fmaf(yv[u], yv[u], acc);
+    for (uint32_t i = threadIdx.x + kNormKeep; i < d; i += 256) acc = fmaf(yr[i], yr[i], acc);
+    const float inv = 1.0f / sqrtf(block_sum(acc, s_red) / (float)d + eps);
+#pragma unroll
+    for (int u = 0; u < kNormUnroll; ++u) {
+        const uint32_t i = threadIdx.x + u * 256;
+        if (i >= d) break;
+        float v = yv[u] * inv * (sv[u] + offset);
+        if (layer_scale) v *= lv[u];
+        rv[u] = rv[u] + v;
+        o[i] = rv[u];
+        acc2 = fmaf(rv[u], rv[u], acc2);
+    }
+    for (uint32_t i = threadIdx.x + kNormKeep; i < d; i += 256) {
+        float v = yr[i] * inv * (scales[i] + offset);
+        if (layer_scale) v *= layer_scale[i];
+        v = res[i] + v;
+        o[i] = v;
+        acc2 = fmaf(v, v, acc2);
     }
     if (!next) return;
-    __syncthreads(); // s_red[0] has been read by everyone
-    s_red[threadIdx.x] = acc2;
-    __syncthreads();
-    for (uint32_t w = 128; w > 0; w >>= 1) {
-        if (threadIdx.x < w) s_red[threadIdx.x] += s_red[threadIdx.x + w];
-        __syncthreads();
-    }
-    const float inv2 = 1.0f / sqrtf(s_red[0] / (float)d + next_eps);
+    const float inv2 = 1.0f / sqrtf(block_sum(acc2, s_red) / (float)d + next_eps);
     float* nx = next + (size_t)r * d;
-    for (uint32_t i0 = threadIdx.x; i0 < d; i0 += 256 * kNormUnroll) { // (o: the thread's own stores)
-        float ov[kNormUnroll], sv[kNormUnroll];
 #pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            ov[u] = i < d ? o[i] : 0.0f, sv[u] = i < d ? next_scales[i] : 0.0f;
-        }
-#pragma unroll
-        for (int u = 0; u < kNormUnroll; ++u) {
-            const uint32_t i = i0 + u * 256;
-            if (i >= d) break;
-            nx[i] = ov[u] * inv2 * (sv[u] + next_offset);
-        }
+    for (int u = 0; u < kNormUnroll; ++u) {
+        const uint32_t i = threadIdx.x + u * 256;
+        if (i >= d) break;
+        nx[i] = rv[u] * inv2 * (nv[u] + next_offset);
     }
+    for (uint32_t i = threadIdx.x + kNormKeep; i < d; i += 256) nx[i] = o[i] * inv2 * (next_scales[i] + next_offset); // (o: the thread's own stores)
 }
 
 __global__ void __launch_bounds__(256) dyn_tanh_kernel(DynTanhParams p) {
