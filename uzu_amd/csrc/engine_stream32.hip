@@ -359,21 +359,35 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         float* qkv_rows = S.q;
         uint32_t ldqkv = L.qkv.n;
         const bool joint = X.joint.w != nullptr;
+        k::CausalConvParams conv{}; // its launch; a decode step's rides in the rotation's
         auto mixer_conv = [&](uint32_t ldx) {
-            k::CausalConvParams cp{};
-            cp.x = S.q, cp.ldx = ldx, cp.out = S.dn_cv, cp.ldo = X.conv_channels, cp.w = X.conv_w, cp.bias = X.conv_b, cp.channels = X.conv_channels, cp.taps = X.conv_taps;
-            cp.act = X.conv_act_from < X.conv_channels ? 1 : 0, cp.act_from = X.conv_act_from;
-            cp.states = S.d_pair_conv_ptrs + (size_t)l * S.max_seqs, cp.spans = S.d_spans, cp.row_seq = S.d_row_seq, cp.nseq = nseq, cp.rows = rows, cp.max_count = max_count;
-            RUN("causal_conv_rows", (size_t)rows * cp.channels * 4 * (cp.taps + 1), k::causal_conv_rows(s, cp));
-            if (cp.taps > 1 && max_count > 1) RUN("causal_conv_commit", (size_t)nseq * cp.channels * 8 * (cp.taps - 1), k::causal_conv_commit(s, cp));
+            conv.x = S.q, conv.ldx = ldx, conv.out = S.dn_cv, conv.ldo = X.conv_channels, conv.w = X.conv_w, conv.bias = X.conv_b, conv.channels = X.conv_channels, conv.taps = X.conv_taps;
+            conv.act = X.conv_act_from < X.conv_channels ? 1 : 0, conv.act_from = X.conv_act_from, conv.states = S.d_pair_conv_ptrs + (size_t)l * S.max_seqs;
+            conv.spans = S.d_spans, conv.row_seq = S.d_row_seq, conv.nseq = nseq, conv.rows = rows, conv.max_count = max_count;
             qkv_rows = S.dn_cv, ldqkv = X.conv_channels;
         };
+        auto run_mixer_conv = [&]() {
+            RUN("causal_conv_rows", (size_t)rows * conv.channels * 4 * (conv.taps + 1), k::causal_conv_rows(s, conv));
+            if (conv.taps > 1 && max_count > 1) RUN("causal_conv_commit", (size_t)nseq * conv.channels * 8 * (conv.taps - 1), k::causal_conv_commit(s, conv));
+        };
+        k::RopeAppendParams rp{}; // attention's rotation and append
+        if (h.mixer_kind == UZU_MIXER_ATTENTION) {
+            const uint32_t H = h.num_heads, G = h.num_groups, hd = h.head_dim;
+            rp.k_col = H * hd, rp.v_col = h.values_are_keys ? H * hd : H * hd + G * hd, rp.heads = H, rp.kv_heads = h.is_kv_sharing ? 0u : G, rp.dim = hd, rp.vdim = h.value_head_dim;
+            rp.rope_dim = h.use_rope ? L.rope_dim : 0u, rp.cosines = L.rope_cos, rp.sines = L.rope_sin, rp.key_scale = h.key_scale != 0.0f ? h.key_scale : 1.0f;
+            rp.norm_whole = h.qk_norm_whole, rp.interleaved = h.rope_interleaved;
+            rp.key_caches = caches, rp.value_caches = S.d_cache2_ptrs + (size_t)l * S.max_seqs, rp.cache_bf16 = bf, rp.spans = S.d_spans, rp.row_seq = S.d_row_seq, rp.rows = rows;
+            rp.q_norm = L.qn.present ? L.qn.scales : nullptr, rp.k_norm = L.kn.present && !h.is_kv_sharing ? L.kn.scales : nullptr, rp.norm_eps = L.qn.present ? L.qn.eps : L.kn.eps;
+        }
+        bool conv_rides = false;
         const uint32_t ldj = (X.joint.n + 3) / 4 * 4, ldo_joint = X.joint_out.k; // row pitches of the joint projection and of its halves' results
         if (joint) {
             k::LinearF32Params jp = lin(S, X.joint, mix_in, S.q, rows);
             jp.ldy = ldj;
             run_linear(e, jp);
             mixer_conv(ldj);
+            conv_rides = rows < 256 && k::conv_rope_append_supported(rp, conv);
+            if (!conv_rides) run_mixer_conv();
         }
         // prompt-sized pass over a pair of mixers: the first one's projection, rotation / append and attention core go to the side stream (they touch S.q, S.attn and
         // the caches; the second mixer touches its own rows); not while a launch is being timed or captured
@@ -386,7 +400,11 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         }
         if (!joint) {
             run_linear(e, lin(S, L.qkv, mix_in, S.q, rows)); // the packed projection of the mixer (queries first)
-            if (X.conv_w) mixer_conv(L.qkv.n);
+            if (X.conv_w) {
+                mixer_conv(L.qkv.n);
+                conv_rides = rows < 256 && k::conv_rope_append_supported(rp, conv);
+                if (!conv_rides) run_mixer_conv();
+            }
         }
         if (h.mixer_kind == UZU_MIXER_GATED_LRU) {
             const uint32_t w = h.lru_width, bw = w / h.lru_blocks;
@@ -407,13 +425,9 @@ uzu_status s32_encode(uzu_hip_model* m, const std::vector<uint32_t>& counts, con
         } else if (h.mixer_kind == UZU_MIXER_ATTENTION) {
             const uint32_t G = h.num_groups, ldq = ldqkv;
             void* const* vcaches = S.d_cache2_ptrs + (size_t)l * S.max_seqs;
-            k::RopeAppendParams rp{};
-            rp.qkv = qkv_rows, rp.ld = ldq, rp.k_col = H * hd, rp.v_col = h.values_are_keys ? H * hd : H * hd + G * hd, rp.heads = H, rp.kv_heads = h.is_kv_sharing ? 0u : G, rp.dim = hd, rp.vdim = vd;
-            rp.rope_dim = h.use_rope ? L.rope_dim : 0u, rp.cosines = L.rope_cos, rp.sines = L.rope_sin, rp.key_scale = h.key_scale != 0.0f ? h.key_scale : 1.0f;
-            rp.norm_whole = h.qk_norm_whole, rp.interleaved = h.rope_interleaved;
-            rp.key_caches = caches, rp.value_caches = vcaches, rp.cache_bf16 = bf, rp.spans = S.d_spans, rp.row_seq = S.d_row_seq, rp.rows = rows;
-            rp.q_norm = L.qn.present ? L.qn.scales : nullptr, rp.k_norm = L.kn.present && !h.is_kv_sharing ? L.kn.scales : nullptr, rp.norm_eps = L.qn.present ? L.qn.eps : L.kn.eps;
-            RUN("rope_append", (size_t)rows * ldq * 8, k::rope_append(s, rp));
+            rp.qkv = qkv_rows, rp.ld = ldq;
+            if (conv_rides) RUN("conv_rope_append", (size_t)rows * conv.channels * 12 * conv.taps, k::conv_rope_append(s, rp, conv));
+            else RUN("rope_append", (size_t)rows * ldq * 8, k::rope_append(s, rp));
             k::WindowAttentionParams ap{};
             ap.q = qkv_rows, ap.ldq = ldq, ap.out = S.attn, ap.key_caches = caches, ap.value_caches = vcaches, ap.cache_bf16 = bf, ap.sinks = X.sinks, ap.spans = S.d_spans;
             ap.row_seq = S.d_row_seq, ap.rows = rows, ap.heads = H, ap.kv_heads = G, ap.dim = hd, ap.vdim = vd, ap.window = h.sliding_window_size;

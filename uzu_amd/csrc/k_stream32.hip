@@ -605,17 +605,26 @@ __global__ void __launch_bounds__(1024) moe_bucket_kernel(const int32_t* ids, ui
         offsets[routed] = run;
     }
 }
-// a pair's place inside its expert's bucket: the order of arrival (any order gives the same numbers: a row's product does not depend on its place in a tile)
+// a pair's place inside its expert's bucket: the order of arrival (any order gives the same numbers: a row's product does not depend on its place in a tile).  A workgroup
+// counts its own pairs in LDS and takes one stretch per expert from the bucket's cursor.
 __global__ void __launch_bounds__(256) moe_scatter_kernel(const int32_t* ids, uint32_t slots, uint32_t routed, uint32_t top, const uint32_t* offsets, uint32_t* cursor, uint32_t* perm,
                                                          uint32_t* slot_pos, const float* weights, float* pos_weight) {
+    extern __shared__ uint32_t s_next[]; // [routed]: pairs of this workgroup, then the next free place
+    for (uint32_t e = threadIdx.x; e < routed; e += blockDim.x) s_next[e] = 0;
+    __syncthreads();
     const uint32_t i = blockIdx.x * blockDim.x + threadIdx.x;
+    const int32_t e = i < slots ? ids[i] : -1;
+    const bool hit = e >= 0 && (uint32_t)e < routed;
+    const uint32_t rank = hit ? atomicAdd(&s_next[e], 1u) : 0u;
+    __syncthreads();
+    for (uint32_t x = threadIdx.x; x < routed; x += blockDim.x) s_next[x] = s_next[x] ? offsets[x] + atomicAdd(&cursor[x], s_next[x]) : 0u;
+    __syncthreads();
     if (i >= slots) return;
-    const int32_t e = ids[i];
-    if (e < 0 || (uint32_t)e >= routed) {
+    if (!hit) {
         slot_pos[i] = 0xFFFFFFFFu;
         return;
     }
-    const uint32_t pos = offsets[e] + atomicAdd(&cursor[e], 1u);
+    const uint32_t pos = s_next[e] + rank;
     perm[pos] = i / top;
     slot_pos[i] = pos;
     if (pos_weight) pos_weight[pos] = weights[i];
@@ -663,7 +672,7 @@ uzu_status moe_experts_grouped(hipStream_t s, const MoeGroupedParams& p) {
     UZU_REQUIRE(!p.pos_weight || !p.act.plain, "moe_experts_grouped: weights on the inputs of plain experts");
     const uint32_t slots = p.rows * p.top;
     UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_bucket_kernel, dim3(1), dim3(1024), (size_t)p.routed * 4, s, p.ids, slots, p.routed, p.offsets, p.cursor); }, "moe_bucket"));
-    UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_scatter_kernel, dim3((slots + 255) / 256), dim3(256), 0, s, p.ids, slots, p.routed, p.top, p.offsets, p.cursor, p.perm, p.slot_pos, p.weights, p.pos_weight); },
+    UZU_PROPAGATE(launch_check([&] { hipLaunchKernelGGL(moe_scatter_kernel, dim3((slots + 255) / 256), dim3(256), (size_t)p.routed * 4, s, p.ids, slots, p.routed, p.top, p.offsets, p.cursor, p.perm, p.slot_pos, p.weights, p.pos_weight); },
                                "moe_scatter"));
     LinearF32Params q{};
     const uint32_t n1 = p.act.plain ? p.ff : 2 * p.ff;

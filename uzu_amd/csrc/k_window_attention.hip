@@ -98,6 +98,65 @@ __global__ void __launch_bounds__(1024) rope_append_kernel(RopeAppendParams p) {
         }
     }
 }
+// The same behind a causal convolution of the row, for passes of one row per sequence: a workgroup takes whole query heads, whole key heads, or 256 of the channels behind
+// them (values to the cache, what stands behind the values back to the rows).  A channel's window is replaced by the thread that alone reads it; taps in tap order, as in
+// causal_conv_rows.
+__device__ __forceinline__ uint32_t conv_rope_heads_per_block(uint32_t dim) { return dim < 256 ? 256 / dim : 1; }
+template <int T> __device__ __forceinline__ float conv_channel(const CausalConvParams& c, const SeqSpan& sp, float* window, uint32_t r, uint32_t ch) {
+    float in[T], w[T];
+    in[T - 1] = c.x[(size_t)r * c.ldx + c.x_col + ch];
+    float acc = c.bias ? c.bias[ch] : 0.0f;
+#pragma unroll
+    for (int j = 0; j < T; ++j) {
+        w[j] = c.w[(size_t)ch * T + j];
+        if (j < T - 1) in[j] = (uint32_t)(T - 1 - j) <= sp.start ? window[(size_t)j * c.channels + ch] : 0.0f; // (in front of position 0: zeros)
+    }
+#pragma unroll
+    for (int j = 0; j < T; ++j) acc = fmaf(w[j], in[j], acc);
+    if (c.act == 1 && ch >= c.act_from) acc = acc / (1.0f + expf(-acc));
+    if (c.add_input) acc = in[T - 1] + acc;
+#pragma unroll
+    for (int j = 0; j < T - 1; ++j) window[(size_t)j * c.channels + ch] = in[j + 1];
+    return acc;
+}
+template <int T> __global__ void __launch_bounds__(256) conv_rope_append_kernel(RopeAppendParams p, CausalConvParams c) {
+    extern __shared__ float s_h[]; // the block's heads
+    const uint32_t r = blockIdx.x, z = p.row_seq[r], hpb = conv_rope_heads_per_block(p.dim), qb = (p.heads + hpb - 1) / hpb, kb = (p.kv_heads + hpb - 1) / hpb;
+    const SeqSpan sp = p.spans[z];
+    const uint32_t t = sp.start;
+    float* window = c.states[z] + c.state_offset;
+    float* row = p.qkv + (size_t)r * p.ld;
+    if (blockIdx.y >= qb + kb) { // values and what stands behind them
+        const uint32_t ch = p.v_col + (blockIdx.y - qb - kb) * 256 + threadIdx.x;
+        if (ch >= c.channels) return;
+        const float v = conv_channel<T>(c, sp, window, r, ch);
+        if (ch < p.v_col + p.kv_heads * p.vdim) cache_st(p.value_caches[z], p.cache_bf16, (size_t)t * p.kv_heads * p.vdim + (ch - p.v_col), v);
+        else row[ch] = v;
+        return;
+    }
+    const bool is_q = blockIdx.y < qb;
+    const uint32_t h0 = (is_q ? blockIdx.y : blockIdx.y - qb) * hpb, heads = is_q ? p.heads : p.kv_heads, n = (h0 + hpb < heads ? hpb : heads - h0) * p.dim;
+    const uint32_t c0 = (is_q ? 0 : p.k_col) + h0 * p.dim, half = p.rope_dim / 2;
+    for (uint32_t i = threadIdx.x; i < n; i += 256) s_h[i] = conv_channel<T>(c, sp, window, r, c0 + i);
+    __syncthreads();
+    const float *cs = p.cosines + (size_t)t * p.rope_dim, *sn = p.sines + (size_t)t * p.rope_dim;
+    void* kc = is_q ? nullptr : p.key_caches[z];
+    const float scale = is_q ? 1.0f : p.key_scale;
+    for (uint32_t i = threadIdx.x; i < n; i += 256) {
+        const uint32_t d = i % p.dim, head = i - d;
+        float v = s_h[i];
+        if (d < p.rope_dim) {
+            const uint32_t pair = p.interleaved ? d >> 1 : d < half ? d : d - half;
+            const bool first = p.interleaved ? (d & 1) == 0 : d < half;
+            const uint32_t iu = head + (p.interleaved ? 2 * pair : pair), iv = iu + (p.interleaved ? 1 : half);
+            const float a = s_h[iu], b = s_h[iv], co = cs[pair], si = sn[pair];
+            v = first ? a * co - b * si : b * co + a * si;
+        }
+        v *= scale;
+        if (is_q) row[c0 + i] = v;
+        else cache_st(kc, p.cache_bf16, (size_t)t * p.kv_heads * p.dim + h0 * p.dim + i, v);
+    }
+}
 
 // ---- the simple form: a wave per (row, head).  Keys in blocks of 64 from the row's first visible key: a lane scores one key of the block (the whole dot
 // product, the query staged in LDS), the block's weights go through LDS, then a lane owns value coordinates lane, lane + 64, ... of the running sum.
@@ -191,6 +250,30 @@ uzu_status rope_append(hipStream_t s, const RopeAppendParams& p) {
     UZU_REQUIRE(!p.kv_heads || ((p.key_caches != nullptr) == (p.value_caches != nullptr)), "rope_append: key and value caches come together");
     UZU_REQUIRE(p.v_col != p.k_col || !p.kv_heads || (p.vdim == p.dim && p.value_caches), "rope_append: values that are the key rows have the keys' width and go to a cache");
     return launch_check([&] { hipLaunchKernelGGL(rope_append_kernel, dim3(p.rows), dim3(p.rows <= 64 && !p.norm_whole ? 1024 : 256), 0, s, p); }, "rope_append");
+}
+
+bool conv_rope_append_supported(const RopeAppendParams& p, const CausalConvParams& c) {
+    return c.max_count == 1 && c.taps >= 1 && c.taps <= 4 && !p.q_norm && !p.k_norm && p.kv_heads && p.v_col != p.k_col && p.key_caches && p.value_caches && p.dim <= 8192;
+}
+
+uzu_status conv_rope_append(hipStream_t s, const RopeAppendParams& p, const CausalConvParams& c) {
+    if (!p.rows) return UZU_OK;
+    UZU_REQUIRE(conv_rope_append_supported(p, c) && c.x && c.w && (c.states || c.taps == 1) && c.out == p.qkv && c.ldo == p.ld && !c.o_col && c.rows == p.rows && c.x != c.out,
+                "conv_rope_append: one row per sequence, 1 .. 4 taps, no head norms, the convolution's result in place of the packed rows");
+    UZU_REQUIRE(p.spans && p.row_seq && p.heads && p.dim && p.rope_dim % 2 == 0 && p.rope_dim <= p.dim && (!p.rope_dim || (p.cosines && p.sines)), "conv_rope_append: an even rotation width with its tables");
+    UZU_REQUIRE(p.k_col == p.heads * p.dim && p.v_col == p.k_col + p.kv_heads * p.dim && p.v_col + p.kv_heads * p.vdim <= c.channels && c.x_col + c.channels <= c.ldx && c.channels <= c.ldo,
+                "conv_rope_append: rows of queries | keys | values (| ..)");
+    const uint32_t hpb = p.dim < 256 ? 256 / p.dim : 1, blocks = (p.heads + hpb - 1) / hpb + (p.kv_heads + hpb - 1) / hpb + (c.channels - p.v_col + 255) / 256;
+    UZU_REQUIRE(blocks <= 65535, "conv_rope_append: too many channels for one launch");
+#define UZU_CR(T) case T: return launch_check([&] { hipLaunchKernelGGL(conv_rope_append_kernel<T>, dim3(p.rows, blocks), dim3(256), (size_t)hpb * p.dim * 4, s, p, c); }, "conv_rope_append")
+    switch (c.taps) {
+        UZU_CR(1);
+        UZU_CR(2);
+        UZU_CR(3);
+        UZU_CR(4);
+        default: return UZU_ERR_INVALID_ARGUMENT;
+    }
+#undef UZU_CR
 }
 
 uzu_status window_attention_mfma(hipStream_t s, const WindowAttentionParams& p); // k_window_attention_mfma.hip

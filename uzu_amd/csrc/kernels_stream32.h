@@ -438,6 +438,11 @@ struct CausalConvParams {
 uzu_status causal_conv_rows(hipStream_t s, const CausalConvParams& p);
 uzu_status causal_conv_commit(hipStream_t s, const CausalConvParams& p);
 
+// causal_conv_rows and rope_append of its result in one launch, for passes in which every sequence brings one row (windows are replaced as well): c.out = p.qkv, the packed
+// queries | keys | values are the first of c's channels.  The same numbers as the two launches, but key and value columns of c.out are left unwritten (they go to the caches).
+bool conv_rope_append_supported(const RopeAppendParams& p, const CausalConvParams& c);
+uzu_status conv_rope_append(hipStream_t s, const RopeAppendParams& p, const CausalConvParams& c);
+
 // Per head, in place: x[r, a, :] <- x[r, a, :] / sqrt(mean(x[r, a, :]^2) + eps) * weight[:] * gate(g[r, a, :])    (x f32 rows of pitch ldx, heads * width used;
 // weight f32 [width] or null; g f32 rows of pitch ldgate or null; gate = sigmoid (gate_sigmoid) or silu)
 struct HeadNormGateParams {
