@@ -729,7 +729,7 @@ def rilavik_bundles(z, context):
             return loader.load_model_dir(tmp, max_context_length=context)
     mlp = rilavik.moe_mlp(z["experts"], z["top"], z["eff"])
     par = rilavik.parallel_layer(rilavik.attention_half(H, G, dim, vd, window, conv=4, rot_dims=dim, rot_base=500000.0, factor=8.0),
-                                 rilavik.state_space_half(z["width"] // 64, 64, 128, groups=2, norm_groups=2, conv=4), 0.8, 1.1, mlp=mlp)
+                                 rilavik.state_space_half(z["width"] // 64, 64, 128, groups=2, norm_groups=2, conv=4), 0.7, 1.2, mlp=mlp)
     gla = rilavik.gla_layer(H, dim, vd, rank=16, mlp=mlp)
     out = {"rilavik": bundle(rilavik, rilavik.config(z["vocab"], z["width"], ([par, par, par, gla] * ((z["layers"] + 3) // 4))[:z["layers"]]))}
     rmlp = relulix.moe_mlp(z["experts"], z["top"], z["eff"], limit=7.0)
@@ -737,7 +737,7 @@ def rilavik_bundles(z, context):
     ret = relulix.retention_layer(H, dim, vd, relulix.rotation(dim, 1e6), [1.0 - 2.0 ** -(5 + (a % 6)) for a in range(H)], mlp=rmlp)
     out["closest"] = bundle(relulix, relulix.config(z["vocab"], z["width"], ([att, att, att, ret] * ((z["layers"] + 3) // 4))[:z["layers"]]))
     zmlp = zovolorn.dense_mlp(z["top"] * z["eff"])  # the active experts' width
-    zpar = zovolorn.parallel_layer(H, G, dim, window, 32, 2048.0, z["width"] // 64, 2, 128, 64, 4, rank=16, left_scale=0.8, right_scale=1.1, mlp=zmlp)
+    zpar = zovolorn.parallel_layer(H, G, dim, window, 32, 2048.0, z["width"] // 64, 2, 128, 64, 4, rank=16, left_scale=0.7, right_scale=1.2, mlp=zmlp)
     out["closest_pairs"] = bundle(zovolorn, zovolorn.config(z["vocab"], z["width"], [zpar] * z["layers"], taps=4))
     return out
 

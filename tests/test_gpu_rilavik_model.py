@@ -1,0 +1,626 @@
+"""Rilavik through the engine (HipModel: states, batched steps, prefill / decode, sampling, the generate loops) against the float64 oracle on small models of the tests'
+own making: odd sizes, both layer types in several orders, with and without experts, windows of one position up to longer than the prompt, one to seven taps (equal and
+unequal in the two halves), one and several groups, norm parts, heads and winners, temperatures of one and more."""
+
+import dataclasses
+
+import numpy as np
+import pytest
+
+import rilavik_oracle as O
+from uzu_amd import loader
+from uzu_amd.engine import MODEL_BATCH, MODEL_DEBUG_TAPS, MODEL_FULL_F32, HipModel
+
+pytestmark = pytest.mark.gpu
+
+TOL = {True: 4e-5, False: 6e-2}  # full f32 / bf16 products: rms logit error relative to the rms of the logits
+
+
+def rows_ok(err, full, tol=None):
+    """True f32: every row inside the tolerance.  bf16 products: the rounding noise of a narrow stream grows through the layers and a router's near tie may tip: nine rows in
+    ten must be inside and the median well inside.  (What tips early in a stack is carried on by the recurrences behind it: the models of the bf16 tests choose among
+    experts in their last layer only and use all of them in front.)"""
+    err, tol = np.asarray(err), TOL[full] if tol is None else tol
+    return bool(err.max() < tol) if full else bool(np.median(err) < tol / 2 and np.mean(err < tol) >= 0.9)
+
+
+def cfg_a():  # odd sizes: nothing is a multiple of 8, so every kernel runs its general form
+    return O.config(vocab=61, width=36, eps=1e-5, layers=[
+        O.parallel_layer(O.left_half(3, 1, 10, 6, 7, conv=3, rot_dims=4, base=5000.0, factor=3.0, scale=0.4), O.right_half(3, 5, 7, groups=1, norm_groups=3, conv=2), 0.6, 0.9, mlp=O.moe(2, 2, 20)),
+        O.gla_layer(2, 9, 11, tau=1.0, rank=3, mlp=None),
+        O.parallel_layer(O.left_half(4, 2, 6, 10, 40, conv=2, base=100.0), O.right_half(4, 3, 6, groups=2, norm_groups=1, conv=5), 1.1, 0.5, mlp=None),
+        O.gla_layer(1, 6, 5, tau=16.0, rank=2, mlp=O.moe(3, 1, 28)),
+    ])
+
+
+def cfg_b():  # matrix-core friendly sizes; linear attention first; windows on and beside key-block borders
+    return O.config(vocab=97, width=64, layers=[
+        O.gla_layer(2, 32, 48, tau=8.0, rank=8, mlp=O.moe(3, 3, 32)),
+        O.parallel_layer(O.left_half(4, 2, 16, 32, 32, conv=4, rot_dims=8, base=500000.0, factor=8.0, scale=0.25), O.right_half(4, 16, 16, groups=2, norm_groups=2, conv=4), 0.7, 1.2, mlp=O.moe(2, 2, 48)),
+        O.parallel_layer(O.left_half(2, 2, 24, 16, 70, conv=3), O.right_half(2, 64, 32, groups=1, norm_groups=4, conv=4), mlp=None),
+        O.gla_layer(4, 16, 16, tau=16.0, rank=4, mlp=O.moe(8, 2, 32)),
+    ])
+
+
+@pytest.fixture(scope="module")
+def models(hip_ctx, tmp_path_factory):
+    out = {}
+    for name, cfg, seed in (("a", cfg_a(), 11), ("b", cfg_b(), 12)):
+        W = O.weights(cfg, seed)
+        path = str(tmp_path_factory.mktemp("rilavik") / name)
+        O.write_model_dir(path, cfg, W)
+        bundle = loader.load_model_dir(path, max_context_length=512)
+        W64 = {k: v.astype(np.float64) for k, v in W.items()}
+        out[name] = (cfg, W64, {full: HipModel(hip_ctx, bundle, MODEL_BATCH(6) | MODEL_DEBUG_TAPS | (MODEL_FULL_F32 if full else 0)) for full in (True, False)})
+    yield out
+    for _, _, ms in out.values():
+        for m in ms.values():
+            m.close()
+
+
+def prompt(cfg, n, seed):
+    return [int(t) for t in np.random.default_rng(seed).integers(0, cfg["vocab"], size=n)]
+
+
+def make(hip_ctx, tmp_path, cfg, seed, flags=MODEL_FULL_F32, ctx_len=256, edit=None, name="m"):
+    W = O.weights(cfg, seed)
+    if edit:
+        edit(W)
+    O.write_model_dir(str(tmp_path / name), cfg, W)
+    W64 = {k: v.astype(np.float64) for k, v in W.items()}
+    return W64, HipModel(hip_ctx, loader.load_model_dir(str(tmp_path / name), max_context_length=ctx_len), MODEL_BATCH(2) | MODEL_DEBUG_TAPS | flags)
+
+
+def in_portions(m, toks, cuts):
+    """logits of every position, the prompt cut into portions"""
+    assert sum(cuts) == len(toks)
+    st, rows, at = m.new_state(), [], 0
+    for n in cuts:
+        rows.append(m.step_batch([st], [toks[at:at + n]], [list(range(n))])[0])
+        at += n
+    assert st.context_length == len(toks)
+    st.close()
+    return np.concatenate(rows)
+
+
+@pytest.mark.parametrize("name", ["a", "b"])
+@pytest.mark.parametrize("full", [True, False])
+def test_whole_prompt_every_position_and_every_layer(models, name, full):
+    cfg, W, ms = models[name]
+    m = ms[full]
+    toks = prompt(cfg, 150, 1)  # positions on both sides of the windows' edges, of the recurrences' 16-row blocks and 64-row chunks and of the attention kernels' key blocks
+    want, streams = O.forward(cfg, W, toks)
+    st = m.new_state()
+    got, _ = m.step_batch([st], [toks], [list(range(len(toks)))])
+    for l, ref in enumerate(streams):  # the residual stream behind every layer: names the first layer that differs
+        err = np.abs(m.read_layer_output_f32(l) - ref).max(-1) / np.abs(ref).max()
+        assert rows_ok(err, full, 2e-5 if full else 5e-2), (l, err.max(), np.median(err))
+    assert rows_ok(O.logit_error(got, want), full)
+    st.close()
+
+
+def one_layer(layer, vocab=53, width=40, **kw):
+    return O.config(vocab=vocab, width=width, layers=[layer], **kw)
+
+
+LEFT = dict(heads=2, kv_heads=1, dim=8, vdim=8, window=9, conv=3)
+RIGHT = dict(heads=2, vdim=8, state=8, groups=1, norm_groups=1, conv=4)
+left = lambda mlp=None, **kw: one_layer(O.parallel_layer(O.left_half(**{**LEFT, **kw}), O.right_half(**RIGHT), 1.0, 0.0, mlp=mlp))    # the state-space half takes no part
+right = lambda mlp=None, **kw: one_layer(O.parallel_layer(O.left_half(**LEFT), O.right_half(**{**RIGHT, **kw}), 0.0, 1.0, mlp=mlp))  # the attention half takes no part
+both = lambda lk=None, rk=None, ls=0.7, rs=1.2, mlp=None: one_layer(O.parallel_layer(O.left_half(**{**LEFT, **(lk or {})}), O.right_half(**{**RIGHT, **(rk or {})}), ls, rs, mlp=mlp))
+gla = lambda heads=2, dim=8, vdim=8, tau=16.0, rank=3, mlp=None, **kw: one_layer(O.gla_layer(heads, dim, vdim, tau, rank, mlp), **kw)
+MECHANISMS = {
+    "attention_grouped": left(heads=6, kv_heads=3, dim=12, vdim=20, scale=0.9),
+    "attention_as_many_kv_heads": left(heads=3, kv_heads=3, dim=16, vdim=4),
+    "attention_one_head": left(heads=1, kv_heads=1, dim=6, vdim=70),
+    "attention_wide_values": left(heads=2, kv_heads=1, dim=16, vdim=136),
+    "attention_wide_keys": left(heads=2, kv_heads=1, dim=160, vdim=24),
+    "attention_beyond_a_workgroup": left(heads=2, kv_heads=1, dim=300, vdim=12, rot_dims=280),
+    "partial_rotation": left(dim=12, rot_dims=4, base=50.0),
+    "scaled_rotation": left(dim=16, rot_dims=16, base=1000.0, factor=5.5),
+    "scaling_by_one": left(dim=8, factor=1.0),
+    "two_rotated_coordinates": left(dim=10, rot_dims=2, base=10.0),
+    "window_of_one": left(window=1),
+    "window_of_two": left(window=2),
+    "window_longer_than_the_prompt": left(window=500),
+    "one_tap": left(conv=1),
+    "two_taps": left(conv=2),
+    "five_taps": left(conv=5),
+    "seven_taps": left(conv=7),
+    "state_space_alone": right(),
+    "state_space_odd": right(heads=3, vdim=7, state=5, groups=3, norm_groups=7, conv=3),
+    "state_space_grouped": right(heads=6, vdim=4, state=12, groups=2, norm_groups=3),
+    "state_space_one_head": right(heads=1, vdim=40, state=16, norm_groups=5),
+    "state_space_wide_state": right(heads=2, vdim=8, state=130, conv=2),
+    "state_space_wide_values": right(heads=1, vdim=150, state=8),
+    "state_space_one_state_row": right(state=1),
+    "state_space_one_tap": right(conv=1),
+    "state_space_six_taps": right(conv=6),
+    "every_coordinate_its_own_norm_part": one_layer(O.parallel_layer(O.left_half(**LEFT), O.right_half(**{**RIGHT, "norm_groups": 16}), 0.0, 1.0), eps=0.25),
+    "both_halves": both(),
+    "both_halves_equal_taps": both(dict(conv=4), dict(conv=4)),
+    "both_halves_more_taps_on_the_left": both(dict(conv=4), dict(conv=2)),
+    "both_halves_negative_scale": both(ls=-0.7, rs=0.3),
+    "both_halves_with_experts": both(mlp=O.moe(4, 1, 24)),
+    "linear_attention": gla(),
+    "linear_attention_temperature_of_one": gla(tau=1.0),
+    "linear_attention_fast": gla(tau=0.25),
+    "linear_attention_one_head": gla(heads=1, dim=20, vdim=12),
+    "linear_attention_odd": gla(heads=3, dim=7, vdim=5, rank=1),
+    "linear_attention_wide": gla(heads=2, dim=130, vdim=70, rank=9),
+    "linear_attention_of_256": gla(heads=1, dim=256, vdim=256, rank=16),
+    "experts_one_of_one": gla(mlp=O.moe(1, 1, 24)),
+    "experts_all_of_them": gla(mlp=O.moe(3, 3, 16)),
+    "experts_one_of_many": gla(mlp=O.moe(70, 1, 12)),
+    "experts_four_of_nine_odd": gla(mlp=O.moe(9, 4, 13)),
+    "large_epsilon": gla(mlp=O.moe(4, 2, 16), eps=0.3),
+}
+
+
+@pytest.mark.parametrize("full", [True, False])
+@pytest.mark.parametrize("which", sorted(MECHANISMS))
+def test_each_mechanism_alone_in_a_one_layer_model(hip_ctx, tmp_path, which, full):
+    cfg = MECHANISMS[which]
+    W, m = make(hip_ctx, tmp_path, cfg, 5, flags=MODEL_FULL_F32 if full else 0)
+    toks = prompt(cfg, 90, 3)
+    want, streams = O.forward(cfg, W, toks)
+    st = m.new_state()
+    got, _ = m.step_batch([st], [toks], [list(range(len(toks)))])
+    if full:
+        assert np.abs(m.read_layer_output_f32(0) - streams[0]).max() < 2e-5 * np.abs(streams[0]).max()
+    assert rows_ok(O.logit_error(got, want), full)
+    st.reset()  # and token by token from a reused state: the decode forms of the same kernels
+    rows = [m.step_batch([st], [[t]], [[0]])[0][0] for t in toks[:40]]
+    assert rows_ok(O.logit_error(np.stack(rows), want[:40]), full)
+    st.close()
+    m.close()
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_heads_of_128_in_both_precisions(hip_ctx, tmp_path, full):
+    """Head widths of real models: the serving precision runs the attention on the matrix cores over bf16 caches and the experts in buckets; prompt rows, a portion across the
+    window's edge and decoded tokens against the oracle."""
+    cfg = O.config(vocab=97, width=64, layers=[
+        O.parallel_layer(O.left_half(2, 1, 128, 128, 48, conv=4, base=5e5, factor=4.0, scale=0.09), O.right_half(2, 64, 128, groups=1, norm_groups=2), 0.7, 1.2, mlp=O.moe(2, 2, 32)),
+        O.gla_layer(2, 128, 128, rank=16, mlp=O.moe(4, 1, 32))])
+    W, m = make(hip_ctx, tmp_path, cfg, 13, flags=MODEL_FULL_F32 if full else 0)
+    toks = prompt(cfg, 170, 4)
+    want, _ = O.forward(cfg, W, toks)
+    assert rows_ok(O.logit_error(in_portions(m, toks, [120, 30] + [1] * 20), want), full)
+    m.close()
+
+
+@pytest.mark.parametrize("name", ["a", "b"])
+@pytest.mark.parametrize("full", [True, False])
+def test_prefill_then_token_by_token_and_portions_down_to_two_tokens(models, name, full):
+    cfg, W, ms = models[name]
+    m = ms[full]
+    toks = prompt(cfg, 120, 2)
+    want, _ = O.forward(cfg, W, toks)
+    for cuts in ([100] + [1] * 20, [1] * 30 + [90], [2, 3, 2, 50, 7, 2, 54], [33, 31, 17, 39], [64, 1, 55], [2] * 5 + [110], [7, 7, 2, 16, 32, 56]):
+        assert rows_ok(O.logit_error(in_portions(m, toks, cuts), want), full), cuts
+
+
+@pytest.mark.parametrize("name", ["a", "b"])
+def test_unequal_batch_equals_each_request_alone_and_reused_states(models, name):
+    cfg, W, ms = models[name]
+    m = ms[True]
+    reqs = [prompt(cfg, n, 10 + n) for n in (1, 37, 90, 5, 64)]
+    alone = []
+    for r in reqs:
+        st = m.new_state()
+        first, _ = m.step_batch([st], [r[:-3]] if len(r) > 3 else [r], [[len(r) - 4] if len(r) > 3 else [0]])
+        tail = [m.step_batch([st], [[t]], [[0]])[0] for t in (r[-3:] if len(r) > 3 else [])]
+        alone.append(np.concatenate([first] + tail))
+        st.close()
+    pool = [m.new_state() for _ in reqs]
+    for turn in range(2):  # the second turn reuses the states the first one gave back (reset), in another order: caches, recurrent states and windows of other requests
+        states = pool if turn == 0 else pool[::-1]
+        heads = [r[:-3] if len(r) > 3 else r for r in reqs]
+        lg, _ = m.step_batch(states, heads, [[len(h) - 1] for h in heads])
+        got = [[lg[i]] for i in range(len(reqs))]
+        for step in range(3):  # decoded together; the one-token request has left the batch
+            live = [i for i, r in enumerate(reqs) if len(r) > 3]
+            lg, _ = m.step_batch([states[i] for i in live], [[reqs[i][len(reqs[i]) - 3 + step]] for i in live], [[0]] * len(live))
+            for row, i in zip(lg, live):
+                got[i].append(row)
+        for i in range(len(reqs)):
+            assert np.abs(np.stack(got[i]) - alone[i]).max() < 2e-4 * np.abs(alone[i]).max(), (turn, i)
+            assert O.logit_error(np.stack(got[i])[-1:], O.forward(cfg, W, reqs[i])[0][-1:]).max() < TOL[True]
+        for st in states:
+            st.reset()
+    for st in pool:
+        st.close()
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_a_decoding_request_a_continued_one_and_a_prompt_in_one_pass(models, full):
+    cfg, W, ms = models["b"]
+    m = ms[full]
+    a, b, c = prompt(cfg, 81, 21), prompt(cfg, 110, 22), prompt(cfg, 70, 23)
+    sa, sb, sc = (m.new_state() for _ in range(3))
+    m.step_batch([sa, sb], [a[:80], b[:41]], [[], []])
+    lg, _ = m.step_batch([sc, sa, sb], [c, a[80:], b[41:]], [[69], [0], [68]])
+    want = np.stack([O.forward(cfg, W, t)[0][-1] for t in (c, a, b)])
+    assert O.logit_error(lg, want).max() < (TOL[True] if full else 0.2)
+    for st in (sa, sb, sc):
+        st.close()
+
+
+def test_more_requests_than_a_pass_carries_and_prompts_longer_than_a_pass(hip_ctx, tmp_path):
+    cfg = O.config(vocab=31, width=16, layers=[
+        O.parallel_layer(O.left_half(2, 1, 8, 8, 48, conv=3), O.right_half(2, 8, 4, norm_groups=2), mlp=None),
+        O.gla_layer(2, 4, 8, rank=2, mlp=O.moe(3, 1, 8))])
+    W, m = make(hip_ctx, tmp_path, cfg, 21, ctx_len=3000)
+    reqs = [prompt(cfg, n, n) for n in (9, 2100, 4, 30, 2)]  # 2100 > one pass of 2048 rows; five requests > two per pass
+    states = [m.new_state() for _ in reqs]
+    lg, sampled = m.step_batch(states, reqs, [[len(r) - 1] for r in reqs], sample=True)
+    for i, r in enumerate(reqs):
+        want = O.forward(cfg, W, r)[0][-1:]
+        assert O.logit_error(lg[i:i + 1], want).max() < (TOL[True] if len(r) < 200 else 2e-4), i
+        assert len(r) > 200 or int(sampled[i]) == int(np.argmax(want))
+        assert states[i].context_length == len(r)
+    st = m.new_state()  # the long prompt: against the same prompt through two explicit portions
+    m.step_batch([st], [reqs[1][:1500]], [[]])
+    two, _ = m.step_batch([st], [reqs[1][1500:]], [[599]])
+    assert np.abs(two[0] - lg[1]).max() < 2e-4 * np.abs(two).max()
+    m.close()
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_long_decoding(models, full):
+    cfg, W, ms = models["b"]
+    m = ms[full]
+    toks = prompt(cfg, 230, 5)
+    want, _ = O.forward(cfg, W, toks)
+    st = m.new_state()
+    m.step_batch([st], [toks[:10]], [[]])
+    rows = [m.step_batch([st], [[t]], [[0]])[0][0] for t in toks[10:]]  # 220 decoded tokens: the windows pass over decoded tokens several times
+    assert rows_ok(O.logit_error(np.stack(rows), want[10:]), full)
+    st.close()
+
+
+def look_alike(W, dim):
+    """the left half's keys become the rows of its first query head, so that a token's query points at the keys of its own token; two taps: queries and keys are (nearly) the
+    current position's, values the previous one's -- two places of one token carry different values"""
+    W["l0.mix.left.k"] = W["l0.mix.left.q"][:dim].copy()
+    for n, taps in (("q", (0.02, 1.0)), ("k", (0.02, 1.0)), ("v", (1.0, 0.02))):
+        W[f"l0.mix.left.{n}.conv"] = O.to_bf16(np.tile(np.array([taps]), (W[f"l0.mix.left.{n}.conv"].shape[0], 1)))
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_a_far_key_among_hundreds_decides_the_logits(hip_ctx, tmp_path, full):
+    """The last token of a 700-token prompt also stands at position 2 and nowhere else, and queries look for the keys of their own token: that one far key takes a visible
+    share of the softmax.  Replacing it must move the last logits exactly as the oracle says, in a whole prompt and when the tail is decoded token by token -- a key that
+    is dropped, doubled, rotated by a wrong position or read from a neighbouring row shows."""
+    cfg = O.config(vocab=41, width=32, layers=[O.parallel_layer(O.left_half(2, 1, 16, 8, 1000, conv=2, rot_dims=2, base=1e5, factor=4000.0, scale=1.0), O.right_half(**RIGHT), 1.0, 0.0)])
+    W, m = make(hip_ctx, tmp_path, cfg, 8, ctx_len=1024, edit=lambda W: look_alike(W, 16), flags=MODEL_FULL_F32 if full else 0)
+    base = [int(t) for t in np.random.default_rng(4).integers(0, 39, size=700)]  # tokens 39 and 40 are kept for the marked positions
+    base[2] = base[-1] = 39
+    other = list(base)
+    other[2] = 40
+    want = [O.forward(cfg, W, t)[0][-1] for t in (base, other)]
+    assert O.logit_error(want[0][None], want[1][None]).max() > 0.05, "the oracle itself does not see the token"
+    for toks, ref in zip((base, other), want):
+        st = m.new_state()
+        whole, _ = m.step_batch([st], [toks], [[699]])
+        st.reset()
+        m.step_batch([st], [toks[:640]], [[]])
+        for t in toks[640:-1]:
+            m.step_batch([st], [[t]], [[]])
+        dec, _ = m.step_batch([st], [[toks[-1]]], [[0]])
+        tol = TOL[True] if full else 0.03
+        assert O.logit_error(whole, ref[None]).max() < tol and O.logit_error(dec, ref[None]).max() < tol
+        st.close()
+    m.close()
+
+
+@pytest.mark.parametrize("window", [1, 5, 32, 33, 64, 130])
+def test_keys_just_inside_and_just_outside_a_window(hip_ctx, tmp_path, window):
+    """Token 40 stands at one place; `window - 1` positions later it is the last key a query sees, one more and it is gone.  Queries look for their own token's keys, and the
+    row at either distance IS token 40: with the key in sight it takes a visible share.  Whole prompts, cuts around the edge and decoded tokens are held to the oracle,
+    which itself tells a window that is one off."""
+    n, at = 3 * window + 8, window + 2
+    cfg = O.config(vocab=41, width=32, layers=[O.parallel_layer(O.left_half(2, 1, 16, 8, window, conv=2, rot_dims=2, base=1e5, factor=4000.0, scale=1.0), O.right_half(**RIGHT), 1.0, 0.0)])
+    W, m = make(hip_ctx, tmp_path, cfg, 8, ctx_len=512, edit=lambda W: look_alike(W, 16))
+    for inside in (True, False):
+        toks = prompt(dict(vocab=39), n, 6)
+        row = at + window - (1 if inside else 0)
+        toks[at] = toks[row] = 40
+        want, _ = O.forward(cfg, W, toks)
+        if window > 1:
+            off = [O.forward(dict(cfg, layers=[O.parallel_layer(dict(cfg["layers"][0]["mixer"]["left"], mask={"size": w}), cfg["layers"][0]["mixer"]["right"], 1.0, 0.0)]), W, toks)[0][row]
+                   for w in (window - 1, window + 1)]
+            assert O.logit_error(off[0 if inside else 1][None], want[row][None]).max() > 0.01, "the oracle itself does not tell the window's edge"
+        for cuts in ([n], [row, n - row], [row - 1, 2, n - row - 1], [at + 1] + [1] * (n - at - 1), [at, 2, n - at - 2]):
+            assert O.logit_error(in_portions(m, toks, cuts), want).max() < TOL[True], (inside, cuts)
+    m.close()
+
+
+def test_taps_that_grow_with_the_distance_at_every_cut(hip_ctx, tmp_path):
+    """Convolutions whose oldest tap is the largest, four taps on the left and three on the right: every cut of the prompt puts the carried windows to use at a different place."""
+    cfg = O.config(vocab=41, width=32, layers=[O.parallel_layer(O.left_half(2, 1, 8, 8, 20, conv=4), O.right_half(2, 8, 8, conv=3), 0.7, 1.2)])
+
+    def edit(W):
+        for n in ("left.q.conv", "left.k.conv", "left.v.conv", "right.conv"):
+            w = W["l0.mix." + n]
+            W["l0.mix." + n] = O.to_bf16(np.sign(w) * (0.3 + np.arange(w.shape[1])[::-1] * 0.5))
+    W, m = make(hip_ctx, tmp_path, cfg, 9, edit=edit)
+    toks = prompt(cfg, 24, 7)
+    want, _ = O.forward(cfg, W, toks)
+    for k in range(1, 24):
+        assert O.logit_error(in_portions(m, toks, [k, 24 - k]), want).max() < TOL[True], k
+    for cuts in ([1] * 24, [2] * 12, [3] * 8, [1, 2] * 8, [20, 1, 1, 1, 1]):
+        assert O.logit_error(in_portions(m, toks, cuts), want).max() < TOL[True], cuts
+    m.close()
+
+
+@pytest.mark.parametrize("kind", ["gla", "state_space"])
+def test_a_far_token_reaches_the_logits_only_through_the_state(hip_ctx, tmp_path, kind):
+    """What position 3 leaves at position 300 travels in the recurrent state alone (slow decays, a window of 8 positions), through a prompt, through portions and through
+    decoded tokens."""
+    if kind == "gla":
+        cfg = O.config(vocab=41, width=32, layers=[O.gla_layer(2, 16, 16, rank=2), O.gla_layer(3, 8, 12, tau=4.0, rank=2, mlp=O.moe(3, 1, 16))])
+    else:
+        pair = lambda *r, **k: O.parallel_layer(O.left_half(2, 1, 8, 8, 8, conv=2), O.right_half(*r, **k), 0.3, 1.0)
+        cfg = O.config(vocab=41, width=32, layers=[pair(2, 16, 16, conv=2), pair(3, 8, 12, groups=3, conv=3)])
+
+    def slow(W):
+        for i in (0, 1):
+            if kind == "gla":
+                W[f"l{i}.mix.a2.b"] = O.to_bf16(np.full_like(W[f"l{i}.mix.a2.b"], 9.0))
+            else:
+                W[f"l{i}.mix.right.A_log"] = O.to_bf16(np.full_like(W[f"l{i}.mix.right.A_log"], -7.0))
+    W, m = make(hip_ctx, tmp_path, cfg, 8, ctx_len=512, edit=slow)
+    base = prompt(cfg, 301, 4)
+    other = list(base)
+    other[3] = (base[3] + 7) % cfg["vocab"]
+    want = [O.forward(cfg, W, t)[0][-1] for t in (base, other)]
+    assert O.logit_error(want[0][None], want[1][None]).max() > 1e-3, "the oracle itself does not carry the token: slow the decays"
+    for toks, ref in zip((base, other), want):
+        st = m.new_state()
+        whole, _ = m.step_batch([st], [toks], [[300]])
+        st.reset()
+        m.step_batch([st], [toks[:100]], [[]])
+        m.step_batch([st], [toks[100:102]], [[]])
+        for t in toks[102:-1]:
+            m.step_batch([st], [[t]], [[]])
+        dec, _ = m.step_batch([st], [[toks[-1]]], [[0]])
+        assert O.logit_error(whole, ref[None]).max() < TOL[True] and O.logit_error(dec, ref[None]).max() < TOL[True]
+        st.close()
+    m.close()
+
+
+def test_the_score_multiplies_the_experts_input(hip_ctx, tmp_path):
+    """silu is not linear: scores on the input give another result than on the output -- in the bucketed prompt form and in the decode form"""
+    cfg = O.config(vocab=41, width=64, layers=[O.gla_layer(1, 8, 8, rank=2, mlp=O.moe(4, 4, 32))])
+
+    def edit(W):
+        W["l0.mlp.router"] = O.to_bf16(W["l0.mlp.router"] * 1.5)  # scores from a tenth to nine tenths
+        W["l0.ls2"] = O.to_bf16(W["l0.ls2"] * 3.0)
+    W, m = make(hip_ctx, tmp_path, cfg, 3, flags=0, edit=edit)
+    toks = prompt(cfg, 100, 2)
+    want, _ = O.forward(cfg, W, toks)
+
+    def on_output(h, w, p, ml):
+        s = O.sigmoid(h @ w[p + "router"].T)
+        return sum(s[:, e:e + 1] * ((O.silu(h @ w[f"{p}e{e}.gate"].T) * (h @ w[f"{p}e{e}.up"].T)) @ w[f"{p}e{e}.down"].T) for e in range(4))
+    keep = O.moe_mlp
+    try:
+        O.moe_mlp = on_output
+        wrong, _ = O.forward(cfg, W, toks)
+    finally:
+        O.moe_mlp = keep
+    assert np.median(O.logit_error(wrong, want)) > 0.15
+    assert rows_ok(O.logit_error(in_portions(m, toks, [80] + [1] * 20), want), False, 0.03)
+    m.close()
+
+
+def test_the_first_tokens_and_a_state_that_held_another_request(models):
+    """Positions 0, 1, 2 of a sequence: zeros in front of every convolution, zero states, one-key softmaxes -- also on a state that another, longer request has just left
+    (reset): nothing of it may be read."""
+    cfg, W, ms = models["a"]
+    m = ms[True]
+    st = m.new_state()
+    m.step_batch([st], [prompt(cfg, 80, 9)], [[]])
+    for n, seed in ((1, 1), (2, 2), (3, 3), (20, 4)):
+        st.reset()
+        toks = prompt(cfg, n, seed)
+        got, _ = m.step_batch([st], [toks], [list(range(n))])
+        assert O.logit_error(got, O.forward(cfg, W, toks)[0]).max() < TOL[True]
+    st.reset()
+    toks = prompt(cfg, 6, 7)
+    rows = [m.step_batch([st], [[t]], [[0]])[0][0] for t in toks]
+    assert O.logit_error(np.stack(rows), O.forward(cfg, W, toks)[0]).max() < TOL[True]
+    st.close()
+
+
+@pytest.mark.parametrize("name", ["a", "b"])
+def test_greedy_generation_through_prefill_and_decode(models, name):
+    """The engine's own entry points: HipModel.prefill + chained decode (the sampled token is fed back on the device), then the stochastic sampler's plumbing."""
+    cfg, W, ms = models[name]
+    m = ms[True]
+    p = prompt(cfg, 25, 7)
+    m.reset()
+    m.set_sampling(None)
+    first = m.prefill(np.asarray(p, dtype=np.uint32))
+    rest, _ = m.decode(9)
+    got = [int(first)] + [int(t) for t in rest]
+    want, margin_ok = [], True
+    toks = list(p)
+    for _ in range(10):
+        row = O.forward(cfg, W, toks)[0][-1]
+        top2 = np.sort(row)[-2:]
+        margin_ok = margin_ok and (top2[1] - top2[0]) > 1e-3 * np.abs(row).max()
+        want.append(int(np.argmax(row)))
+        toks.append(want[-1])
+    assert margin_ok, "the oracle's own greedy stream has a near tie: pick another seed"
+    assert got == want and m.context_length == len(p) + 9
+    assert np.argmax(m.read_logits_f32()) == want[-1]
+    m.reset()
+    m.set_sampling(seed=3, temperature=1e-4)  # temperature -> 0 of the stochastic sampler is greedy
+    s1 = [int(m.prefill(np.asarray(p, dtype=np.uint32)))] + [int(t) for t in m.decode(4)[0]]
+    assert s1 == want[:5]
+    m.set_sampling(None)
+    m.reset()
+
+
+def test_generate_loop_of_the_text_front_end_and_the_pool(hip_ctx, tmp_path):
+    """LanguageModel.generate on a directory without tokenizer.json, and SequencePool.generate: prompts of unequal length prefilled in one batch and decoded together,
+    requests leaving as they finish (one by a stop token), their states reused by a second call -- against each prompt generated alone by the oracle"""
+    from uzu_amd.language_model import LanguageModel
+    from uzu_amd.serving import SequencePool
+    cfg = cfg_a()
+    W = O.weights(cfg, 31)
+    W["head"] = O.to_bf16(W["head"] * 3.0)  # wider margins between the logits
+    O.write_model_dir(str(tmp_path / "g"), cfg, W)
+    W64 = {k: v.astype(np.float64) for k, v in W.items()}
+    lm = LanguageModel(hip_ctx, str(tmp_path / "g"), max_context_length=128, flags=MODEL_FULL_F32, tokenizer_required=False)
+    p = prompt(cfg, 12, 3)
+    res = lm.generate(p, max_tokens=11, chunk=4)
+    assert res.token_ids == O.greedy(cfg, W64, p, 11) and res.prompt_tokens == 12
+    lm.close()
+    m = HipModel(hip_ctx, loader.load_model_dir(str(tmp_path / "g"), max_context_length=128), MODEL_BATCH(4) | MODEL_FULL_F32)
+    prompts = {"x": prompt(cfg, 3, 41), "y": prompt(cfg, 40, 42), "z": prompt(cfg, 17, 43)}
+    want = {k: O.greedy(cfg, W64, q, 8) for k, q in prompts.items()}
+    stop = want["y"][4]
+    cut = lambda seq: seq[:seq.index(stop)] if stop in seq else seq
+    pool = SequencePool(m)
+    for _ in range(2):
+        got = pool.generate(prompts, max_tokens=8, stop_token_ids=[stop])
+        assert got == {k: cut(v) for k, v in want.items()}
+        assert not pool.live and len(pool.free) == 3
+    pool.close()
+    m.close()
+
+
+@pytest.mark.parametrize("full", [True, False])
+def test_decode_graph_replays_equal_plain_launches(hip_ctx, tmp_path, full):
+    """The chained decode step is ONE captured hipGraph per state that reads its position from device memory.  Replayed in several calls, with eager batched steps of OTHER
+    states (which overwrite the model's pass tables) and synchronisations between them, every token and the logits after every call must equal those of a model that
+    decodes with plain launches."""
+    from uzu_amd.engine import MODEL_NO_GRAPH
+    cfg = cfg_b()
+    W = O.weights(cfg, 77)
+    O.write_model_dir(str(tmp_path / "m"), cfg, W)
+    bundle = loader.load_model_dir(str(tmp_path / "m"), max_context_length=256)
+    base = MODEL_BATCH(4) | (MODEL_FULL_F32 if full else 0)
+    graph, plain = HipModel(hip_ctx, bundle, base), HipModel(hip_ctx, bundle, base | MODEL_NO_GRAPH)
+    p, other = prompt(cfg, 70, 8), prompt(cfg, 33, 9)
+    firsts = [m.prefill(np.asarray(p, dtype=np.uint32)) for m in (graph, plain)]
+    assert firsts[0] == firsts[1]
+    side = [m.new_state() for m in (graph, plain)]
+    for call in range(4):
+        toks = [m.decode(5)[0] for m in (graph, plain)]
+        assert list(toks[0]) == list(toks[1]), call
+        assert np.array_equal(graph.read_logits_f32(), plain.read_logits_f32()), call
+        for m, st in zip((graph, plain), side):  # eager work on another state between the replays
+            m.step_batch([st], [other[call * 8:(call + 1) * 8]], [[7]])
+    assert graph.context_length == 70 + 20
+    for m in (graph, plain):
+        m.close()
+
+
+def test_copied_states_go_their_own_ways(models):
+    cfg, W, ms = models["a"]
+    m = ms[True]
+    toks = prompt(cfg, 60, 6)
+    a, b = m.new_state(), m.new_state()
+    m.step_batch([a], [toks[:50]], [[]])
+    b.copy_from(a)
+    m.step_batch([a], [prompt(cfg, 5, 8)], [[]])
+    got, _ = m.step_batch([b], [toks[50:]], [list(range(10))])
+    assert O.logit_error(got, O.forward(cfg, W, toks)[0][50:]).max() < TOL[True]
+    a.close(), b.close()
+
+
+def test_the_mechanisms_in_other_company(hip_ctx, tmp_path):
+    """The mechanisms are options of the engine, not of this design: convolved attention without a second mixer (with and without head norms behind the convolution), held
+    to the oracle's functions."""
+    cfg = O.config(vocab=41, width=32, layers=[O.parallel_layer(O.left_half(4, 2, 8, 16, 12, conv=3, scale=0.6), O.right_half(**RIGHT), 1.0, 0.0)])
+    W = O.weights(cfg, 4)
+    O.write_model_dir(str(tmp_path / "m"), cfg, W)
+    bundle = loader.load_model_dir(str(tmp_path / "m"), max_context_length=128)
+    W64 = {k: v.astype(np.float64) for k, v in W.items()}
+    single = dataclasses.replace(bundle, layers=[dataclasses.replace(bundle.layers[0], pair_mixer=None)])
+    toks = prompt(cfg, 70, 5)
+    want, _ = O.forward(cfg, W64, toks)
+    m = HipModel(hip_ctx, single, MODEL_FULL_F32)
+    assert O.logit_error(in_portions(m, toks, [50, 2] + [1] * 18), want).max() < TOL[True]
+    m.close()
+    ones = lambda n: type(bundle.output_norm)(present=True, epsilon=1e-5, scales=np.full(n, 1.3, dtype=np.float32))
+    normed = dataclasses.replace(single, layers=[dataclasses.replace(single.layers[0], query_norm=ones(8), key_norm=ones(8))])
+    keep = O.rotate_half
+    try:
+        O.rotate_half = lambda a, *r, **k: keep(O.rms_norm(a, 1.3, 1e-5), *r, **k)
+        want, _ = O.forward(cfg, W64, toks)
+    finally:
+        O.rotate_half = keep
+    m = HipModel(hip_ctx, normed, MODEL_FULL_F32)
+    assert O.logit_error(in_portions(m, toks, [50, 2] + [1] * 18), want).max() < TOL[True]
+    m.close()
+
+
+def test_refusals_of_the_engine(hip_ctx, tmp_path):
+    """what the engine does not run it refuses at creation, by name"""
+    from uzu_amd import _ffi, desc as D
+    cfg = cfg_b()
+    O.write_model_dir(str(tmp_path / "m"), cfg, O.weights(cfg, 3))
+    bundle = loader.load_model_dir(str(tmp_path / "m"), max_context_length=64)
+    g, p = bundle.layers[0], bundle.layers[1]
+    absent = type(p.post_mixer_norm)(present=False)
+    changed = lambda i, **kw: dataclasses.replace(bundle, layers=bundle.layers[:i] + [dataclasses.replace(bundle.layers[i], **kw)] + bundle.layers[i + 1:])
+    for broken, why in ((changed(1, post_mixer_norm=absent, layer_scale_mixer=None), "joins the stream behind a post-mixer norm"), (changed(1, ssd_norm_groups=3), "equal parts"),
+                        (changed(1, ssd_skip=None), "skip and norm"), (changed(1, pair_mixer=D.MIXER_RETENTION), "second mixer of a pair"), (changed(1, has_gate=True), "head gates"),
+                        (changed(1, kv_source_layer_index=0), "convolved queries on another layer's cache"), (changed(0, decay_temperature=0.0), "temperature"),
+                        (changed(0, sliding_window_size=4), "attention options on gated linear attention"), (changed(0, qkv_conv=p.qkv_conv), "options of attention"),
+                        (changed(0, moe=dataclasses.replace(g.moe, plain_experts=True)), "weights on the inputs"),
+                        (changed(0, moe=dataclasses.replace(g.moe, routing=D.MOE_ROUTE_TOPK_LOGITS)), "raw scores"), (dataclasses.replace(bundle, f32_stream=False), "")):
+        with pytest.raises(_ffi.UzuHipError, match=why):
+            HipModel(hip_ctx, broken, MODEL_FULL_F32 if broken.f32_stream else 0)
+
+
+def random_config(seed):
+    """a configuration drawn at random: sizes, head counts, layer order, constants"""
+    rng = np.random.default_rng(seed)
+    pick = lambda *xs: xs[int(rng.integers(len(xs)))]
+    width = pick(24, 40, 64, 96, 120)
+    layers = []
+    count = int(rng.integers(2, 6))
+    for i in range(count):
+        E = pick(1, 2, 5, 8, 12) if i == count - 1 else pick(1, 2, 3)
+        mlp = pick(None, O.moe(E, min(E, pick(1, 1, 2, 3)) if i == count - 1 else E, pick(16, 40, 72)))
+        if pick("gla", "parallel") == "gla":
+            layers.append(O.gla_layer(pick(1, 2, 3, 6), pick(8, 24, 32, 48), pick(8, 16, 40, 72), tau=pick(1.0, 4.0, 16.0, 32.0), rank=pick(1, 4, 16), mlp=mlp))
+        else:
+            G, dim = pick(1, 2, 3), pick(8, 16, 32, 64)
+            Gs, parts, vd = pick(1, 2), pick(1, 2, 4), pick(8, 16, 32, 64)
+            layers.append(O.parallel_layer(
+                O.left_half(G * pick(1, 2, 4), G, dim, pick(8, 16, 24, 128), pick(1, 6, 32, 64, 100, 300), conv=pick(1, 2, 3, 4, 5), rot_dims=pick(2, dim // 2, dim), base=pick(1e3, 1e4, 5e5),
+                            factor=pick(None, 1.0, 4.0, 8.0), scale=pick(0.1, 0.2, 0.35)),
+                O.right_half(Gs * pick(1, 2, 4), vd, pick(4, 16, 32, 80), groups=Gs, norm_groups=parts, conv=pick(1, 2, 3, 4)), pick(0.3, 0.7, 1.0), pick(0.4, 1.2, 1.0), mlp=mlp))
+    return O.config(vocab=pick(50, 257, 640), width=width, layers=layers, eps=pick(1e-6, 1e-5, 1e-3))
+
+
+@pytest.mark.parametrize("seed", range(12))
+def test_configurations_drawn_at_random(hip_ctx, tmp_path, seed):
+    """whole prompt, prompt + decoded tail and an unequal batch on a configuration nobody chose, in both precisions"""
+    cfg = random_config(100 + seed)
+    W = O.weights(cfg, seed)
+    O.write_model_dir(str(tmp_path / "m"), cfg, W)
+    W64 = {k: v.astype(np.float64) for k, v in W.items()}
+    bundle = loader.load_model_dir(str(tmp_path / "m"), max_context_length=400)
+    a, b = prompt(cfg, 170, seed), prompt(cfg, 45, seed + 50)
+    want_a, want_b = O.forward(cfg, W64, a)[0], O.forward(cfg, W64, b)[0]
+    for full in (True, False):
+        m = HipModel(hip_ctx, bundle, MODEL_BATCH(3) | (MODEL_FULL_F32 if full else 0))
+        st, st2 = m.new_state(), m.new_state()
+        whole, _ = m.step_batch([st], [a], [list(range(170))])
+        tail = in_portions(m, a, [130] + [1] * 40)
+        st.reset()
+        both_, _ = m.step_batch([st2, st], [b, a[:100]], [list(range(45)), list(range(100))])
+        for got, want in ((whole, want_a), (tail, want_a), (both_[:45], want_b), (both_[45:], want_a[:100])):
+            err = O.logit_error(got, want)
+            # (a router's near tie may tip in bf16 products: single rows may stand out there)
+            assert (err.max() < 2e-4 and np.median(err) < 1e-5) if full else (np.median(err) < 3e-2 and np.mean(err < 8e-2) >= 0.85), (cfg, full, err.max(), np.median(err))
+        m.close()
